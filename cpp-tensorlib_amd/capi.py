@@ -25,7 +25,7 @@ OPS = dict(add=0, sub=1, mul=2, div=3, pow=4, exp=5, log=6, sqrt=7, sigmoid=8, r
 CENSUS = ["binary", "bcast", "unary", "row_op", "gemm", "gemv_f32", "gemv_bf16", "gemv_bf16_row",
           "gemv_q4", "attn_decode", "rope", "rmsnorm", "rmsnorm_res", "swiglu", "argmax",
           "kv_append", "kv_fill", "split_heads", "merge_heads", "gemm_bf16_nt", "attn_prefill",
-          "convert", "quantize_q4"]
+          "convert", "quantize_q4", "mix_step", "window_attn", "linear_attn", "polynorm", "embed", "residual"]
 
 # name -> (restype, argtypes): exactly the declarations of include/tensorlib_hip.h
 SIGNATURES = {
@@ -124,6 +124,17 @@ SIGNATURES = {
     "tlhip_gemv_bf16_row_rmsnorm": (cint, [P, P, P, P, P, P, i64, i64, f32]),
     "tlhip_gemv_q4_rmsnorm_gateup": (cint, [P, P, P, P, P, P, P, i64, i64, i64, f32]),
     "tlhip_gemv_bf16_row_rmsnorm_gateup": (cint, [P, P, P, P, P, P, i64, i64, f32]),
+    "tlhip_window_ring_ld": (i64, [i64]),
+    "tlhip_linear_state_bytes": (i64, [i64, i64, i64]),
+    "tlhip_mix_partials_bytes": (i64, [P]),
+    "tlhip_mix_step": (cint, [P, P, P, P, P, i64, P, P, i64]),
+    "tlhip_window_fill": (cint, [P, i64, P, i64, i64]),
+    "tlhip_window_attn_chunk": (cint, [P, i64, P, i64, P, i64, i64]),
+    "tlhip_linear_attn_chunk": (cint, [P, i64, P, i64, P, i64, i64]),
+    "tlhip_polynorm_rows": (cint, [P, i64, P, i64, P, i64]),
+    "tlhip_embed_sinusoid": (cint, [P, P, P, i64, i64, i64, i64, i64, P]),
+    "tlhip_residual_sum": (cint, [P, P, i64, P, P, P, i64, i64]),
+    "tlhip_gather_rows": (cint, [P, P, P, i64, i64, i64]),
     "tlhip_tune_gemv_q4": (cint, [cint, cint, cint, cint, cint]),
     "tlhip_tune_gemv_cols": (cint, [cint]),
     "tlhip_tune_attn_prefill": (cint, [cint]),
@@ -136,6 +147,24 @@ SIGNATURES = {
     "tlhip_warm_fork": (cint, [P, P, cint, cint, cint]),
     "tlhip_warm_join": (cint, []),
 }
+
+
+class WindowAttn(C.Structure):
+    """tlhip_window_attn"""
+    _fields_ = [(n, i64) for n in ("heads", "kv_heads", "dim", "window", "q_off", "k_off", "gate_off", "y_off")] + \
+               [("ring", P), ("ring_rows", i64), ("ring_ld", i64)] + \
+               [(n, f32) for n in ("scale", "temp_coef", "temp_every", "slope_exp", "out_scale")]
+
+
+class LinearAttn(C.Structure):
+    """tlhip_linear_attn"""
+    _fields_ = [(n, i64) for n in ("heads", "dim", "vdim", "rank", "q_off", "k_off", "v_off", "gate_off", "low_off", "y_off")] + \
+               [(n, P) for n in ("a2", "bias", "norm", "state")] + [(n, f32) for n in ("q_scale", "tau", "eps", "out_scale")]
+
+
+class PolyNorm(C.Structure):
+    """tlhip_polynorm"""
+    _fields_ = [(n, i64) for n in ("ff", "z_off", "y_off")] + [(n, f32) for n in ("a", "b", "c", "e", "eps")]
 
 
 class TlHipError(RuntimeError):
@@ -546,6 +575,36 @@ class TlHip:
     def attn_prefill_tok(self, q, K, V, out, Hq, Hkv, T, kv_max, D, scale, kv_bf16=False, pos0=0):
         self._chk(self.c.tlhip_attn_prefill_tok(q.ptr, K.ptr, V.ptr, out.ptr, Hq, Hkv, T, kv_max, D, scale,
                                                 1 if kv_bf16 else 0, pos0))
+
+    # layers with two mixers side by side: at / la / pn are WindowAttn / LinearAttn / PolyNorm or None
+    def mix_step(self, u, y, at, la, pn, pos, d_pos=None, partials=None):
+        ref = lambda s: C.byref(s) if s is not None else None
+        self._chk(self.c.tlhip_mix_step(u.ptr, y.ptr, ref(at), ref(la), ref(pn), pos, d_pos.ptr if d_pos else None,
+                                        partials.ptr if partials else None, partials.nbytes if partials else 0))
+
+    def mix_partials_bytes(self, at):
+        return int(self.c.tlhip_mix_partials_bytes(C.byref(at)))
+
+    def window_attn_chunk(self, u, ldu, y, ldy, at, T, pos0):
+        self._chk(self.c.tlhip_window_fill(u.ptr, ldu, C.byref(at), T, pos0))
+        self._chk(self.c.tlhip_window_attn_chunk(u.ptr, ldu, y.ptr, ldy, C.byref(at), T, pos0))
+
+    def linear_attn_chunk(self, u, ldu, y, ldy, la, T, pos0):
+        self._chk(self.c.tlhip_linear_attn_chunk(u.ptr, ldu, y.ptr, ldy, C.byref(la), T, pos0))
+
+    def polynorm_rows(self, u, ldu, y, ldy, pn, T):
+        self._chk(self.c.tlhip_polynorm_rows(u.ptr, ldu, y.ptr, ldy, C.byref(pn), T))
+
+    def embed_sinusoid(self, table, tokens, out, T, width, ld, vocab, pos0, d_pos=None):
+        self._chk(self.c.tlhip_embed_sinusoid(table.ptr, tokens.ptr, out.ptr, T, width, ld, vocab, pos0,
+                                              d_pos.ptr if d_pos else None))
+
+    def residual_sum(self, x, parts, S, add, vec, out, n, rows):
+        opt = lambda b: b.ptr if b is not None else None
+        self._chk(self.c.tlhip_residual_sum(x.ptr, opt(parts), S, opt(add), opt(vec), out.ptr, n, rows))
+
+    def gather_rows(self, src, idx, out, n, rows, src_rows):
+        self._chk(self.c.tlhip_gather_rows(src.ptr, idx.ptr, out.ptr, n, rows, src_rows))
 
     def tune_attn_prefill(self, kernel):
         """0 / False: built-in choice, 1 / True: VALU kernel, 2: fp32 matrix pipe, 4: f16 terms."""

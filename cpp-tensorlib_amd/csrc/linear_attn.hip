@@ -1,0 +1,318 @@
+// Prompt chunks of the gated linear attention. The recurrence
+//   S_t = diag(a_t) S_(t-1) + k_t v_t^T,   o_t = S_t^T q_t
+// over pieces of C tokens: with b_t the base-2 log of the decay product since the piece began,
+//   o_t = (q_t 2^b_t) S_0 + sum_(s <= t) [sum_d q_td k_sd 2^(b_td - b_sd)] v_s
+//   S_C = 2^b_C S_0 + sum_s (k_s 2^(b_C - b_s)) v_s^T.
+// Three launches: linear_piece_kernel does, for all pieces at once, what needs no state (the second
+// term of o, the sum of S_C, the decay products); linear_scan_kernel carries the state through the
+// pieces; linear_out_kernel adds the first term and applies norm and gate.
+//
+// 2^(b_t - b_s) is never formed as 2^b_t 2^-b_s over a whole piece, which overflows under strong
+// decays. A piece is cut into blocks of 16 tokens; L_t is the log decay since the block began and tot
+// the block's total. Q' = q 2^L_t and K' = k 2^(tot - L_s) have exponents <= 0, and block i sees block
+// j < i as  sum_d Q'_td K'_sd 2^(sum of the totals between them). On the diagonal the factor is
+// 2^-tot, which is safe while |tot| stays below kFastRange; beyond it the block takes 2^(L_t - L_s)
+// pair by pair.
+//
+// All products run on the fp32 matrix pipe (v_mfma_f32_16x16x4_f32: exact f32 products, fp32 sums).
+#include "linear_attn.hpp"
+
+namespace tlhip {
+
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+__device__ __forceinline__ f32x4 mfma16(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+
+constexpr float kFastRange = 96.f;
+constexpr int kVSlice = 64;        // value columns of one block of linear_piece_kernel
+
+// Scratch of a call, per head and piece: decay products [dp], state term [dp][vp]; per head and
+// token: decayed query [dp], inner output [vp]. dp, vp: dim and vdim rounded up to 16.
+struct PieceBuf {
+  float *dec, *st, *qd, *oi;
+  int C, np, dp, vp;               // tokens per piece, pieces
+};
+
+// Block (piece, head, value slice) of 512 threads.
+__global__ __launch_bounds__(512) void linear_piece_kernel(const float* __restrict__ u, int64_t ldu, const tlhip_linear_attn a,
+                                                           int T, const PieceBuf pb) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int tid = threadIdx.x, lane = tid & 63, l15 = lane & 15, lg = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int piece = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * kVSlice;
+  const int C = pb.C, dp = pb.dp, vp = pb.vp, dim = (int)a.dim, vdim = (int)a.vdim;
+  const int NB = C / 16, QS = dp + 4, nv = min(kVSlice, vp - v0);
+  constexpr int VS = kVSlice + 4;
+  const int AS = C + 4;
+  float* Q = lds;                      // [C][QS] q, then Q'
+  float* K = Q + C * QS;               // [C][QS] k, then K'
+  float* Lg = K + C * QS;              // [C][QS] log2 decays since the block began
+  float* V = Lg + C * QS;              // [C][VS]
+  float* A = V + C * VS;               // [C][AS]
+  float* tot = A + C * AS;             // [NB][dp] block totals
+  int* slow = reinterpret_cast<int*>(tot + NB * dp);   // [NB]
+  const int t0 = piece * C, nt = min(C, T - t0);
+  const float inv_tau = 1.0f / a.tau;
+
+  if (tid < NB) slow[tid] = 0;
+  for (int i = tid; i < C * dp; i += 512) {
+    const int t = i / dp, d = i - t * dp;
+    float q = 0.f, k = 0.f, lg2 = 0.f;
+    if (t < nt && d < dim) {
+      const float* row = u + (size_t)(t0 + t) * ldu;
+      q = row[a.q_off + h * dim + d] * a.q_scale;
+      k = row[a.k_off + h * dim + d];
+      lg2 = log2_decay(decay_logit(a, row + a.low_off, h * dim + d), inv_tau);
+    }
+    Q[t * QS + d] = q;
+    K[t * QS + d] = k;
+    Lg[t * QS + d] = lg2;
+  }
+  for (int i = tid; i < C * kVSlice; i += 512) {
+    const int t = i / kVSlice, v = i % kVSlice;
+    V[t * VS + v] = t < nt && v0 + v < vdim ? u[(size_t)(t0 + t) * ldu + a.v_off + (int64_t)h * vdim + v0 + v] : 0.f;
+  }
+  __syncthreads();
+  for (int i = tid; i < NB * dp; i += 512) {         // running sums of the logs inside each block
+    const int b = i / dp, d = i - b * dp;
+    float s = 0.f;
+    for (int t = 16 * b; t < 16 * b + 16; t++) {
+      s += Lg[t * QS + d];
+      Lg[t * QS + d] = s;
+    }
+    tot[b * dp + d] = s;
+    if (s < -kFastRange) slow[b] = 1;                // (every writer stores the same value)
+  }
+  __syncthreads();
+  // diagonal blocks with strong decays, from q and k as they are
+  for (int b = 0; b < NB; b++) {
+    if (!slow[b]) continue;
+    if (tid < 256) {
+      const int t = 16 * b + tid / 16, s = 16 * b + tid % 16;
+      float acc = 0.f;
+      if (s <= t)
+        for (int d = 0; d < dim; d++) acc = fmaf(Q[t * QS + d] * K[s * QS + d], exp2f(Lg[t * QS + d] - Lg[s * QS + d]), acc);
+      A[t * AS + s] = acc;
+    }
+  }
+  __syncthreads();
+  for (int i = tid; i < C * dp; i += 512) {
+    const int t = i / dp, d = i - t * dp, b = t >> 4;
+    const float L = Lg[t * QS + d];
+    Q[t * QS + d] *= exp2f(L);
+    K[t * QS + d] *= exp2f(tot[b * dp + d] - L);
+  }
+  __syncthreads();
+  // A[t][s]: 16 x 16 tiles on and below the diagonal, dealt over the wavefronts
+  for (int tile = wave; tile < NB * (NB + 1) / 2; tile += 8) {
+    int i = 0, j = tile;
+    while (j > i) { i++; j -= i; }
+    if (i == j && slow[i]) continue;
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    for (int d0 = 0; d0 < dp; d0 += 16) {
+      const int d = d0 + 4 * lg;
+      float4 q = *reinterpret_cast<const float4*>(Q + (16 * i + l15) * QS + d);
+      const float4 k = *reinterpret_cast<const float4*>(K + (16 * j + l15) * QS + d);
+      if (i == j) {
+        const float* tp = tot + i * dp + d;
+        q.x *= exp2f(-tp[0]); q.y *= exp2f(-tp[1]); q.z *= exp2f(-tp[2]); q.w *= exp2f(-tp[3]);
+      } else if (i > j + 1) {
+        float4 e = make_float4(0.f, 0.f, 0.f, 0.f);
+        for (int m = j + 1; m < i; m++) {
+          const float* tp = tot + m * dp + d;
+          e.x += tp[0]; e.y += tp[1]; e.z += tp[2]; e.w += tp[3];
+        }
+        q.x *= exp2f(e.x); q.y *= exp2f(e.y); q.z *= exp2f(e.z); q.w *= exp2f(e.w);
+      }
+      acc = mfma16(q.x, k.x, acc);
+      acc = mfma16(q.y, k.y, acc);
+      acc = mfma16(q.z, k.z, acc);
+      acc = mfma16(q.w, k.w, acc);
+    }
+#pragma unroll
+    for (int v = 0; v < 4; v++) {
+      const int t = 4 * lg + v;
+      A[(16 * i + t) * AS + 16 * j + l15] = i == j && l15 > t ? 0.f : acc[v];
+    }
+  }
+  const size_t hp = (size_t)h * pb.np + piece;
+  if (blockIdx.z == 0) {                             // decayed queries and the piece's decay products
+    for (int i = tid; i < C * dp; i += 512) {
+      const int t = i / dp, d = i - t * dp, b = t >> 4;
+      float e = 0.f;
+      for (int m = 0; m < b; m++) e += tot[m * dp + d];
+      pb.qd[(hp * C + t) * dp + d] = Q[t * QS + d] * exp2f(e);
+    }
+    for (int d = tid; d < dp; d += 512) {
+      float e = 0.f;
+      for (int m = 0; m < NB; m++) e += tot[m * dp + d];
+      pb.dec[hp * dp + d] = exp2f(e);
+    }
+  }
+  // state term: sum over s of K'_sd 2^(totals after s's block) V_sv
+  for (int tile = wave; tile < (dp / 16) * (nv / 16); tile += 8) {
+    const int dt = tile / (nv / 16), vt = tile % (nv / 16), d = 16 * dt + l15;
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    float e = 0.f;
+    for (int b = NB - 1; b >= 0; b--) {
+      const float w = exp2f(e);
+#pragma unroll
+      for (int j = 0; j < 4; j++) {
+        const int s = 16 * b + 4 * lg + j;
+        acc = mfma16(K[s * QS + d] * w, V[s * VS + 16 * vt + l15], acc);
+      }
+      e += tot[b * dp + d];
+    }
+#pragma unroll
+    for (int v = 0; v < 4; v++) pb.st[(hp * dp + 16 * dt + 4 * lg + v) * vp + v0 + 16 * vt + l15] = acc[v];
+  }
+  __syncthreads();
+  // inner output: A V
+  for (int tile = wave; tile < NB * (nv / 16); tile += 8) {
+    const int i = tile / (nv / 16), vt = tile % (nv / 16);
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    for (int b = 0; b <= i; b++) {
+      const int s = 16 * b + 4 * lg;
+      const float4 p = *reinterpret_cast<const float4*>(A + (16 * i + l15) * AS + s);
+      const float* vp4 = V + s * VS + 16 * vt + l15;
+      acc = mfma16(p.x, vp4[0], acc);
+      acc = mfma16(p.y, vp4[VS], acc);
+      acc = mfma16(p.z, vp4[2 * VS], acc);
+      acc = mfma16(p.w, vp4[3 * VS], acc);
+    }
+#pragma unroll
+    for (int v = 0; v < 4; v++) pb.oi[(hp * C + 16 * i + 4 * lg + v) * vp + v0 + 16 * vt + l15] = acc[v];
+  }
+}
+
+// The state through the pieces: st[piece] becomes the state ahead of the piece, the last state goes to
+// its slot. A thread owns four value columns of one row.
+__global__ __launch_bounds__(256) void linear_scan_kernel(const tlhip_linear_attn a, int T, int pos0, const PieceBuf pb) {
+  const int dim = (int)a.dim, ld = (int)linear_state_ld(a.vdim), nv4 = pb.vp / 4;
+  const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+  if (i >= (size_t)a.heads * pb.dp * nv4) return;
+  const int v = 4 * (int)(i % nv4), d = (int)(i / nv4 % pb.dp), h = (int)(i / nv4 / pb.dp);
+  const size_t slot = (size_t)a.heads * dim * ld, at = ((size_t)h * dim + d) * ld + v;
+  const bool kept = d < dim && v < ld;
+  float* state = static_cast<float*>(a.state);
+  float4 s = make_float4(0.f, 0.f, 0.f, 0.f);
+  if (kept && pos0 > 0) s = *reinterpret_cast<const float4*>(state + (size_t)(pos0 & 1) * slot + at);
+  constexpr int U = 8;                               // pieces requested at once
+  for (int p0 = 0; p0 < pb.np; p0 += U) {
+    float4 t[U];
+    float w[U];
+#pragma unroll
+    for (int k = 0; k < U; k++) {
+      const size_t hp = (size_t)h * pb.np + min(p0 + k, pb.np - 1);
+      t[k] = *reinterpret_cast<const float4*>(pb.st + (hp * pb.dp + d) * pb.vp + v);
+      w[k] = pb.dec[hp * pb.dp + d];
+    }
+#pragma unroll
+    for (int k = 0; k < U; k++)
+      if (p0 + k < pb.np) {
+        const size_t hp = (size_t)h * pb.np + p0 + k;
+        *reinterpret_cast<float4*>(pb.st + (hp * pb.dp + d) * pb.vp + v) = s;
+        s.x = fmaf(w[k], s.x, t[k].x); s.y = fmaf(w[k], s.y, t[k].y); s.z = fmaf(w[k], s.z, t[k].z); s.w = fmaf(w[k], s.w, t[k].w);
+      }
+  }
+  if (kept) *reinterpret_cast<float4*>(state + (size_t)((pos0 + T) & 1) * slot + at) = s;
+}
+
+// Block (TM tokens, head) of 512 threads: the state's part of o, norm over vdim, gate.
+template <int MT>
+__global__ __launch_bounds__(512) void linear_out_kernel(const float* __restrict__ u, int64_t ldu, float* __restrict__ y,
+                                                         int64_t ldy, const tlhip_linear_attn a, int T, const PieceBuf pb) {
+  constexpr int TM = 16 * MT;
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int tid = threadIdx.x, lane = tid & 63, l15 = lane & 15, lg = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int t0 = blockIdx.x * TM, h = blockIdx.y, dp = pb.dp, vp = pb.vp, OS = vp + 4, vdim = (int)a.vdim;
+  const size_t hp = (size_t)h * pb.np + t0 / pb.C, hr = (size_t)h * pb.np * pb.C + t0;
+  for (int vt = wave; vt < vp / 16; vt += 8) {
+    f32x4 acc[MT];
+#pragma unroll
+    for (int mt = 0; mt < MT; mt++)
+#pragma unroll
+      for (int v = 0; v < 4; v++) acc[mt][v] = pb.oi[(hr + 16 * mt + 4 * lg + v) * vp + 16 * vt + l15];
+    for (int d0 = 0; d0 < dp; d0 += 16) {
+      const int d = d0 + 4 * lg;
+      const float* sp = pb.st + (hp * dp + d) * vp + 16 * vt + l15;
+      const float s0 = sp[0], s1 = sp[vp], s2 = sp[2 * vp], s3 = sp[3 * vp];
+#pragma unroll
+      for (int mt = 0; mt < MT; mt++) {
+        const float4 q = *reinterpret_cast<const float4*>(pb.qd + (hr + 16 * mt + l15) * dp + d);
+        acc[mt] = mfma16(q.x, s0, acc[mt]);
+        acc[mt] = mfma16(q.y, s1, acc[mt]);
+        acc[mt] = mfma16(q.z, s2, acc[mt]);
+        acc[mt] = mfma16(q.w, s3, acc[mt]);
+      }
+    }
+#pragma unroll
+    for (int mt = 0; mt < MT; mt++)
+#pragma unroll
+      for (int v = 0; v < 4; v++) lds[(16 * mt + 4 * lg + v) * OS + 16 * vt + l15] = acc[mt][v];
+  }
+  __syncthreads();
+  for (int r = wave; r < TM && t0 + r < T; r += 8) {
+    float ss = 0.f;
+    for (int v = lane; v < vdim; v += 64) ss = fmaf(lds[r * OS + v], lds[r * OS + v], ss);
+    ss = wave_sum(ss);
+    const float inv = 1.0f / sqrtf(ss / (float)vdim + a.eps);
+    const float* g = u + (size_t)(t0 + r) * ldu + a.gate_off + (int64_t)h * vdim;
+    float* o = y + (size_t)(t0 + r) * ldy + a.y_off + (int64_t)h * vdim;
+    for (int v = lane; v < vdim; v += 64)
+      o[v] = lds[r * OS + v] * inv * static_cast<const float*>(a.norm)[v] * (g[v] * sigmoid_f(g[v])) * a.out_scale;
+  }
+}
+
+static size_t piece_lds(int C, int dp) {
+  return (size_t)(3 * C * (dp + 4) + C * (kVSlice + 4) + C * (C + 4) + (C / 16) * dp + 16) * sizeof(float);
+}
+
+}  // namespace tlhip
+
+using namespace tlhip;
+
+extern "C" {
+
+int tlhip_linear_attn_chunk(const void* u, int64_t ldu, void* y, int64_t ldy, const tlhip_linear_attn* la, int64_t T,
+                            int64_t pos0) {
+  TLHIP_REQUIRE_READY();
+  if (!u || !y || !la || ldu <= 0 || ldy <= 0) return fail(TLHIP_EINVAL, "tlhip_linear_attn_chunk: bad operands");
+  if (T <= 0 || T > (1 << 20) || pos0 < 0 || pos0 + T > (1 << 30)) return fail(TLHIP_EINVAL, "tlhip_linear_attn_chunk: bad chunk");
+  if (int rc = check_linear_attn(la, "tlhip_linear_attn_chunk")) return rc;
+  Context& c = ctx();
+  PieceBuf pb{};
+  pb.dp = (int)(la->dim + 15) / 16 * 16;
+  pb.vp = (int)(la->vdim + 15) / 16 * 16;
+  pb.C = 64;
+  while (pb.C > 16 && (piece_lds(pb.C, pb.dp) > (size_t)c.lds_per_cu || pb.C / 2 >= T)) pb.C /= 2;
+  const size_t lds1 = piece_lds(pb.C, pb.dp);
+  const int mt = pb.C >= 32 ? 2 : 1;
+  const size_t lds3 = (size_t)16 * mt * (pb.vp + 4) * sizeof(float);
+  if (lds1 > (size_t)c.lds_per_cu || lds3 > (size_t)c.lds_per_cu)
+    return fail(TLHIP_EUNSUPPORTED, "tlhip_linear_attn_chunk: head too large for LDS");
+  pb.np = (int)((T + pb.C - 1) / pb.C);
+  const size_t hp = (size_t)la->heads * pb.np, n_dec = hp * pb.dp, n_st = hp * pb.dp * pb.vp, n_qd = hp * pb.C * pb.dp,
+               n_oi = hp * pb.C * pb.vp;
+  float* s = static_cast<float*>(scratch((n_dec + n_st + n_qd + n_oi) * sizeof(float)));
+  if (!s) return fail(TLHIP_ENOMEM, "tlhip_linear_attn_chunk: no scratch");
+  pb.dec = s;
+  pb.st = pb.dec + n_dec;
+  pb.qd = pb.st + n_st;
+  pb.oi = pb.qd + n_qd;
+  const float* pu = static_cast<const float*>(u);
+  hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(linear_piece_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds1);
+  if (e != hipSuccess) return hip_fail(e, "hipFuncSetAttribute(LDS)");
+  hipLaunchKernelGGL(linear_piece_kernel, dim3((unsigned)pb.np, (unsigned)la->heads, (unsigned)((pb.vp + kVSlice - 1) / kVSlice)),
+                     dim3(512), lds1, c.stream, pu, ldu, *la, (int)T, pb);
+  const size_t ns = (size_t)la->heads * pb.dp * (pb.vp / 4);
+  hipLaunchKernelGGL(linear_scan_kernel, dim3((unsigned)((ns + 255) / 256)), dim3(256), 0, c.stream, *la, (int)T, (int)pos0, pb);
+  auto out = mt == 2 ? linear_out_kernel<2> : linear_out_kernel<1>;
+  e = hipFuncSetAttribute(reinterpret_cast<const void*>(out), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds3);
+  if (e != hipSuccess) return hip_fail(e, "hipFuncSetAttribute(LDS)");
+  hipLaunchKernelGGL(out, dim3((unsigned)((T + 16 * mt - 1) / (16 * mt)), (unsigned)la->heads), dim3(512), lds3, c.stream, pu, ldu,
+                     static_cast<float*>(y), ldy, *la, (int)T, pb);
+  TLHIP_CHECK_LAUNCH(TLHIP_C_LINEAR_ATTN);
+}
+
+}  // extern "C"

@@ -185,6 +185,20 @@ struct api {
   int (*gemv_bf16_row_attn)(const void*, int64_t, int64_t, int64_t, const void*, void*, int64_t, int64_t) = nullptr;
   int (*warm_fork)(const void* const*, const int64_t*, int, int, int) = nullptr;
   int (*warm_join)() = nullptr;
+  int64_t (*window_ring_ld)(int64_t) = nullptr;
+  int64_t (*linear_state_bytes)(int64_t, int64_t, int64_t) = nullptr;
+  int64_t (*mix_partials_bytes)(const void*) = nullptr;
+  int (*mix_step)(const void*, void*, const void*, const void*, const void*, int64_t, const void*, void*,
+                  int64_t) = nullptr;
+  int (*window_fill)(const void*, int64_t, const void*, int64_t, int64_t) = nullptr;
+  int (*window_attn_chunk)(const void*, int64_t, void*, int64_t, const void*, int64_t, int64_t) = nullptr;
+  int (*linear_attn_chunk)(const void*, int64_t, void*, int64_t, const void*, int64_t, int64_t) = nullptr;
+  int (*polynorm_rows)(const void*, int64_t, void*, int64_t, const void*, int64_t) = nullptr;
+  int (*embed_sinusoid)(const void*, const void*, void*, int64_t, int64_t, int64_t, int64_t, int64_t,
+                        const void*) = nullptr;
+  int (*residual_sum)(const void*, const void*, int64_t, const void*, const void*, void*, int64_t,
+                      int64_t) = nullptr;
+  int (*gather_rows)(const void*, const void*, void*, int64_t, int64_t, int64_t) = nullptr;
   int (*event_create)(void**) = nullptr;
   int (*event_record)(void*) = nullptr;
   int (*event_elapsed_ms)(void*, void*, float*) = nullptr;
@@ -380,7 +394,13 @@ struct context {
               bind(f.attn_parts_splits, "tlhip_attn_parts_splits") &&
               bind(f.attn_decode_qkv_parts, "tlhip_attn_decode_qkv_parts") &&
               bind(f.gemv_q4_attn, "tlhip_gemv_q4_attn") &&
-              bind(f.gemv_bf16_row_attn, "tlhip_gemv_bf16_row_attn");
+              bind(f.gemv_bf16_row_attn, "tlhip_gemv_bf16_row_attn") &&
+              bind(f.window_ring_ld, "tlhip_window_ring_ld") && bind(f.linear_state_bytes, "tlhip_linear_state_bytes") &&
+              bind(f.mix_partials_bytes, "tlhip_mix_partials_bytes") && bind(f.mix_step, "tlhip_mix_step") &&
+              bind(f.window_fill, "tlhip_window_fill") && bind(f.window_attn_chunk, "tlhip_window_attn_chunk") &&
+              bind(f.linear_attn_chunk, "tlhip_linear_attn_chunk") && bind(f.polynorm_rows, "tlhip_polynorm_rows") &&
+              bind(f.embed_sinusoid, "tlhip_embed_sinusoid") && bind(f.residual_sum, "tlhip_residual_sum") &&
+              bind(f.gather_rows, "tlhip_gather_rows");
     if (!ok) return;
     bind(f.warm_fork, "tlhip_warm_fork") && bind(f.warm_join, "tlhip_warm_join");   // optional
     why.clear();
@@ -1567,6 +1587,116 @@ struct kv_cache {
     K = V = dpos_partials = nullptr;
   }
 };
+
+// ---- layers with two mixers side by side (no counterpart in the reference) ----------------------
+// Descriptions of the sublayers of such a layer: where their columns lie in the row u that the
+// layer's projection writes and in the row y that its output product reads, sizes, constants and
+// state. Same memory layout as the structs of the C ABI (tensorlib_hip.h says what each field means).
+struct window_attn {
+  int64_t heads = 0, kv_heads = 0, dim = 0, window = 0;
+  int64_t q_off = 0, k_off = 0, gate_off = -1, y_off = 0;
+  void* ring = nullptr;
+  int64_t ring_rows = 0, ring_ld = 0;
+  float scale = 1, temp_coef = 0, temp_every = 0, slope_exp = 0, out_scale = 1;
+};
+struct linear_attn {
+  int64_t heads = 0, dim = 0, vdim = 0, rank = 0;
+  int64_t q_off = 0, k_off = 0, v_off = 0, gate_off = 0, low_off = 0, y_off = 0;
+  void *a2 = nullptr, *bias = nullptr, *norm = nullptr;
+  void* state = nullptr;
+  float q_scale = 1, tau = 1, eps = 0, out_scale = 1;
+};
+struct polynorm {
+  int64_t ff = 0, z_off = 0, y_off = 0;
+  float a = 0, b = 0, c = 0, e = 0, eps = 0;
+};
+inline int64_t window_ring_ld(int64_t dim) {
+  auto& c = context::get();
+  return c.ready ? c.f.window_ring_ld(dim) : 0;
+}
+inline int64_t linear_state_bytes(int64_t heads, int64_t dim, int64_t vdim) {
+  auto& c = context::get();
+  return c.ready ? c.f.linear_state_bytes(heads, dim, vdim) : 0;
+}
+inline int64_t mix_partials_bytes(const window_attn* at) {
+  auto& c = context::get();
+  return c.ready ? c.f.mix_partials_bytes(at) : 0;
+}
+// One token through the sublayers given (nullptr: absent), one launch: u -> y, new key and state stored.
+inline bool mix_step(void* u, void* y, const window_attn* at, const linear_attn* la, const polynorm* pn, int64_t pos,
+                     void* d_pos, void* partials, int64_t partials_bytes) {
+  launch L;
+  if (!L.ok || !u || !y) return false;
+  L.reads(u);
+  if (d_pos) L.reads(d_pos);
+  if (la) L.reads(la->a2, la->bias, la->norm);
+  L.writes(y);
+  if (at) L.writes(at->ring);
+  if (la) L.writes(la->state);
+  if (partials) L.writes(partials);
+  return L.sent(L.lib.mix_step(u, y, at, la, pn, pos, d_pos, partials, partials_bytes));
+}
+// The same for a chunk of T tokens at pos0, one mechanism per call.
+inline bool window_attn_chunk(void* u, int64_t ldu, void* y, int64_t ldy, const window_attn& at, int64_t T, int64_t pos0) {
+  launch L;
+  if (!L.ok || !u || !y) return false;
+  L.reads(u);
+  L.writes(y, at.ring);
+  return L.sent(L.lib.window_fill(u, ldu, &at, T, pos0)) && L.sent(L.lib.window_attn_chunk(u, ldu, y, ldy, &at, T, pos0));
+}
+inline bool linear_attn_chunk(void* u, int64_t ldu, void* y, int64_t ldy, const linear_attn& la, int64_t T, int64_t pos0) {
+  launch L;
+  if (!L.ok || !u || !y) return false;
+  L.reads(u, la.a2, la.bias, la.norm);
+  L.writes(y, la.state);
+  return L.sent(L.lib.linear_attn_chunk(u, ldu, y, ldy, &la, T, pos0));
+}
+inline bool polynorm_rows(void* u, int64_t ldu, void* y, int64_t ldy, const polynorm& pn, int64_t T) {
+  launch L;
+  if (!L.ok || !u || !y) return false;
+  L.reads(u);
+  L.writes(y);
+  return L.sent(L.lib.polynorm_rows(u, ldu, y, ldy, &pn, T));
+}
+// Token rows + sinusoidal positions; tokens: device int32.
+inline bool embed_sinusoid(void* table, void* tokens, void* out, int64_t T, int64_t width, int64_t ld, int64_t vocab,
+                           int64_t pos0, void* d_pos = nullptr) {
+  launch L;
+  if (!L.ok) return false;
+  L.reads(table, tokens);
+  if (d_pos) L.reads(d_pos);
+  L.writes(out);
+  return L.sent(L.lib.embed_sinusoid(table, tokens, out, T, width, ld, vocab, pos0, d_pos));
+}
+// out = x + parts + add + vec (each may be nullptr)
+inline bool residual_sum(void* x, void* parts, int64_t n_parts, void* add, void* vec, void* out, int64_t n, int64_t rows) {
+  launch L;
+  if (!L.ok) return false;
+  L.reads(x);
+  if (parts) L.reads(parts);
+  if (add) L.reads(add);
+  if (vec) L.reads(vec);
+  L.writes(out);
+  return L.sent(L.lib.residual_sum(x, parts, n_parts, add, vec, out, n, rows));
+}
+inline bool gather_rows(void* src, void* idx, void* out, int64_t n, int64_t rows, int64_t src_rows) {
+  launch L;
+  if (!L.ok) return false;
+  L.reads(src, idx);
+  L.writes(out);
+  return L.sent(L.lib.gather_rows(src, idx, out, n, rows, src_rows));
+}
+// A device-only buffer of zeros (bytes a multiple of 4).
+inline void* alloc_zeros(int64_t bytes) {
+  void* p = alloc_device(bytes);
+  auto& c = context::get();
+  if (p && c.f.fill_u32(p, 0u, (size_t)(bytes + 3) / 4) != 0) {
+    release(p, 0, nullptr);
+    return nullptr;
+  }
+  if (p) c.pending = true;
+  return p;
+}
 
 }  // namespace hip
 }  // namespace tl

@@ -98,7 +98,8 @@ typedef enum {
   TLHIP_C_ATTN_DECODE, TLHIP_C_ROPE, TLHIP_C_RMSNORM, TLHIP_C_RMSNORM_RES, TLHIP_C_SWIGLU,
   TLHIP_C_ARGMAX, TLHIP_C_KV_APPEND, TLHIP_C_KV_FILL, TLHIP_C_SPLIT_HEADS,
   TLHIP_C_MERGE_HEADS, TLHIP_C_GEMM_BF16_NT, TLHIP_C_ATTN_PREFILL, TLHIP_C_CONVERT,
-  TLHIP_C_QUANTIZE_Q4, TLHIP_C_COUNT
+  TLHIP_C_QUANTIZE_Q4, TLHIP_C_MIX_STEP, TLHIP_C_WINDOW_ATTN, TLHIP_C_LINEAR_ATTN, TLHIP_C_POLYNORM,
+  TLHIP_C_EMBED, TLHIP_C_RESIDUAL, TLHIP_C_COUNT
 } tlhip_census_id;
 int tlhip_census(uint64_t* counts, int n);  /* copies min(n, TLHIP_C_COUNT) counters */
 int tlhip_census_reset(void);
@@ -458,6 +459,80 @@ int tlhip_split_heads(const void* src, const void* bias, void* dst, int64_t T, i
                       int64_t off, int64_t H, int64_t D);
 /* [H,T,D] -> [T,H*D].  cuda.h:866-879 */
 int tlhip_merge_heads(const void* src, void* dst, int64_t T, int64_t H, int64_t D);
+
+/* ---- layers with two mixers side by side (no reference counterpart) -------------------------------
+ * One projection writes a row u of everything a layer's sublayers read (queries, keys, gates, ...);
+ * each sublayer writes its part of a row y, and one product over y is the layer's output. The
+ * structs below say where a sublayer's columns lie in u and y (element offsets into a row) and hold
+ * its sizes and constants. Sizes are free unless stated; a refusal is TLHIP_EUNSUPPORTED.
+ *
+ * Sliding-window attention whose values are its keys. Position i sees j with 0 <= i - j < window;
+ * score = (q_i * t(i)) . k_j * scale - slope_h (i - j), with
+ *   t(p) = 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1)     (temp_every <= 0: 1), and
+ *   slope_h = 2^(-slope_exp (h + 1) / heads)                       (slope_exp <= 0: no bias);
+ * y = out_scale * softmax(score) . k, times sigmoid(gate) when gate_off >= 0.
+ * Keys live in a ring: position p in row p % ring_rows, [kv_heads][ring_rows][ring_ld] f32,
+ * ring_ld = tlhip_window_ring_ld(dim) with zeros past dim, ring_rows a multiple of 32 and at least
+ * window - 1 + (rows of the longest chunk). The whole ring must be zeroed before its first use. */
+typedef struct {
+  int64_t heads, kv_heads, dim, window;
+  int64_t q_off, k_off, gate_off, y_off;
+  void* ring;
+  int64_t ring_rows, ring_ld;
+  float scale, temp_coef, temp_every, slope_exp, out_scale;
+} tlhip_window_attn;
+int64_t tlhip_window_ring_ld(int64_t dim);   /* 0: dim beyond what the kernels hold (256) */
+
+/* Gated linear attention. Per head, S [dim][vdim]: S_t = diag(a_t) S_(t-1) + k_t v_t^T,
+ * o_t = S_t^T (q_t * q_scale), a_t = sigmoid(z)^(1/tau), z = A2 (low) + bias with low the rank
+ * columns at low_off, A2 bf16 [heads*dim][rank]; y = out_scale * rmsnorm_vdim(o) * norm * silu(gate).
+ * The state has two slots of tlhip_linear_state_bytes / 2 bytes, [heads][dim][vdim rounded up to 4]:
+ * the state ahead of position p is slot p % 2, and the step at p (chunk p .. p + T - 1) writes slot
+ * (p + 1) % 2 ((p + T) % 2): a step can be repeated at its position. At position 0 the state is
+ * zero, whatever the slot holds. */
+typedef struct {
+  int64_t heads, dim, vdim, rank;
+  int64_t q_off, k_off, v_off, gate_off, low_off, y_off;
+  const void *a2, *bias, *norm;
+  void* state;
+  float q_scale, tau, eps, out_scale;
+} tlhip_linear_attn;
+int64_t tlhip_linear_state_bytes(int64_t heads, int64_t dim, int64_t vdim);
+
+/* y = a N(z) + b N(z^2) + c N(z^3) + e over the row's ff values; powers element by element,
+ * N(w) = w / sqrt(mean(w^2) + eps). */
+typedef struct {
+  int64_t ff, z_off, y_off;
+  float a, b, c, e, eps;
+} tlhip_polynorm;
+
+/* One token: u [one row] -> y [one row] for the sublayers given (NULL: not there), all in one launch
+ * and, where the window is cut into splits, a second one that merges them. The new key goes to the
+ * ring, the new state to its slot. Position: pos, or *d_pos when d_pos is non-NULL. `partials`
+ * (tlhip_mix_partials_bytes bytes; may be NULL when that is 0) is the caller's. */
+int64_t tlhip_mix_partials_bytes(const tlhip_window_attn* at);
+int tlhip_mix_step(const void* u, void* y, const tlhip_window_attn* at, const tlhip_linear_attn* la,
+                   const tlhip_polynorm* pn, int64_t pos, const void* d_pos, void* partials,
+                   int64_t partials_bytes);
+/* A chunk of T tokens at positions pos0 .. pos0 + T - 1, u rows ldu and y rows ldy elements apart. */
+int tlhip_window_fill(const void* u, int64_t ldu, const tlhip_window_attn* at, int64_t T, int64_t pos0);
+int tlhip_window_attn_chunk(const void* u, int64_t ldu, void* y, int64_t ldy, const tlhip_window_attn* at,
+                            int64_t T, int64_t pos0);
+int tlhip_linear_attn_chunk(const void* u, int64_t ldu, void* y, int64_t ldy, const tlhip_linear_attn* la,
+                            int64_t T, int64_t pos0);
+int tlhip_polynorm_rows(const void* u, int64_t ldu, void* y, int64_t ldy, const tlhip_polynorm* pn, int64_t T);
+
+/* out[t][ld] f32 = widened bf16 row tokens[t] of a [vocab, width] table + the sinusoid of position
+ * pos0 + t (or *d_pos + t): column 2i adds sin(p 10000^(-2i/width)), column 2i + 1 the cosine; columns
+ * width .. ld - 1 are zero. tokens: device int32, clamped to [0, vocab). */
+int tlhip_embed_sinusoid(const void* table, const void* tokens, void* out, int64_t T, int64_t width,
+                         int64_t ld, int64_t vocab, int64_t pos0, const void* d_pos);
+/* out[t] = x[t] + parts[0][t] + ... + parts[S-1][t] + add[t] + vec, rows of n; parts, add and vec may
+ * be NULL; vec is one row. out may alias x. */
+int tlhip_residual_sum(const void* x, const void* parts, int64_t S, const void* add, const void* vec,
+                       void* out, int64_t n, int64_t rows);
+/* out[i] = src[idx[i]], rows of n f32; idx: device int32, clamped to [0, src_rows). */
+int tlhip_gather_rows(const void* src, const void* idx, void* out, int64_t n, int64_t rows, int64_t src_rows);
 
 /* Upper bound on the K splits of the [K,N] GEMVs (tlhip_gemv_f32 / tlhip_gemv_bf16); 1 = no
  * split, 0 = the built-in choice. The reference's diagnostic knob set_no_splitk (cuda.h:193-197,

@@ -79,11 +79,11 @@ QWEN_LIB = os.path.join(LIBDIR, "libtl_qwen.so")
 def build_host(force=False, verbose=True):
     """libtl_qwen.so: the header-only C++ host layer (include/tl/) behind a C entry
     layer, compiled with plain g++; it reaches the HIP library through dlopen."""
-    src = os.path.join(CSRC, "qwen_capi.cpp")
+    srcs = [os.path.join(CSRC, f) for f in ("qwen_capi.cpp", "model_capi.cpp")]
     inc = os.path.join(HERE, "include")
-    deps = [src] + [os.path.join(inc, "tl", f) for f in os.listdir(os.path.join(inc, "tl"))]
+    deps = srcs + [os.path.join(inc, "tl", f) for f in os.listdir(os.path.join(inc, "tl"))]
     if force or _stale(QWEN_LIB, deps):
-        cmd = ["g++", "-std=c++17", "-O2", "-fPIC", "-shared", "-Wall", "-Wextra", "-I", inc, src,
+        cmd = ["g++", "-std=c++17", "-O2", "-fPIC", "-shared", "-Wall", "-Wextra", "-I", inc] + srcs + [
                "-o", QWEN_LIB, "-ldl"]
         if verbose:
             print(" ".join(cmd), flush=True)

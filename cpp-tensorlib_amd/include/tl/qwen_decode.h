@@ -31,12 +31,16 @@
 #include <string>
 #include <vector>
 
+#include "decode_loop.h"
 #include "gguf.h"
 #include "hip.h"
+#include "linear.h"
 #include "types.h"
 
 namespace tl {
 namespace qwen {
+
+using namespace weights;
 
 struct dims {
   int64_t n_layers, hidden, n_q_heads, n_kv_heads, head_dim, ff, vocab, max_ctx;
@@ -51,83 +55,6 @@ inline dims qwen25_05b(int64_t max_ctx = 4096) {
 }
 inline dims qwen25_7b(int64_t max_ctx = 4352) {
   return dims{28, 3584, 28, 4, 128, 18944, 152064, max_ctx, 1e-6f, 1e6f};
-}
-
-// A linear weight resident on the device. q4: the reference's one-buffer layout
-// [packed [N][K/2] | scales [N][K/32]] (types.h:25-31). bf16_row: [N][K] bf16,
-// the layout gemv_bf16_row and gemm_bf16_nt share (cuda.h:765-841).
-enum class wfmt { q4, bf16_row };
-struct linear {
-  void* w = nullptr;
-  int64_t N = 0, K = 0;
-  wfmt fmt = wfmt::q4;
-  int64_t bytes() const { return fmt == wfmt::q4 ? q4_bytes(N, K) : N * K * 2; }
-};
-
-// y[N] = a[K] . W
-inline bool gemv(const linear& L, void* a, void* y) {
-  if (L.fmt == wfmt::q4) {
-    void* scales = static_cast<char*>(L.w) + L.N * L.K / 2;
-    return hip::gemv_q4(a, L.w, scales, y, L.N, L.K, kQ4Group);
-  }
-  return hip::gemv_bf16_row(a, L.w, y, L.N, L.K);
-}
-
-// y = W . (attention output merged from n_parts split partials)
-inline bool gemv_attn(const linear& L, void* parts, int n_parts, int64_t heads, int64_t head_dim, void* y) {
-  if (L.fmt == wfmt::q4)
-    return hip::gemv_q4_attn(parts, n_parts, heads, head_dim, L.w, static_cast<char*>(L.w) + L.N * L.K / 2, y, L.N,
-                             L.K, kQ4Group);
-  return hip::gemv_bf16_row_attn(parts, n_parts, heads, head_dim, L.w, y, L.N, L.K);
-}
-
-// Prompt-chunk products, T rows at a time: out[T, N] = a[T, K] . W^T for either weight format
-// (bf16 rows or int4); `_parts` leaves the K-split parts for the launch that consumes them,
-// `_swiglu` takes the fused [gate | up] weight and writes the gated activation [T, N / 2].
-inline bool gemm(const linear& L, void* a, void* out, int64_t T) {
-  if (L.fmt == wfmt::q4)
-    return hip::gemm_q4_nt(a, L.w, static_cast<char*>(L.w) + L.N * L.K / 2, out, T, L.N, L.K, kQ4Group);
-  return hip::gemm_bf16_nt(a, L.w, out, T, L.N, L.K);
-}
-inline bool gemm_parts(const linear& L, void* a, void* parts, int64_t parts_bytes, int64_t T, int* n_parts) {
-  if (L.fmt == wfmt::q4)
-    return hip::gemm_q4_nt_parts(a, L.w, static_cast<char*>(L.w) + L.N * L.K / 2, parts, parts_bytes, T, L.N,
-                                 L.K, n_parts, kQ4Group);
-  return hip::gemm_bf16_nt_parts(a, L.w, parts, parts_bytes, T, L.N, L.K, n_parts);
-}
-inline bool gemm_swiglu(const linear& L, void* a, void* act, int64_t T) {
-  if (L.fmt == wfmt::q4)
-    return hip::gemm_q4_nt_swiglu(a, L.w, static_cast<char*>(L.w) + L.N * L.K / 2, act, T, L.N / 2, L.K,
-                                  kQ4Group);
-  return hip::gemm_bf16_nt_swiglu(a, L.w, act, T, L.N / 2, L.K);
-}
-
-// y = W . swiglu(gu)
-inline bool gemv_swiglu(const linear& L, void* gu, void* y) {
-  if (L.fmt == wfmt::q4) {
-    void* scales = static_cast<char*>(L.w) + L.N * L.K / 2;
-    return hip::gemv_q4_swiglu(gu, L.w, scales, y, L.N, L.K, kQ4Group);
-  }
-  return hip::gemv_bf16_row_swiglu(gu, L.w, y, L.N, L.K);
-}
-// s = x (+ delta) -> xout ; y = W . rmsnorm(s, norm_w)
-inline bool gemv_rmsnorm(const linear& L, void* x, void* delta, void* norm_w, void* xout, void* y,
-                         float eps) {
-  if (L.fmt == wfmt::q4) {
-    void* scales = static_cast<char*>(L.w) + L.N * L.K / 2;
-    return hip::gemv_q4_rmsnorm(x, delta, norm_w, xout, L.w, scales, y, L.N, L.K, kQ4Group, eps);
-  }
-  return hip::gemv_bf16_row_rmsnorm(x, delta, norm_w, xout, L.w, y, L.N, L.K, eps);
-}
-
-// L = [gate rows | up rows]; s = x (+ delta) -> xout ; act = swiglu(gate . n, up . n), n = rmsnorm(s, norm_w)
-inline bool gemv_rmsnorm_gateup(const linear& L, void* x, void* delta, void* norm_w, void* xout, void* act,
-                                float eps) {
-  if (L.fmt == wfmt::q4) {
-    void* scales = static_cast<char*>(L.w) + L.N * L.K / 2;
-    return hip::gemv_q4_rmsnorm_gateup(x, delta, norm_w, xout, L.w, scales, act, L.N, L.K, kQ4Group, eps);
-  }
-  return hip::gemv_bf16_row_rmsnorm_gateup(x, delta, norm_w, xout, L.w, act, L.N, L.K, eps);
 }
 
 struct layer {
@@ -204,14 +131,7 @@ struct model {
 
 namespace detail {
 
-inline void* dev_from_host(const void* src, int64_t bytes) {
-  float* host = nullptr;
-  void* n = hip::alloc(bytes, &host);
-  if (!n) return nullptr;
-  std::memcpy(host, src, (size_t)bytes);
-  hip::upload(n, host, (bytes + 3) / 4);  // device copy current from now on
-  return n;
-}
+using weights::detail::dev_from_host;
 
 // Rows of several q4 matrices with the same K, stacked: packed parts first,
 // then the scale parts, which is again a valid q4 buffer of N = sum(N_i).
@@ -817,21 +737,6 @@ inline bool profile_step(model& M, int64_t token, int64_t pos, step_prof& p) {
   return ok;
 }
 
-// embed -> layers -> device argmax. Returns the greedy token, or -1 when any
-// launch was declined.
-inline int64_t step_greedy(model& M, int64_t token, int64_t pos) {
-  if (!stage_embed(M, token) || !run_layers(M, M.s.embedb, pos)) return -1;
-  int64_t idx = -1;
-  if (!hip::argmax(M.s.logitsb, M.d.vocab, &idx)) return -1;
-  return idx;
-}
-
-// Host view of the logits the last step left on the device.
-inline const float* logits(model& M) {
-  hip::sync_to_host(M.s.logitsb, false);
-  return M.s.logits_host;
-}
-
 // ---- prompt chunks ---------------------------------------------------------------------------
 
 inline bool prefill_reserve(model& M, int64_t T) {
@@ -947,41 +852,6 @@ inline bool stage_chunk(model& M, const int64_t* tokens, int64_t T) {
   return true;
 }
 
-// Consume a prompt in chunks; logits of its LAST token land in s.logitsb (only
-// that row is ever read, so only it meets the lm_head: qm:396-401).
-inline bool prefill(model& M, const int64_t* tokens, int64_t n, int64_t chunk = 512) {
-  if (n <= 0 || chunk <= 0) return false;
-  bool ok = true;
-  int64_t last_T = 0;
-  for (int64_t t0 = 0; t0 < n && ok; t0 += chunk) {
-    last_T = std::min(chunk, n - t0);
-    ok = stage_chunk(M, tokens + t0, last_T) && prefill_layers(M, last_T);
-  }
-  if (!ok) return false;
-  void* last = static_cast<char*>(M.ps.h) + (last_T - 1) * M.d.hidden * 4;
-  return gemv(M.lm_head, last, M.s.logitsb);
-}
-
-// One decode step recorded as a hipGraph at a FIXED position (the throughput
-// measurement replays the same step; replaying re-writes the same cache row).
-struct captured_step {
-  void* graph = nullptr;
-  bool capture(model& M, int64_t pos) {
-    // warm: lets the library size its scratch before the capture opens
-    if (!run_layers(M, M.s.embedb, pos)) return false;
-    hip::flush();
-    if (!hip::capture_begin()) return false;
-    const bool ok = run_layers(M, M.s.embedb, pos);
-    graph = hip::capture_end();
-    return ok && graph != nullptr;
-  }
-  bool replay() { return hip::graph_launch(graph); }
-  void destroy() {
-    hip::graph_destroy(graph);
-    graph = nullptr;
-  }
-};
-
 // Copy the host embedding table to the device once, through a pinned staging block.
 inline bool upload_embed(model& M) {
   if (M.embed_dev) return true;
@@ -1005,139 +875,48 @@ inline bool upload_embed(model& M) {
   return ok;
 }
 
-// Greedy decoding with the whole token loop on the device: one recorded graph does
-//   embedding gather of *d_tok -> layers at *d_pos -> lm_head -> argmax -> *d_tok,
-//   history[*d_pos] = *d_tok, *d_pos += 1
-// so consecutive tokens are queued back to back with no host round trip between them
-// (the reference stages each embedding on the host and reads every argmax back:
-// qm:530-535, 642-647). The host reads the generated ids from the history afterwards.
-struct greedy_loop {
-  void *d_pos = nullptr, *d_tok = nullptr, *history = nullptr, *graph = nullptr;
-  float* history_host = nullptr;
-  int64_t cur_pos = 0, max_ctx = 0;
+// ---- what the decode loops (decode_loop.h) ask of a model --------------------------------------
+inline int64_t vocab_size(const model& M) { return M.d.vocab; }
+inline int64_t context_capacity(const model& M) { return M.layers.empty() ? 0 : M.layers[0].cache.max_ctx; }
+inline int64_t cache_pos(const model& M) { return M.layers.empty() ? 0 : M.layers[0].cache.pos; }
+inline void* logits_device(model& M) { return M.s.logitsb; }
+inline const float* logits_host(const model& M) { return M.s.logits_host; }
+inline const linear& head(const model& M) { return M.lm_head; }
+// One token through all layers; the logits land in logits_device().
+inline bool step_layers(model& M, int64_t pos, void* d_pos = nullptr, bool advance = true) {
+  return run_layers(M, M.s.embedb, pos, nullptr, d_pos, advance);
+}
+// The same with its input taken from a token id on the device.
+inline bool step_layers_from(model& M, void* d_tok, void* d_pos) {
+  const dims& d = M.d;
+  const bool ok = M.embed_f16 ? hip::embed_gather_f16(M.embed_dev, d_tok, M.s.embedb, d.hidden, d.vocab)
+                              : hip::embed_gather_bf16(M.embed_dev, d_tok, M.s.embedb, d.hidden, d.vocab);
+  return ok && step_layers(M, 0, d_pos, /*advance=*/false);
+}
+// What steps with the position on the device need besides the model; false: this model has no such steps.
+inline bool reserve_device_steps(model& M, bool device_tokens) {
+  const dims& d = M.d;
+  if (M.layers.empty() || !M.fused || !hip::graph_available()) return false;
+  if (!M.attn_partials) {
+    M.attn_partials_bytes = hip::attn_partials_bytes(d.n_q_heads, d.n_kv_heads, context_capacity(M), d.head_dim);
+    M.attn_partials = hip::alloc_device(M.attn_partials_bytes);
+  }
+  return M.attn_partials && (!device_tokens || upload_embed(M));
+}
+// T prompt tokens through all layers at the caches' position; final-norm rows in chunk_rows().
+inline bool prompt_chunk(model& M, const int64_t* tokens, int64_t T) {
+  return stage_chunk(M, tokens, T) && prefill_layers(M, T);
+}
+inline void* chunk_rows(model& M) { return M.ps.h; }
+inline int64_t chunk_row_width(const model& M) { return M.d.hidden; }
+inline int64_t longest_chunk(const model&) { return 0; }   // no bound of its own
 
-  bool init(model& M, int64_t first_id, int64_t pos) {
-    if (M.layers.empty() || !M.fused || !hip::graph_available()) return false;
-    const dims& d = M.d;
-    if (first_id < 0 || first_id >= d.vocab) return false;   // later ids are argmax results, in range by construction
-    max_ctx = M.layers[0].cache.max_ctx;
-    cur_pos = pos;
-    if (!upload_embed(M)) return false;
-    if (!M.attn_partials) {
-      M.attn_partials_bytes = hip::attn_partials_bytes(d.n_q_heads, d.n_kv_heads, max_ctx, d.head_dim);
-      M.attn_partials = hip::alloc_device(M.attn_partials_bytes);
-      if (!M.attn_partials) return false;
-    }
-    d_pos = hip::alloc(4, nullptr);
-    d_tok = hip::alloc(4, nullptr);
-    history = hip::alloc(max_ctx * 4, &history_host);
-    if (!d_pos || !d_tok || !history) return false;
-    auto one = [&]() {
-      bool ok = M.embed_f16 ? hip::embed_gather_f16(M.embed_dev, d_tok, M.s.embedb, d.hidden, d.vocab)
-                            : hip::embed_gather_bf16(M.embed_dev, d_tok, M.s.embedb, d.hidden, d.vocab);
-      ok = ok && run_layers(M, M.s.embedb, 0, nullptr, d_pos, /*advance=*/false);
-      ok = ok && hip::argmax_async(M.s.logitsb, d.vocab, d_tok);
-      return ok && hip::token_advance(d_pos, d_tok, history, max_ctx);
-    };
-    hip::upload_u32(d_pos, (unsigned)pos);
-    hip::upload_u32(d_tok, (unsigned)first_id);
-    if (!one()) return false;            // warm run (sizes the library's scratch)
-    hip::flush();
-    hip::upload_u32(d_pos, (unsigned)pos);
-    hip::upload_u32(d_tok, (unsigned)first_id);
-    if (!hip::capture_begin()) return false;
-    const bool ok = one();
-    graph = hip::capture_end();
-    if (!ok && graph) { hip::graph_destroy(graph); graph = nullptr; }
-    return graph != nullptr;
-  }
-  // Queue n greedy steps (no sync). Returns how many were queued before the cache filled.
-  int64_t run(int64_t n) {
-    int64_t done = 0;
-    while (done < n && cur_pos < max_ctx && graph && hip::graph_launch(graph)) {
-      cur_pos++;
-      done++;
-    }
-    return done;
-  }
-  // The token generated at position p (p in [first pos, cur_pos)); blocks until the queue drained.
-  const int32_t* tokens() {
-    hip::sync_to_host(history, false);
-    return reinterpret_cast<const int32_t*>(history_host);
-  }
-  void sync_host_pos(model& M) const { set_cache_pos(M, cur_pos); }
-  void destroy() {
-    if (graph) hip::graph_destroy(graph);
-    for (void* b : {d_pos, d_tok, history})
-      if (b) hip::release(b, 0, nullptr);
-    graph = d_pos = d_tok = history = nullptr;
-  }
-};
-
-// A decode loop on ONE recorded graph (qm:791-905): the position lives in a device
-// scalar that the recorded forward advances itself, so feed()/step() replay the same
-// graph for every token. Falls back to the imperative path when capture is not
-// available; callers never branch on ok().
-struct captured_decoder {
-  void* d_pos = nullptr;
-  void* graph = nullptr;
-  int64_t cur_pos = 0, max_ctx = 0;
-
-  // Record the forward at `pos` (the first position this decoder will process).
-  bool init(model& M, int64_t first_id, int64_t pos) {
-    if (M.layers.empty()) return false;
-    max_ctx = M.layers[0].cache.max_ctx;
-    cur_pos = pos;
-    if (!hip::graph_available() || !M.fused) return false;
-    const dims& d = M.d;
-    if (!M.attn_partials) {
-      M.attn_partials_bytes = hip::attn_partials_bytes(d.n_q_heads, d.n_kv_heads, max_ctx, d.head_dim);
-      M.attn_partials = hip::alloc_device(M.attn_partials_bytes);
-      if (!M.attn_partials) return false;
-    }
-    d_pos = hip::alloc(4, nullptr);
-    if (!d_pos) return false;
-    if (!stage_embed(M, first_id)) return false;
-    hip::upload_u32(d_pos, (unsigned)pos);
-    // warm run: real launches (they also size the library's scratch); it advances d_pos
-    // and writes cache row pos, which the first recorded step rewrites identically
-    if (!run_layers(M, M.s.embedb, pos, nullptr, d_pos)) return false;
-    hip::flush();
-    hip::upload_u32(d_pos, (unsigned)pos);
-    if (!hip::capture_begin()) return false;
-    const bool ok = run_layers(M, M.s.embedb, pos, nullptr, d_pos);  // recorded, not executed
-    graph = hip::capture_end();
-    if (!ok && graph) { hip::graph_destroy(graph); graph = nullptr; }
-    return graph != nullptr;
-  }
-  // Feed token `id` at the current position without reading a token back.
-  bool feed(model& M, int64_t id) {
-    if (cur_pos >= max_ctx || !stage_embed(M, id)) return false;
-    bool ok;
-    if (graph) ok = hip::graph_launch(graph);
-    else ok = run_layers(M, M.s.embedb, cur_pos);
-    cur_pos++;
-    return ok;
-  }
-  // One decode step: feed + greedy token (-1 when the cache is full or a launch failed).
-  int64_t step(model& M, int64_t id) {
-    if (!feed(M, id)) return -1;
-    int64_t idx = -1;
-    return hip::argmax(M.s.logitsb, M.d.vocab, &idx) ? idx : -1;
-  }
-  // Replays advance only the device counter; bring the host cache position up to date
-  // before switching to a host-position call.
-  void sync_host_pos(model& M) const {
-    if (graph) set_cache_pos(M, cur_pos);
-  }
-  bool ok() const { return graph != nullptr; }
-  void destroy() {
-    if (graph) hip::graph_destroy(graph);
-    if (d_pos) hip::release(d_pos, 0, nullptr);
-    graph = nullptr;
-    d_pos = nullptr;
-  }
-};
+using captured_step = loops::captured_step<model>;
+using greedy_loop = loops::greedy_loop<model>;
+using captured_decoder = loops::captured_decoder<model>;
+using loops::logits;
+using loops::prefill;
+using loops::step_greedy;
 
 }  // namespace qwen
 }  // namespace tl

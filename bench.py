@@ -540,8 +540,101 @@ def prefill_7b(lib, rounds=3):
     }
 
 
+# Lusadra layers of three sizes, and a Qwen2.5-architecture model of about the same weights per layer.
+# window: keys a position sees; the Qwen step and chunk run at a context of the same number of keys, and
+# at 4096.
+LUSADRA_SIZES = {
+    "small": dict(layers=12, vocab=32000, width=896, left=(14, 2, 64, 512), right=(7, 64, 128), ff=4864,
+                  qwen=dict(n_q_heads=14, n_kv_heads=2, head_dim=64, ff=4864)),
+    "medium": dict(layers=8, vocab=32000, width=2048, left=(16, 4, 128, 1024), right=(16, 64, 128), ff=8192,
+                   qwen=dict(n_q_heads=16, n_kv_heads=4, head_dim=128, ff=8192)),
+    "large": dict(layers=4, vocab=32000, width=3584, left=(28, 4, 128, 1024), right=(28, 64, 128), ff=18944,
+                  qwen=dict(n_q_heads=28, n_kv_heads=4, head_dim=128, ff=18944)),
+}
+
+
+def lusadra_config(z):
+    H, G, D, window = z["left"]
+    h, d, v = z["right"]
+    layer = {"type": "parallel",
+             "mixer": {"left": {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "mask": {"size": window},
+                                "scale": D ** -0.5, "q_temp": {"coef": 0.1, "every": 1024}},
+                       "right": {"heads": h, "dim": d, "vdim": v, "tau": 16.0}, "left_scale": 0.7, "right_scale": 0.7},
+             "mlp": {"kind": "dense", "ff": z["ff"]}}
+    return {"architecture": "Lusadra", "vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-6},
+            "layers": [layer] * z["layers"], "loop": None}
+
+
+def bench_lusadra(lib, steps, only=None):
+    """Decode step (hipGraph replay at position 4095) and 512-token prompt chunk (at position 3584) of the
+    Lusadra sizes above beside the Qwen2.5-architecture model of the same width, bf16 weights both."""
+    qwen = importlib.import_module("cpp-tensorlib_amd.qwen")
+    Model = importlib.import_module("cpp-tensorlib_amd.model").Model
+    T, pos = 512, 4095
+    ids = np.random.default_rng(5).integers(0, 32000, T)
+    e0, e1 = lib.event(), lib.event()
+
+    def best_ms(call, n, rounds=4):
+        call()
+        ms = []
+        for _ in range(rounds):
+            lib.record(e0)
+            for _ in range(n):
+                call()
+            lib.record(e1)
+            ms.append(lib.elapsed_ms(e0, e1) / n)
+        return min(ms)
+
+    out = {}
+    for name, z in LUSADRA_SIZES.items():
+        if only and name != only:
+            continue
+        H, G, D, window = z["left"]
+        h, d, v = z["right"]
+        E, n = z["width"], z["layers"]
+        per_layer = E * (3 * H * D + G * D + 2 * h * d + 3 * h * v + 16 + 2 * z["ff"])
+        m = Model.random_lusadra(lusadra_config(z), seed=1, rank=16, max_ctx=8192)
+        m.stage_chunk(ids)
+        for p0 in range(0, 3584, T):
+            m.chunk_layers(T, p0)
+        chunk = best_ms(lambda: m.chunk_layers(T, 3584), 2)
+        m.chunk_layers(T - 1, 3584)
+        m.capture_step(11, pos)
+        step = best_ms(m.replay_step, steps)
+        m.close()
+        state = n * (2 * h * d * v * 4 + G * min(window, pos + 1) * D * 4)
+        q = z["qwen"]
+        g = qwen.QwenGPU(dict(n_layers=n, hidden=E, vocab=z["vocab"], max_ctx=8192, eps=1e-6, rope_base=1e6, **q))
+        g.set_random(1, fmt="bf16")
+        g.fill_cache_random(4096, 2)
+        q_layer = E * ((2 * q["n_q_heads"] + 2 * q["n_kv_heads"]) * q["head_dim"] + 3 * q["ff"])
+        beside = {}
+        for ctx in sorted({window, 4096}):
+            g.step(11, ctx - 1)
+            g.capture(11, ctx - 1)
+            beside["decode_ms_ctx_%d" % ctx] = round(best_ms(g.replay, steps), 4)
+        g.stage_chunk(ids)
+        for p0 in (window - T if window >= T else 0, 3584):
+            beside["chunk_ms_pos0_%d" % p0] = round(best_ms(lambda: g.prefill_layers(T, p0), 2), 3)
+        g.close()
+        head = E * z["vocab"]
+        rate = lambda params, ms: round((2 * (n * params + head)) / ms / 1e6, 1)
+        flops = lambda params, ms: round(2.0 * T * n * params / ms / 1e9, 1)
+        out[name] = {
+            "layers": n, "width": E, "window": window, "weights_per_layer": per_layer, "qwen_weights_per_layer": q_layer,
+            "decode_ms": round(step, 4), "decode_tok_s": round(1e3 / step, 1), "decode_weight_GB/s": rate(per_layer, step),
+            "decode_state_bytes": state, "chunk_ms": round(chunk, 3), "prefill_tok_s": round(T / chunk * 1e3, 1),
+            "chunk_TFLOP/s": flops(per_layer, chunk),
+            "qwen": dict(beside, **{"decode_weight_GB/s_ctx_window": rate(q_layer, beside["decode_ms_ctx_%d" % window]),
+                                    "chunk_TFLOP/s_pos0_3584": flops(q_layer, beside["chunk_ms_pos0_3584"])})}
+    return out
+
+
 def main():
     ap = argparse.ArgumentParser()
+    ap.add_argument("--design", default="", choices=["", "lusadra"],
+                    help="instead of the headline workload: decode and prefill of this model design at several sizes")
+    ap.add_argument("--size", default="", choices=[""] + list(LUSADRA_SIZES), help="with --design: one size only")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=20)
     ap.add_argument("--warmup", type=int, default=3)
@@ -567,6 +660,14 @@ def main():
 
     pkg = importlib.import_module("cpp-tensorlib_amd")
     lib = pkg.load()                      # raises when the HIP library or the GPU is missing
+    if a.design:
+        res = bench_lusadra(lib, a.steps, a.size or None)
+        last = res[list(res)[-1]]
+        print(json.dumps({"metric": "lusadra_decode_tok_s", "value": last["decode_tok_s"], "unit": "tokens/s", "n_gpus": 1,
+                          "steps": a.steps, "warmup": a.warmup, "ms_per_step": last["decode_ms"], "higher_is_better": True,
+                          "scaling": "weak", "vs_baseline": None, "dtype": "bf16 weights, f32 activations",
+                          "data": "synthetic, random weights", "config": {"model": "Lusadra, " + list(res)[-1], "sizes": res}}))
+        return
 
     # ---- device-resident inputs: a ring of weight copies per shape -----------------
     def make_ring(N, K, wseed, xseed):

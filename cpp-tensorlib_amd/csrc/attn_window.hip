@@ -18,6 +18,7 @@
 namespace tlhip {
 
 typedef float f32x16 __attribute__((ext_vector_type(16)));
+typedef float f32x4 __attribute__((ext_vector_type(4)));
 
 template <int D, int NW>
 struct WindowLds {
@@ -26,13 +27,27 @@ struct WindowLds {
   static constexpr size_t kBytes = (size_t)((1 + NW) * kRegion + NW * 64) * sizeof(float);
 };
 
+// The 32 key rows of a tile into registers, 16 bytes per lane and load; rows at or past kend are clamped
+// to the last one (masked when used).
+template <int D>
+__device__ __forceinline__ void window_tile(f32x4 (&k)[D / 8], const float* __restrict__ ring, int tile, int kend, int R,
+                                            int lane) {
+  const float* base = ring + (size_t)((tile * 32) % R) * D;
+  const int last = kend - 1 - tile * 32;
+#pragma unroll
+  for (int i = 0; i < D / 8; i++) {
+    const int slot = lane + 64 * i, key = slot / (D / 4), c4 = slot % (D / 4);
+    k[i] = *reinterpret_cast<const f32x4*>(base + (size_t)min(key, last) * D + 4 * c4);
+  }
+}
+
 template <int D, int NW>
 __global__ __launch_bounds__(64 * NW, 1) void window_chunk_kernel(const float* __restrict__ u, int64_t ldu,
                                                                  float* __restrict__ y, int64_t ldy,
                                                                  const tlhip_window_attn a, int T, int pos0) {
   using L = WindowLds<D, NW>;
   constexpr int KS = L::KS, NT = 64 * NW;
-  constexpr int kLoads = 32 * D / 4 / 64;
+  constexpr int kLoads = D / 8;
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int l31 = lane & 31, hi = lane >> 5;
@@ -46,24 +61,15 @@ __global__ __launch_bounds__(64 * NW, 1) void window_chunk_kernel(const float* _
   const int kend = min(pos0 + p0 + 32, pos0 + T);         // keys of this block end here
   const int kt0 = max(0, pos0 + p0 - window + 1) >> 5, kt1 = (kend + 31) >> 5;
 
-  for (int s = tid; s < 32 * D; s += NT) {   // queries times their temperature (rows beyond T clamped, never stored)
-    const int r = s / D, d = s % D, t = min(p0 + r, T - 1);
-    const float v = d < dim ? u[(size_t)t * ldu + a.q_off + (size_t)h * dim + d] : 0.f;
-    Qs[r * KS + d] = v * query_temperature(pos0 + t, a.temp_coef, a.temp_every);
+  for (int r = wave; r < 32; r += NW) {      // queries times their temperature (rows beyond T clamped, never stored)
+    const int t = min(p0 + r, T - 1);
+    const float temp = query_temperature(pos0 + t, a.temp_coef, a.temp_every);
+    const float* q = u + (size_t)t * ldu + a.q_off + (size_t)h * dim;
+    for (int d = lane; d < D; d += 64) Qs[r * KS + d] = d < dim ? q[d] * temp : 0.f;
   }
 
-  float4 kreg[kLoads];
-  const auto request = [&](int tile) {       // rows at or past kend are clamped to the last one, masked when used
-    tile = min(tile, kt1 - 1);
-    const float* base = ring + (size_t)((tile * 32) % R) * D;
-    const int last = kend - 1 - tile * 32;
-#pragma unroll
-    for (int i = 0; i < kLoads; i++) {
-      const int slot = lane + 64 * i, key = slot / (D / 4), c4 = slot % (D / 4);
-      kreg[i] = *reinterpret_cast<const float4*>(base + (size_t)min(key, last) * D + 4 * c4);
-    }
-  };
-  request(kt0 + wave);
+  f32x4 kreg[kLoads];
+  window_tile<D>(kreg, ring, min(kt0 + wave, kt1 - 1), kend, R, lane);
   __syncthreads();
 
   f32x16 o[D / 32];
@@ -78,9 +84,9 @@ __global__ __launch_bounds__(64 * NW, 1) void window_chunk_kernel(const float* _
 #pragma unroll
     for (int i = 0; i < kLoads; i++) {
       const int slot = lane + 64 * i, key = slot / (D / 4), c4 = slot % (D / 4);
-      *reinterpret_cast<float4*>(K + key * KS + 4 * c4) = kreg[i];
+      *reinterpret_cast<f32x4*>(K + key * KS + 4 * c4) = kreg[i];
     }
-    request(kt + NW);
+    window_tile<D>(kreg, ring, min(kt + NW, kt1 - 1), kend, R, lane);
     f32x16 s;
 #pragma unroll
     for (int v = 0; v < 16; v++) s[v] = 0.f;
@@ -104,12 +110,12 @@ __global__ __launch_bounds__(64 * NW, 1) void window_chunk_kernel(const float* _
     const LanePair mp = swap32(mx, mx);
     mx = fmaxf(mp.first, mp.second);
     const float ref = mx == -INFINITY ? 0.f : mx;
-    const float corr = exp2f(m - ref);
+    const float corr = exp2_native(m - ref);
     m = mx;
     float ps = 0.f;
 #pragma unroll
     for (int v = 0; v < 16; v++) {
-      s[v] = exp2f(s[v] - ref);
+      s[v] = exp2_native(s[v] - ref);
       ps += s[v];
     }
     lsum = lsum * corr + ps;                              // this half's keys; the halves meet at the end
@@ -143,7 +149,7 @@ __global__ __launch_bounds__(64 * NW, 1) void window_chunk_kernel(const float* _
 #pragma unroll
   for (int w = 0; w < NW; w++) {
     const float mw = stat[w * 64 + row];
-    f[w] = mw == -INFINITY ? 0.f : exp2f(mw - M);
+    f[w] = mw == -INFINITY ? 0.f : exp2_native(mw - M);
     Ls = fmaf(f[w], stat[w * 64 + 32 + row], Ls);
   }
   const float inv = a.out_scale / Ls;

@@ -13,6 +13,10 @@ namespace tlhip {
 
 constexpr float kLog2e = 1.4426950408889634f;
 
+// v_exp_f32 / v_log_f32 as they are: arguments here never need the library forms' denormal handling
+__device__ __forceinline__ float exp2_native(float x) { return __builtin_amdgcn_exp2f(x); }
+__device__ __forceinline__ float log2_native(float x) { return __builtin_amdgcn_logf(x); }
+
 // Query multiplier at position p.
 __device__ __forceinline__ float query_temperature(int p, float coef, float every) {
   if (every <= 0.f) return 1.f;
@@ -140,14 +144,14 @@ __device__ __forceinline__ void window_step_block(const tlhip_window_attn& a, co
         mn = fmaxf(mn, s[i]);
       }
       const float ref = mn == -INFINITY ? 0.f : mn;
-      const float corr = exp2f(m[h] - ref);
+      const float corr = exp2_native(m[h] - ref);
       m[h] = mn;
       l[h] *= corr;
 #pragma unroll
       for (int f = 0; f < NF; f++) { acc[h][f].x *= corr; acc[h][f].y *= corr; acc[h][f].z *= corr; acc[h][f].w *= corr; }
 #pragma unroll
       for (int i = 0; i < KB; i++) {
-        const float p = exp2f(s[i] - ref);
+        const float p = exp2_native(s[i] - ref);
         l[h] += p;
 #pragma unroll
         for (int f = 0; f < NF; f++) {
@@ -171,7 +175,7 @@ __device__ __forceinline__ void window_step_block(const tlhip_window_attn& a, co
   for (int h = 0; h < NQ; h++) {
     float M = fmaxf(m[h], __shfl_xor(m[h], 16, kWave));
     M = fmaxf(M, __shfl_xor(M, 32, kWave));
-    const float f0 = m[h] == -INFINITY ? 0.f : exp2f(m[h] - M);
+    const float f0 = m[h] == -INFINITY ? 0.f : exp2_native(m[h] - M);
     const auto rows = [&](float v) {
       v *= f0;
       v += __shfl_xor(v, 16, kWave);
@@ -196,7 +200,7 @@ __device__ __forceinline__ void window_step_block(const tlhip_window_attn& a, co
 #pragma unroll
     for (int w = 0; w < 8; w++) {
       const float* p = wl + (w * NQ + h) * WS;
-      const float f = p[0] == -INFINITY ? 0.f : exp2f(p[0] - M);
+      const float f = p[0] == -INFINITY ? 0.f : exp2_native(p[0] - M);
       L = fmaf(f, p[1], L);
       o = fmaf(f, p[2 + d], o);
     }
@@ -227,7 +231,7 @@ __device__ __forceinline__ void window_merge_head(const tlhip_window_attn& a, co
     float L = 0.f, o = 0.f;
     for (int s = 0; s < S; s++) {
       const float* ps = p + (size_t)s * (ld + 2);
-      const float f = ps[0] == -INFINITY ? 0.f : exp2f(ps[0] - M);
+      const float f = ps[0] == -INFINITY ? 0.f : exp2_native(ps[0] - M);
       L = fmaf(f, ps[1], L);
       o = fmaf(f, ps[2 + d], o);
     }

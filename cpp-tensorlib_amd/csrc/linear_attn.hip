@@ -17,19 +17,20 @@
 // All products run on the fp32 matrix pipe (v_mfma_f32_16x16x4_f32: exact f32 products, fp32 sums).
 #include "linear_attn.hpp"
 
+#include <algorithm>
+
 namespace tlhip {
 
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 __device__ __forceinline__ f32x4 mfma16(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
 
 constexpr float kFastRange = 96.f;
-constexpr int kVSlice = 64;        // value columns of one block of linear_piece_kernel
 
 // Scratch of a call, per head and piece: decay products [dp], state term [dp][vp]; per head and
 // token: decayed query [dp], inner output [vp]. dp, vp: dim and vdim rounded up to 16.
 struct PieceBuf {
   float *dec, *st, *qd, *oi;
-  int C, np, dp, vp;               // tokens per piece, pieces
+  int C, np, dp, vp, vs;           // tokens per piece, pieces; vs: value columns of one block of linear_piece_kernel
 };
 
 // Block (piece, head, value slice) of 512 threads.
@@ -38,10 +39,10 @@ __global__ __launch_bounds__(512) void linear_piece_kernel(const float* __restri
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int tid = threadIdx.x, lane = tid & 63, l15 = lane & 15, lg = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int piece = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * kVSlice;
+  const int piece = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * pb.vs;
   const int C = pb.C, dp = pb.dp, vp = pb.vp, dim = (int)a.dim, vdim = (int)a.vdim;
-  const int NB = C / 16, QS = dp + 4, nv = min(kVSlice, vp - v0);
-  constexpr int VS = kVSlice + 4;
+  const int NB = C / 16, QS = dp + 4, nv = min(pb.vs, vp - v0);
+  const int VS = pb.vs + 4;
   const int AS = C + 4;
   float* Q = lds;                      // [C][QS] q, then Q'
   float* K = Q + C * QS;               // [C][QS] k, then K'
@@ -54,22 +55,46 @@ __global__ __launch_bounds__(512) void linear_piece_kernel(const float* __restri
   const float inv_tau = 1.0f / a.tau;
 
   if (tid < NB) slow[tid] = 0;
-  for (int i = tid; i < C * dp; i += 512) {
-    const int t = i / dp, d = i - t * dp;
-    float q = 0.f, k = 0.f, lg2 = 0.f;
-    if (t < nt && d < dim) {
-      const float* row = u + (size_t)(t0 + t) * ldu;
-      q = row[a.q_off + h * dim + d] * a.q_scale;
-      k = row[a.k_off + h * dim + d];
-      lg2 = log2_decay(decay_logit(a, row + a.low_off, h * dim + d), inv_tau);
+  // decay logits: Z = low A2^T in 16 x 16 tiles, and their logs (bias, sigmoid, 1/tau) in Lg
+  {
+    const int rank = (int)a.rank;
+    const uint16_t* a2 = static_cast<const uint16_t*>(a.a2) + (size_t)h * dim * rank;
+    const float* bias = static_cast<const float*>(a.bias) + h * dim;
+    for (int tile = wave; tile < NB * (dp / 16); tile += 8) {
+      const int tt = tile % NB, d = 16 * (tile / NB) + l15, t = 16 * tt + l15;
+      const float* low = u + (size_t)(t0 + min(t, nt - 1)) * ldu + a.low_off;
+      const uint16_t* w = a2 + (size_t)min(d, dim - 1) * rank;
+      f32x4 z = {0.f, 0.f, 0.f, 0.f};
+      for (int r0 = 0; r0 < rank; r0 += 16) {
+        float x[4], y[4];
+#pragma unroll
+        for (int j = 0; j < 4; j++) {
+          const int r = r0 + 4 * lg + j, rc = min(r, rank - 1);
+          x[j] = r < rank ? low[rc] : 0.f;
+          y[j] = __uint_as_float((uint32_t)w[rc] << 16);
+        }
+#pragma unroll
+        for (int j = 0; j < 4; j++) z = mfma16(x[j], y[j], z);
+      }
+      const float bs = bias[min(d, dim - 1)];
+#pragma unroll
+      for (int v = 0; v < 4; v++) {
+        const int tz = 16 * tt + 4 * lg + v;
+        Lg[tz * QS + d] = tz < nt && d < dim ? log2_decay(z[v] + bs, inv_tau) : 0.f;
+      }
     }
-    Q[t * QS + d] = q;
-    K[t * QS + d] = k;
-    Lg[t * QS + d] = lg2;
   }
-  for (int i = tid; i < C * kVSlice; i += 512) {
-    const int t = i / kVSlice, v = i % kVSlice;
-    V[t * VS + v] = t < nt && v0 + v < vdim ? u[(size_t)(t0 + t) * ldu + a.v_off + (int64_t)h * vdim + v0 + v] : 0.f;
+  for (int t = wave; t < C; t += 8) {
+    const float* row = u + (size_t)(t0 + min(t, nt - 1)) * ldu;
+    const float *q = row + a.q_off + h * dim, *k = row + a.k_off + h * dim, *v = row + a.v_off + (int64_t)h * vdim + v0;
+    for (int d = lane; d < dp; d += 64) {
+      const bool live = t < nt && d < dim;
+      const int dc = min(d, dim - 1);
+      const float qd = q[dc], kd = k[dc];
+      Q[t * QS + d] = live ? qd * a.q_scale : 0.f;
+      K[t * QS + d] = live ? kd : 0.f;
+    }
+    for (int c = lane; c < pb.vs; c += 64) V[t * VS + c] = t < nt && v0 + c < vdim ? v[c] : 0.f;
   }
   __syncthreads();
   for (int i = tid; i < NB * dp; i += 512) {         // running sums of the logs inside each block
@@ -90,17 +115,17 @@ __global__ __launch_bounds__(512) void linear_piece_kernel(const float* __restri
       const int t = 16 * b + tid / 16, s = 16 * b + tid % 16;
       float acc = 0.f;
       if (s <= t)
-        for (int d = 0; d < dim; d++) acc = fmaf(Q[t * QS + d] * K[s * QS + d], exp2f(Lg[t * QS + d] - Lg[s * QS + d]), acc);
+        for (int d = 0; d < dim; d++) acc = fmaf(Q[t * QS + d] * K[s * QS + d], exp2_native(Lg[t * QS + d] - Lg[s * QS + d]), acc);
       A[t * AS + s] = acc;
     }
   }
   __syncthreads();
-  for (int i = tid; i < C * dp; i += 512) {
-    const int t = i / dp, d = i - t * dp, b = t >> 4;
-    const float L = Lg[t * QS + d];
-    Q[t * QS + d] *= exp2f(L);
-    K[t * QS + d] *= exp2f(tot[b * dp + d] - L);
-  }
+  for (int t = wave; t < C; t += 8)
+    for (int d = lane; d < dp; d += 64) {
+      const float L = Lg[t * QS + d];
+      Q[t * QS + d] *= exp2_native(L);
+      K[t * QS + d] *= exp2_native(tot[(t >> 4) * dp + d] - L);
+    }
   __syncthreads();
   // A[t][s]: 16 x 16 tiles on and below the diagonal, dealt over the wavefronts
   for (int tile = wave; tile < NB * (NB + 1) / 2; tile += 8) {
@@ -114,14 +139,14 @@ __global__ __launch_bounds__(512) void linear_piece_kernel(const float* __restri
       const float4 k = *reinterpret_cast<const float4*>(K + (16 * j + l15) * QS + d);
       if (i == j) {
         const float* tp = tot + i * dp + d;
-        q.x *= exp2f(-tp[0]); q.y *= exp2f(-tp[1]); q.z *= exp2f(-tp[2]); q.w *= exp2f(-tp[3]);
+        q.x *= exp2_native(-tp[0]); q.y *= exp2_native(-tp[1]); q.z *= exp2_native(-tp[2]); q.w *= exp2_native(-tp[3]);
       } else if (i > j + 1) {
         float4 e = make_float4(0.f, 0.f, 0.f, 0.f);
         for (int m = j + 1; m < i; m++) {
           const float* tp = tot + m * dp + d;
           e.x += tp[0]; e.y += tp[1]; e.z += tp[2]; e.w += tp[3];
         }
-        q.x *= exp2f(e.x); q.y *= exp2f(e.y); q.z *= exp2f(e.z); q.w *= exp2f(e.w);
+        q.x *= exp2_native(e.x); q.y *= exp2_native(e.y); q.z *= exp2_native(e.z); q.w *= exp2_native(e.w);
       }
       acc = mfma16(q.x, k.x, acc);
       acc = mfma16(q.y, k.y, acc);
@@ -136,16 +161,16 @@ __global__ __launch_bounds__(512) void linear_piece_kernel(const float* __restri
   }
   const size_t hp = (size_t)h * pb.np + piece;
   if (blockIdx.z == 0) {                             // decayed queries and the piece's decay products
-    for (int i = tid; i < C * dp; i += 512) {
-      const int t = i / dp, d = i - t * dp, b = t >> 4;
-      float e = 0.f;
-      for (int m = 0; m < b; m++) e += tot[m * dp + d];
-      pb.qd[(hp * C + t) * dp + d] = Q[t * QS + d] * exp2f(e);
-    }
+    for (int t = wave; t < C; t += 8)
+      for (int d = lane; d < dp; d += 64) {
+        float e = 0.f;
+        for (int m = 0; m < t >> 4; m++) e += tot[m * dp + d];
+        pb.qd[(hp * C + t) * dp + d] = Q[t * QS + d] * exp2_native(e);
+      }
     for (int d = tid; d < dp; d += 512) {
       float e = 0.f;
       for (int m = 0; m < NB; m++) e += tot[m * dp + d];
-      pb.dec[hp * dp + d] = exp2f(e);
+      pb.dec[hp * dp + d] = exp2_native(e);
     }
   }
   // state term: sum over s of K'_sd 2^(totals after s's block) V_sv
@@ -154,7 +179,7 @@ __global__ __launch_bounds__(512) void linear_piece_kernel(const float* __restri
     f32x4 acc = {0.f, 0.f, 0.f, 0.f};
     float e = 0.f;
     for (int b = NB - 1; b >= 0; b--) {
-      const float w = exp2f(e);
+      const float w = exp2_native(e);
 #pragma unroll
       for (int j = 0; j < 4; j++) {
         const int s = 16 * b + 4 * lg + j;
@@ -264,8 +289,8 @@ __global__ __launch_bounds__(512) void linear_out_kernel(const float* __restrict
   }
 }
 
-static size_t piece_lds(int C, int dp) {
-  return (size_t)(3 * C * (dp + 4) + C * (kVSlice + 4) + C * (C + 4) + (C / 16) * dp + 16) * sizeof(float);
+static size_t piece_lds(int C, int dp, int vs) {
+  return (size_t)(3 * C * (dp + 4) + C * (vs + 4) + C * (C + 4) + (C / 16) * dp + 16) * sizeof(float);
 }
 
 }  // namespace tlhip
@@ -285,8 +310,10 @@ int tlhip_linear_attn_chunk(const void* u, int64_t ldu, void* y, int64_t ldy, co
   pb.dp = (int)(la->dim + 15) / 16 * 16;
   pb.vp = (int)(la->vdim + 15) / 16 * 16;
   pb.C = 64;
-  while (pb.C > 16 && (piece_lds(pb.C, pb.dp) > (size_t)c.lds_per_cu || pb.C / 2 >= T)) pb.C /= 2;
-  const size_t lds1 = piece_lds(pb.C, pb.dp);
+  while (pb.C > 16 && (piece_lds(pb.C, pb.dp, 64) > (size_t)c.lds_per_cu || pb.C / 2 >= T)) pb.C /= 2;
+  pb.vs = std::min(pb.vp, 128);        // every slice of values repeats the work on queries and keys
+  if (piece_lds(pb.C, pb.dp, pb.vs) > (size_t)c.lds_per_cu) pb.vs = 64;
+  const size_t lds1 = piece_lds(pb.C, pb.dp, pb.vs);
   const int mt = pb.C >= 32 ? 2 : 1;
   const size_t lds3 = (size_t)16 * mt * (pb.vp + 4) * sizeof(float);
   if (lds1 > (size_t)c.lds_per_cu || lds3 > (size_t)c.lds_per_cu)
@@ -303,7 +330,7 @@ int tlhip_linear_attn_chunk(const void* u, int64_t ldu, void* y, int64_t ldy, co
   const float* pu = static_cast<const float*>(u);
   hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(linear_piece_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds1);
   if (e != hipSuccess) return hip_fail(e, "hipFuncSetAttribute(LDS)");
-  hipLaunchKernelGGL(linear_piece_kernel, dim3((unsigned)pb.np, (unsigned)la->heads, (unsigned)((pb.vp + kVSlice - 1) / kVSlice)),
+  hipLaunchKernelGGL(linear_piece_kernel, dim3((unsigned)pb.np, (unsigned)la->heads, (unsigned)((pb.vp + pb.vs - 1) / pb.vs)),
                      dim3(512), lds1, c.stream, pu, ldu, *la, (int)T, pb);
   const size_t ns = (size_t)la->heads * pb.dp * (pb.vp / 4);
   hipLaunchKernelGGL(linear_scan_kernel, dim3((unsigned)((ns + 255) / 256)), dim3(256), 0, c.stream, *la, (int)T, (int)pos0, pb);

@@ -10,10 +10,12 @@
 
 namespace tlhip {
 
-// log2 of sigmoid(z)^(1/tau) = -softplus(-z) log2(e) / tau
+// log2 of sigmoid(z)^(1/tau) = -log2(1 + e^-z) / tau, from e = e^-|z| <= 1. log2(1 + e) keeps e's
+// relative accuracy down to the smallest e: with w = fl(1 + e), log2(w) e / (w - 1) undoes w's rounding.
 __device__ __forceinline__ float log2_decay(float z, float inv_tau) {
-  const float sp = fmaxf(-z, 0.f) + log1pf(expf(-fabsf(z)));
-  return -sp * kLog2e * inv_tau;
+  const float e = exp2_native(-fabsf(z) * kLog2e), w = 1.f + e;
+  const float l = w == 1.f ? e * kLog2e : log2_native(w) * (e / (w - 1.f));
+  return -(fmaxf(-z, 0.f) * kLog2e + l) * inv_tau;
 }
 // z of channel `ch` (head * dim + d): the low-rank product and its bias
 __device__ __forceinline__ float decay_logit(const tlhip_linear_attn& a, const float* __restrict__ low, int ch) {
@@ -53,7 +55,7 @@ __device__ __forceinline__ void linear_step_block(const tlhip_linear_attn& a, co
     const int ch = h * dim + d;
     qs[d] = u[a.q_off + ch] * a.q_scale;
     ks[d] = u[a.k_off + ch];
-    al[d] = exp2f(log2_decay(decay_logit(a, u + a.low_off, ch), 1.0f / a.tau));
+    al[d] = exp2_native(log2_decay(decay_logit(a, u + a.low_off, ch), 1.0f / a.tau));
   }
   for (int v = tid; v < ld; v += 512) vs[v] = v < vdim ? u[a.v_off + (int64_t)h * vdim + v] : 0.f;
   __syncthreads();

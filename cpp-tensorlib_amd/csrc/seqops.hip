@@ -40,10 +40,15 @@ __global__ __launch_bounds__(256) void gather_rows_kernel(const float* __restric
   if (c < n) out[(size_t)blockIdx.y * n + c] = src[(size_t)r * n + c];
 }
 
+// L > 0: rows held in registers (polynorm_row), else any row
+template <int L>
 __global__ __launch_bounds__(512) void polynorm_rows_kernel(const float* __restrict__ u, int64_t ldu, float* __restrict__ y,
                                                             int64_t ldy, const tlhip_polynorm p) {
   __shared__ float red[24];
-  polynorm_block<512>(p, u + (size_t)blockIdx.x * ldu + p.z_off, y + (size_t)blockIdx.x * ldy + p.y_off, 0, (int)p.ff, red);
+  const float* z = u + (size_t)blockIdx.x * ldu + p.z_off;
+  float* o = y + (size_t)blockIdx.x * ldy + p.y_off;
+  if constexpr (L > 0) polynorm_row<512, L>(p, z, o, red);
+  else polynorm_block<512>(p, z, o, 0, (int)p.ff, red);
 }
 
 }  // namespace tlhip
@@ -89,8 +94,12 @@ int tlhip_polynorm_rows(const void* u, int64_t ldu, void* y, int64_t ldy, const 
   if (!u || !y || !pn || !aligned16(u) || ldu <= 0 || ldu % 4 || ldy <= 0 || T <= 0 || T > (1 << 30))
     return fail(TLHIP_EINVAL, "tlhip_polynorm_rows: bad operands");
   if (int rc = check_polynorm(pn, "tlhip_polynorm_rows")) return rc;
-  polynorm_rows_kernel<<<dim3((unsigned)T), dim3(512), 0, ctx().stream>>>(static_cast<const float*>(u), ldu, static_cast<float*>(y),
-                                                                         ldy, *pn);
+  const bool vec = pn->ff % 4 == 0 && ldy % 4 == 0 && pn->y_off % 4 == 0 && aligned16(y);
+  const int64_t per = (pn->ff / 4 + 511) / 512;
+  auto fn = !vec || per > 12 ? polynorm_rows_kernel<0> : per <= 3 ? polynorm_rows_kernel<3> : per <= 6 ? polynorm_rows_kernel<6>
+                                                       : polynorm_rows_kernel<12>;
+  hipLaunchKernelGGL(fn, dim3((unsigned)T), dim3(512), 0, ctx().stream, static_cast<const float*>(u), ldu, static_cast<float*>(y), ldy,
+                     *pn);
   TLHIP_CHECK_LAUNCH(TLHIP_C_POLYNORM);
 }
 

@@ -129,7 +129,7 @@ SIGNATURES = {
     "tlhip_mix_partials_bytes": (i64, [P]),
     "tlhip_mix_step": (cint, [P, P, P, P, P, i64, P, P, i64]),
     "tlhip_window_fill": (cint, [P, i64, P, i64, i64]),
-    "tlhip_window_attn_chunk": (cint, [P, i64, P, i64, P, i64, i64]),
+    "tlhip_window_attn_chunk": (cint, [P, i64, P, i64, P, i64, i64, cint]),
     "tlhip_linear_attn_chunk": (cint, [P, i64, P, i64, P, i64, i64]),
     "tlhip_polynorm_rows": (cint, [P, i64, P, i64, P, i64]),
     "tlhip_embed_sinusoid": (cint, [P, P, P, i64, i64, i64, i64, i64, P]),
@@ -585,9 +585,9 @@ class TlHip:
     def mix_partials_bytes(self, at):
         return int(self.c.tlhip_mix_partials_bytes(C.byref(at)))
 
-    def window_attn_chunk(self, u, ldu, y, ldy, at, T, pos0):
+    def window_attn_chunk(self, u, ldu, y, ldy, at, T, pos0, exact=True):
         self._chk(self.c.tlhip_window_fill(u.ptr, ldu, C.byref(at), T, pos0))
-        self._chk(self.c.tlhip_window_attn_chunk(u.ptr, ldu, y.ptr, ldy, C.byref(at), T, pos0))
+        self._chk(self.c.tlhip_window_attn_chunk(u.ptr, ldu, y.ptr, ldy, C.byref(at), T, pos0, int(exact)))
 
     def linear_attn_chunk(self, u, ldu, y, ldy, la, T, pos0):
         self._chk(self.c.tlhip_linear_attn_chunk(u.ptr, ldu, y.ptr, ldy, C.byref(la), T, pos0))

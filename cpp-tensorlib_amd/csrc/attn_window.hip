@@ -1,7 +1,7 @@
-// Prompt chunks of the sliding-window attention whose values are its keys, on the fp32 matrix pipe,
-// and the copy of a chunk's keys into the ring.
+// Prompt chunks of the sliding-window attention whose values are its keys, in two forms, and the copy of
+// a chunk's keys into the ring.
 //
-// A block owns one query head and 32 consecutive positions; its NW wavefronts deal the 32-key tiles
+// window_chunk_kernel, the exact form, runs on the fp32 matrix pipe. A block owns one query head and 32 consecutive positions; its NW wavefronts deal the 32-key tiles
 // that the window touches, each with its own running (max, sum, output) state, merged through LDS at
 // the end. v_mfma_f32_32x32x2_f32 multiplies f32 by f32 exactly. Both products are formed transposed:
 //   S^T = K Q^T : lane (l % 32) holds 16 scores of query l % 32, keys 8a + 4 (l / 32) + b in
@@ -13,7 +13,18 @@
 // is the operand of both products (rows for the first, columns for the second).
 // Tiles start at multiples of 32 positions, and the ring holds a multiple of 32 rows: a tile never
 // wraps inside the ring.
+//
+// window_terms_kernel runs on the 16-bit matrix cores: every f32 operand is cut into two bf16 terms, each
+// rounded to nearest (16 significant bits, f32's range), and a product is formed from the three term
+// pairs that hold a first term, fp32 sums. Scores, softmax and sums stay f32. A block owns one kv head:
+// its eight wavefronts are the query heads of the group (and, for small groups, consecutive runs of 32
+// positions) and share one 32-key tile, which all 512 threads cut into terms while the tile before it is
+// worked on: rows for K Q^T, and keys in the order in which the score registers hold them, as the
+// operand of K^T P^T. Tiles are dealt over S blocks so that the chip is filled; window_join_kernel
+// adds those up.
 #include "attn_window.hpp"
+
+#include <algorithm>
 
 namespace tlhip {
 
@@ -165,6 +176,284 @@ __global__ __launch_bounds__(64 * NW, 1) void window_chunk_kernel(const float* _
   }
 }
 
+// ---- two bf16 terms ------------------------------------------------------------------------------
+typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
+typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef float f32x2 __attribute__((ext_vector_type(2)));
+
+__device__ __forceinline__ void two_terms(f32x2 x, bf16x2& first, bf16x2& second) {
+  first = __builtin_convertvector(x, bf16x2);
+  const f32x2 back = __builtin_convertvector(first, f32x2);
+  f32x2 rest;
+  rest[0] = x[0] - back[0];
+  rest[1] = x[1] - back[1];
+  second = __builtin_convertvector(rest, bf16x2);
+}
+__device__ __forceinline__ f32x16 mfma_bf16(bf16x8 a, bf16x8 b, f32x16 c) {
+  return __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, b, c, 0, 0, 0);
+}
+
+struct TermPlan {
+  int gh;        // query heads of a block
+  int subs;      // blocks that share a kv head's group
+  int pt;        // runs of 32 positions of a block
+  int S;         // key splits
+};
+
+// LDS: two buffers, each K [term][32 keys][D + 8] and KT [term][key step 2][half 2][D][8 keys], bf16.
+template <int D>
+struct TermLds {
+  static constexpr int kKRow = D + 8, kK = 32 * kKRow, kT = 4 * D * 8;
+  static constexpr int kBuf = 2 * kK + 2 * kT;              // bf16 elements of one buffer
+  static constexpr size_t kBytes = (size_t)2 * kBuf * 2;
+};
+
+template <int D>
+__global__ __launch_bounds__(512, 1) void window_terms_kernel(const float* __restrict__ u, int64_t ldu, float* __restrict__ y,
+                                                             int64_t ldy, const tlhip_window_attn a, int T, int pos0,
+                                                             const TermPlan plan, float* __restrict__ acc_out,
+                                                             float* __restrict__ stat_out) {
+  using L = TermLds<D>;
+  extern __shared__ __attribute__((aligned(16))) __bf16 bl[];
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int l31 = lane & 31, hi = lane >> 5;
+  const int heads = (int)a.heads, group = heads / (int)a.kv_heads, dim = (int)a.dim, window = (int)a.window, R = (int)a.ring_rows;
+  const int kvh = blockIdx.x / plan.subs, sub = blockIdx.x % plan.subs;
+  const int hh = sub * plan.gh + wave % plan.gh, run = wave / plan.gh, h = kvh * group + hh;
+  const int b0 = (int)(gridDim.y - 1 - blockIdx.y) * 32 * plan.pt, p0 = b0 + 32 * run;
+  const bool works = hh < group && run < plan.pt && p0 < T;
+  const float* ring = static_cast<const float*>(a.ring) + (size_t)kvh * R * D;
+  const int kend = min(pos0 + b0 + 32 * plan.pt, pos0 + T);
+  const int kt0 = max(0, pos0 + b0 - window + 1) >> 5, kt1 = (kend + 31) >> 5;
+  // the tiles this wavefront's 32 queries see
+  const int wt0 = works ? max(0, pos0 + p0 - window + 1) >> 5 : 0, wt1 = works ? (min(pos0 + p0 + 32, pos0 + T) + 31) >> 5 : 0;
+
+  // staging: a thread cuts two columns of four keys
+  constexpr int kTasks = 8 * (D / 2);
+  const int kq = tid / (D / 2), d2 = 2 * (tid % (D / 2));
+  const bool stages = tid < kTasks;
+  f32x2 kreg[4];
+  const auto request = [&](f32x2 (&k)[4], int tile) {
+    tile = min(tile, kt1 - 1);
+    const float* base = ring + (size_t)((tile * 32) % R) * D + d2;
+    const int last = kend - 1 - tile * 32;
+#pragma unroll
+    for (int i = 0; i < 4; i++) k[i] = *reinterpret_cast<const f32x2*>(base + (size_t)min(4 * kq + i, last) * D);
+  };
+  const auto stage = [&](const f32x2 (&k)[4], int buf) {
+    __bf16 *K = bl + buf * L::kBuf, *KT = K + 2 * L::kK;
+    bf16x4 t0[2], t1[2];               // [column] four keys: first and second terms
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+      bf16x2 f, g;
+      two_terms(k[i], f, g);
+      *reinterpret_cast<bf16x2*>(K + (4 * kq + i) * L::kKRow + d2) = f;
+      *reinterpret_cast<bf16x2*>(K + L::kK + (4 * kq + i) * L::kKRow + d2) = g;
+      t0[0][i] = f[0]; t0[1][i] = f[1];
+      t1[0][i] = g[0]; t1[1][i] = g[1];
+    }
+    // keys 4kq .. 4kq + 3 are elements 4 (kq / 2 % 2) .. of key step kq / 4, lane half kq % 2
+    const int unit = ((kq >> 2) * 2 + (kq & 1)) * D + d2, off = 4 * ((kq >> 1) & 1);
+#pragma unroll
+    for (int c = 0; c < 2; c++) {
+      *reinterpret_cast<bf16x4*>(KT + (unit + c) * 8 + off) = t0[c];
+      *reinterpret_cast<bf16x4*>(KT + L::kT + (unit + c) * 8 + off) = t1[c];
+    }
+  };
+  int kt = kt0 + (int)blockIdx.z;
+  if (stages) request(kreg, kt);
+
+  // queries times their temperature, cut into terms: lane (hi, l31) holds columns 16s + 8hi .. + 7 of query l31
+  bf16x8 q0[D / 16], q1[D / 16];
+  {
+    const int t = min(max(p0, 0) + l31, T - 1);
+    const float temp = query_temperature(pos0 + t, a.temp_coef, a.temp_every);
+    const float* q = u + (size_t)t * ldu + a.q_off + (size_t)min(h, heads - 1) * dim;
+#pragma unroll
+    for (int s = 0; s < D / 16; s++)
+#pragma unroll
+      for (int j = 0; j < 8; j += 2) {
+        const int d = 16 * s + 8 * hi + j;
+        f32x2 x;
+        x[0] = d < dim ? q[d] * temp : 0.f;
+        x[1] = d + 1 < dim ? q[d + 1] * temp : 0.f;
+        bf16x2 f, g;
+        two_terms(x, f, g);
+        q0[s][j] = f[0]; q0[s][j + 1] = f[1];
+        q1[s][j] = g[0]; q1[s][j + 1] = g[1];
+      }
+  }
+  f32x16 o[D / 32];
+#pragma unroll
+  for (int dt = 0; dt < D / 32; dt++)
+#pragma unroll
+    for (int v = 0; v < 16; v++) o[dt][v] = 0.f;
+  float m = -INFINITY, lsum = 0.f;
+  const int qpos = pos0 + p0 + l31;
+  const float sc2 = a.scale * kLog2e, sl2 = head_slope(h, heads, a.slope_exp) * kLog2e;
+
+  if (stages && kt < kt1) stage(kreg, 0);
+  if (stages) request(kreg, kt + plan.S);
+  __syncthreads();
+  for (int buf = 0; kt < kt1; kt += plan.S, buf ^= 1) {
+    if (kt >= wt0 && kt < wt1) {
+      const __bf16 *K = bl + buf * L::kBuf, *KT = K + 2 * L::kK;
+      f32x16 s, r;                     // first x first, and the two mixed pairs
+#pragma unroll
+      for (int v = 0; v < 16; v++) { s[v] = 0.f; r[v] = 0.f; }
+#pragma unroll
+      for (int g = 0; g < D / 16; g++) {
+        const bf16x8 k0 = *reinterpret_cast<const bf16x8*>(K + l31 * L::kKRow + 16 * g + 8 * hi);
+        const bf16x8 k1 = *reinterpret_cast<const bf16x8*>(K + L::kK + l31 * L::kKRow + 16 * g + 8 * hi);
+        s = mfma_bf16(k0, q0[g], s);
+        r = mfma_bf16(k0, q1[g], r);
+        r = mfma_bf16(k1, q0[g], r);
+      }
+      const int dist0 = qpos - kt * 32 - 4 * hi;
+      float mx = m;
+#pragma unroll
+      for (int v = 0; v < 16; v++) {
+        const int dist = dist0 - (8 * (v >> 2) + (v & 3));
+        s[v] = dist >= 0 && dist < window ? (s[v] + r[v]) * sc2 - sl2 * (float)dist : -INFINITY;
+        mx = fmaxf(mx, s[v]);
+      }
+      const LanePair mp = swap32(mx, mx);
+      mx = fmaxf(mp.first, mp.second);
+      const float ref = mx == -INFINITY ? 0.f : mx;
+      if (__builtin_amdgcn_ballot_w64(mx > m)) {       // some query's maximum moved
+        const float corr = exp2_native(m - ref);
+        m = mx;
+        lsum *= corr;
+#pragma unroll
+        for (int dt = 0; dt < D / 32; dt++)
+#pragma unroll
+          for (int v = 0; v < 16; v++) o[dt][v] *= corr;
+      }
+      bf16x8 w0[2], w1[2];
+      float ps = 0.f;
+#pragma unroll
+      for (int v = 0; v < 16; v += 2) {
+        f32x2 p;
+        p[0] = exp2_native(s[v] - ref);
+        p[1] = exp2_native(s[v + 1] - ref);
+        ps += p[0] + p[1];
+        bf16x2 f, g;
+        two_terms(p, f, g);
+        w0[v >> 3][v & 7] = f[0]; w0[v >> 3][(v & 7) + 1] = f[1];
+        w1[v >> 3][v & 7] = g[0]; w1[v >> 3][(v & 7) + 1] = g[1];
+      }
+      lsum += ps;
+#pragma unroll
+      for (int st = 0; st < 2; st++)
+#pragma unroll
+        for (int dt = 0; dt < D / 32; dt++) {
+          const __bf16* p = KT + ((st * 2 + hi) * D + dt * 32 + l31) * 8;
+          const bf16x8 v0 = *reinterpret_cast<const bf16x8*>(p);
+          const bf16x8 v1 = *reinterpret_cast<const bf16x8*>(p + L::kT);
+          o[dt] = mfma_bf16(v1, w0[st], o[dt]);
+          o[dt] = mfma_bf16(v0, w1[st], o[dt]);
+          o[dt] = mfma_bf16(v0, w0[st], o[dt]);
+        }
+    }
+    // the next tile into the other buffer (last read before the barrier that ended the turn before)
+    if (stages && kt + plan.S < kt1) stage(kreg, buf ^ 1);
+    if (stages) request(kreg, kt + 2 * plan.S);
+    __syncthreads();
+  }
+  const int t = p0 + l31;
+  const LanePair lp = swap32(lsum, lsum);
+  const float Ls = lp.first + lp.second;
+  if (!works || t >= T) return;
+  if (plan.S > 1) {
+    const size_t row = ((size_t)blockIdx.z * T + t) * heads + h;
+    if (hi == 0) { stat_out[2 * row] = m; stat_out[2 * row + 1] = Ls; }
+#pragma unroll
+    for (int dt = 0; dt < D / 32; dt++)
+#pragma unroll
+      for (int q = 0; q < 4; q++)
+        *reinterpret_cast<float4*>(acc_out + row * D + dt * 32 + 8 * q + 4 * hi) =
+            make_float4(o[dt][4 * q], o[dt][4 * q + 1], o[dt][4 * q + 2], o[dt][4 * q + 3]);
+    return;
+  }
+  const float inv = a.out_scale / Ls;
+  const float* gp = u + (size_t)t * ldu + a.gate_off + (size_t)h * dim;
+  float* yp = y + (size_t)t * ldy + a.y_off + (size_t)h * dim;
+#pragma unroll
+  for (int dt = 0; dt < D / 32; dt++)
+#pragma unroll
+    for (int v = 0; v < 16; v++) {
+      const int d = dt * 32 + 8 * (v >> 2) + 4 * hi + (v & 3);
+      if (d < dim) yp[d] = o[dt][v] * inv * (a.gate_off >= 0 ? sigmoid_f(gp[d]) : 1.f);
+    }
+}
+
+// The key splits of (token, head) rows, one wavefront each -> y.
+template <int D>
+__global__ __launch_bounds__(256) void window_join_kernel(const float* __restrict__ u, int64_t ldu, float* __restrict__ y,
+                                                          int64_t ldy, const tlhip_window_attn a, int T, int S,
+                                                          const float* __restrict__ acc, const float* __restrict__ stat) {
+  const int heads = (int)a.heads, dim = (int)a.dim, lane = threadIdx.x & 63;
+  const size_t rows = (size_t)T * heads, i = (size_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (i >= rows) return;
+  const int t = (int)(i / heads), h = (int)(i % heads);
+  float M = -INFINITY;
+  for (int s = 0; s < S; s++) M = fmaxf(M, stat[2 * (s * rows + i)]);
+  float Ls = 0.f, o[(D + 63) / 64] = {};
+  for (int s = 0; s < S; s++) {
+    const size_t r = s * rows + i;
+    const float ms = stat[2 * r], f = ms == -INFINITY ? 0.f : exp2_native(ms - M);
+    Ls = fmaf(f, stat[2 * r + 1], Ls);
+#pragma unroll
+    for (int k = 0; k < (D + 63) / 64; k++) {
+      const int d = lane + 64 * k;
+      if (d < D) o[k] = fmaf(f, acc[r * D + d], o[k]);
+    }
+  }
+  const float inv = a.out_scale / Ls;
+#pragma unroll
+  for (int k = 0; k < (D + 63) / 64; k++) {
+    const int d = lane + 64 * k;
+    if (d < dim) {
+      float v = o[k] * inv;
+      if (a.gate_off >= 0) v *= sigmoid_f(u[(size_t)t * ldu + a.gate_off + (size_t)h * dim + d]);
+      y[(size_t)t * ldy + a.y_off + (size_t)h * dim + d] = v;
+    }
+  }
+}
+
+template <int D>
+static int launch_terms(const float* u, int64_t ldu, float* y, int64_t ldy, const tlhip_window_attn& a, int T, int pos0) {
+  Context& c = ctx();
+  const int group = (int)(a.heads / a.kv_heads);
+  TermPlan p{};
+  p.gh = group < 8 ? group : 8;
+  p.subs = (group + p.gh - 1) / p.gh;
+  p.pt = 8 / p.gh;
+  while (p.pt > 1 && 32 * (p.pt - 1) >= T) p.pt--;
+  const int runs = (T + 32 * p.pt - 1) / (32 * p.pt);
+  const int64_t blocks = a.kv_heads * p.subs * runs, tiles = (std::min<int64_t>(a.window, pos0 + T) + 32 * p.pt + 31) / 32;
+  p.S = (int)std::max<int64_t>(1, std::min<int64_t>({c.cus / blocks, tiles / 3, 16}));
+  float *acc = nullptr, *stat = nullptr;
+  if (p.S > 1) {
+    const size_t rows = (size_t)p.S * T * a.heads;
+    acc = static_cast<float*>(scratch(rows * (D + 2) * sizeof(float)));
+    if (!acc) return fail(TLHIP_ENOMEM, "tlhip_window_attn_chunk: no scratch");
+    stat = acc + rows * D;
+  }
+  auto fn = window_terms_kernel<D>;
+  const size_t lds = TermLds<D>::kBytes;
+  const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+  if (e != hipSuccess) return hip_fail(e, "hipFuncSetAttribute(LDS)");
+  hipLaunchKernelGGL(fn, dim3((unsigned)(a.kv_heads * p.subs), (unsigned)runs, (unsigned)p.S), dim3(512), lds, c.stream, u, ldu, y, ldy,
+                     a, T, pos0, p, acc, stat);
+  if (p.S > 1)
+    hipLaunchKernelGGL(window_join_kernel<D>, dim3((unsigned)(((size_t)T * a.heads + 3) / 4)), dim3(256), 0, c.stream, u, ldu, y, ldy, a,
+                       T, p.S, acc, stat);
+  TLHIP_CHECK_LAUNCH(TLHIP_C_WINDOW_ATTN);
+}
+
 // Keys of the chunk's tokens -> ring rows, zeros past dim.
 __global__ __launch_bounds__(256) void window_fill_kernel(const float* __restrict__ u, int64_t ldu, const tlhip_window_attn a,
                                                           int T, int pos0) {
@@ -214,12 +503,19 @@ int tlhip_window_fill(const void* u, int64_t ldu, const tlhip_window_attn* at, i
 }
 
 int tlhip_window_attn_chunk(const void* u, int64_t ldu, void* y, int64_t ldy, const tlhip_window_attn* at, int64_t T,
-                            int64_t pos0) {
+                            int64_t pos0, int exact) {
   TLHIP_REQUIRE_READY();
   if (!y || ldy <= 0) return fail(TLHIP_EINVAL, "tlhip_window_attn_chunk: bad operands");
   if (int rc = check_chunk(u, ldu, T, pos0, at, "tlhip_window_attn_chunk")) return rc;
   const float* pu = static_cast<const float*>(u);
   float* py = static_cast<float*>(y);
+  if (!exact && T >= 16) switch (at->ring_ld) {
+      case 32: return launch_terms<32>(pu, ldu, py, ldy, *at, (int)T, (int)pos0);
+      case 64: return launch_terms<64>(pu, ldu, py, ldy, *at, (int)T, (int)pos0);
+      case 96: return launch_terms<96>(pu, ldu, py, ldy, *at, (int)T, (int)pos0);
+      case 128: return launch_terms<128>(pu, ldu, py, ldy, *at, (int)T, (int)pos0);
+      default: break;                // larger heads: the exact form
+    }
   // few key tiles: more wavefronts than tiles would only add to the merge
   const bool few = at->window <= 96;
 #define TLHIP_WIN(D, NW) return launch_window<D, NW>(pu, ldu, py, ldy, *at, (int)T, (int)pos0)

@@ -32,7 +32,7 @@ extern "C" {
 
 const char* tlm_error() { return g_error.c_str(); }
 
-// exact != 0: prompt products in three exact terms; q4 != 0: int4 weights (GGUF only). NULL on error.
+// exact != 0: prompt products exact in f32; q4 != 0: int4 weights (GGUF only). NULL on error.
 void* tlm_open(const char* path, int64_t max_ctx, int64_t chunk, int exact, int q4) {
   return guarded([&]() -> void* {
     models::options o;
@@ -51,7 +51,7 @@ void* tlm_random_lusadra(const char* config, uint32_t seed, int64_t rank, int64_
   return guarded([&]() -> void* {
     auto h = std::make_unique<handle>();
     auto p = std::make_unique<models::of<lusadra::model>>(lusadra::kArchitecture, chunk);
-    p->m.prompt_f16 = !exact;
+    p->m.exact = exact != 0;
     lusadra::load_random(p->m, json::parse(config), seed, rank, max_ctx, chunk);
     h->lus = p.get();
     h->p = std::move(p);

@@ -191,7 +191,7 @@ struct api {
   int (*mix_step)(const void*, void*, const void*, const void*, const void*, int64_t, const void*, void*,
                   int64_t) = nullptr;
   int (*window_fill)(const void*, int64_t, const void*, int64_t, int64_t) = nullptr;
-  int (*window_attn_chunk)(const void*, int64_t, void*, int64_t, const void*, int64_t, int64_t) = nullptr;
+  int (*window_attn_chunk)(const void*, int64_t, void*, int64_t, const void*, int64_t, int64_t, int) = nullptr;
   int (*linear_attn_chunk)(const void*, int64_t, void*, int64_t, const void*, int64_t, int64_t) = nullptr;
   int (*polynorm_rows)(const void*, int64_t, void*, int64_t, const void*, int64_t) = nullptr;
   int (*embed_sinusoid)(const void*, const void*, void*, int64_t, int64_t, int64_t, int64_t, int64_t,
@@ -1637,12 +1637,13 @@ inline bool mix_step(void* u, void* y, const window_attn* at, const linear_attn*
   return L.sent(L.lib.mix_step(u, y, at, la, pn, pos, d_pos, partials, partials_bytes));
 }
 // The same for a chunk of T tokens at pos0, one mechanism per call.
-inline bool window_attn_chunk(void* u, int64_t ldu, void* y, int64_t ldy, const window_attn& at, int64_t T, int64_t pos0) {
+inline bool window_attn_chunk(void* u, int64_t ldu, void* y, int64_t ldy, const window_attn& at, int64_t T, int64_t pos0,
+                              bool exact = false) {
   launch L;
   if (!L.ok || !u || !y) return false;
   L.reads(u);
   L.writes(y, at.ring);
-  return L.sent(L.lib.window_fill(u, ldu, &at, T, pos0)) && L.sent(L.lib.window_attn_chunk(u, ldu, y, ldy, &at, T, pos0));
+  return L.sent(L.lib.window_fill(u, ldu, &at, T, pos0)) && L.sent(L.lib.window_attn_chunk(u, ldu, y, ldy, &at, T, pos0, exact ? 1 : 0));
 }
 inline bool linear_attn_chunk(void* u, int64_t ldu, void* y, int64_t ldy, const linear_attn& la, int64_t T, int64_t pos0) {
   launch L;

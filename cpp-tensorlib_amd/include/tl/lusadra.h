@@ -160,9 +160,10 @@ struct model {
   int64_t u_cols = 0, y_cols = 0;    // widest rows
   // true: the decode step's three launches per layer; false: one launch per op
   bool fused = true;
-  // prompt chunks of large products on the backend's prepared f16 form of the bf16 weights; false: on
-  // the bf16 rows, three exact terms per activation
-  bool prompt_f16 = true;
+  // prompt chunks: every product exact (bf16 weights times three exact terms of an activation, attention
+  // on the fp32 matrix pipe); false: large products on the backend's prepared f16 form of the weights and
+  // attention on the 16-bit matrix cores, two rounded terms per f32 operand
+  bool exact = false;
   std::vector<void*> owned;          // every device buffer, for destroy()
 
   model() = default;
@@ -494,7 +495,7 @@ inline bool chunk_layers(model& M, int64_t T, float* layer_out = nullptr) {
   chunk_scratch& P = M.ps;
   const int64_t WP = M.wp, E = M.c.width, pos0 = M.pos;
   const auto vec = [&](int64_t t) { return static_cast<char*>(M.steps) + t * WP * 4; };
-  hip::set_prompt_f16(M.prompt_f16);
+  hip::set_prompt_f16(!M.exact);
   bool ok = hip::embed_sinusoid(M.embed, P.tok, P.emb, T, E, WP, M.c.vocab, pos0);
   void* x = P.emb;
   int np = 0;                        // K-split parts of the previous layer's output, not yet added
@@ -517,7 +518,7 @@ inline bool chunk_layers(model& M, int64_t T, float* layer_out = nullptr) {
     } else {
       ok = ok && hip::rmsnorm(x, L.norm, P.h, WP, M.eps, T);
     }
-    ok = ok && gemm(L.win, P.h, P.u, T) && hip::window_attn_chunk(P.u, ldu, P.y, ldy, a, T, pos0) &&
+    ok = ok && gemm(L.win, P.h, P.u, T) && hip::window_attn_chunk(P.u, ldu, P.y, ldy, a, T, pos0, M.exact) &&
          hip::linear_attn_chunk(P.u, ldu, P.y, ldy, r, T, pos0) &&
          (!L.mlp || hip::polynorm_rows(P.u, ldu, P.y, ldy, L.pn, T)) &&
          gemm_parts(L.wout, P.y, P.parts, P.parts_bytes, T, &np);

@@ -24,7 +24,7 @@ namespace models {
 struct options {
   int64_t max_ctx = 4096;
   int64_t chunk = 512;         // longest prompt chunk
-  bool exact = false;          // prompt products on three exact terms per activation, not two rounded ones
+  bool exact = false;          // prompt products exact in f32, not in two rounded terms per operand
   bool q4 = false;             // int4 weights (models loaded from GGUF)
 };
 
@@ -63,7 +63,7 @@ class of : public any {
 // ---- folders: config.json + model.safetensors ---------------------------------------------------
 inline std::unique_ptr<any> open_lusadra(const json::value& cfg, const std::string& dir, const options& o) {
   auto p = std::make_unique<of<lusadra::model>>(lusadra::kArchitecture, o.chunk);
-  p->m.prompt_f16 = !o.exact;
+  p->m.exact = o.exact;
   lusadra::load(p->m, cfg, dir, o.max_ctx, o.chunk);
   return p;
 }

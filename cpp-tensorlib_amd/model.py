@@ -61,7 +61,7 @@ class Model:
 
     @classmethod
     def open(cls, path, max_ctx=4096, chunk=512, exact=False, q4=False):
-        """exact: prompt products in three exact terms per activation instead of two rounded ones."""
+        """exact: prompt products exact in f32 instead of in two rounded terms per operand."""
         L = _load()
         return cls(L, L.tlm_open(os.fsencode(path), max_ctx, chunk, int(exact), int(q4)))
 

@@ -514,10 +514,13 @@ int64_t tlhip_mix_partials_bytes(const tlhip_window_attn* at);
 int tlhip_mix_step(const void* u, void* y, const tlhip_window_attn* at, const tlhip_linear_attn* la,
                    const tlhip_polynorm* pn, int64_t pos, const void* d_pos, void* partials,
                    int64_t partials_bytes);
-/* A chunk of T tokens at positions pos0 .. pos0 + T - 1, u rows ldu and y rows ldy elements apart. */
+/* A chunk of T tokens at positions pos0 .. pos0 + T - 1, u rows ldu and y rows ldy elements apart.
+ * exact != 0: attention products in f32 on the fp32 matrix pipe; 0: chunks of 16 tokens up of heads up to
+ * 128 cut every f32 operand into two bf16 terms (2^-17 relative) on the 16-bit matrix cores; scores,
+ * weights and sums are f32 in both. */
 int tlhip_window_fill(const void* u, int64_t ldu, const tlhip_window_attn* at, int64_t T, int64_t pos0);
 int tlhip_window_attn_chunk(const void* u, int64_t ldu, void* y, int64_t ldy, const tlhip_window_attn* at,
-                            int64_t T, int64_t pos0);
+                            int64_t T, int64_t pos0, int exact);
 int tlhip_linear_attn_chunk(const void* u, int64_t ldu, void* y, int64_t ldy, const tlhip_linear_attn* la,
                             int64_t T, int64_t pos0);
 int tlhip_polynorm_rows(const void* u, int64_t ldu, void* y, int64_t ldy, const tlhip_polynorm* pn, int64_t T);

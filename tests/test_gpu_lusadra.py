@@ -63,6 +63,26 @@ def test_prompt_portions_and_steps(tmp_path, Model, name, exact):
     m.close()
 
 
+def test_large_products_in_both_forms(Model):
+    """At sizes where prompt products run over the prepared weights and the attention on the 16-bit matrix
+    cores, the serving form stays within its rounding of the exact one; a chunk equals steps."""
+    l = LM.layer(12, 4, 96, 160, 0.3, 50, 0.1, 8, 64, 96, 6.0, 0.9, 0.8, 3000)
+    cfg = LM.config(2000, 1120, [l, l, l], loop=(1, 2, 2))
+    t = ids(cfg, 700, 12)
+    want = [0, 1, 100, 159, 160, 161, 511, 512, 513, 699]
+    lg = {}
+    for exact in (True, False):
+        m = Model.random_lusadra(cfg, seed=3, rank=10, max_ctx=800, exact=exact)
+        lg[exact] = m.feed(t, want)
+        if exact:
+            m.reset()
+            m.feed(t[:600])
+            steps = np.concatenate([m.feed([x], [0]) for x in t[600:]])
+            close(steps[-1], lg[True][-1], 1e-4)
+        m.close()
+    close(lg[False], lg[True], 1e-3)
+
+
 def test_unfused_step_equals_fused(tmp_path, Model):
     cfg, orc, m = make(tmp_path, Model, "loop_of_unlike_layers")
     m.set_fused(False)

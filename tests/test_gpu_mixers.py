@@ -38,7 +38,8 @@ def close(got, want, tol=2e-5):
 class Window:
     """One attention on the GPU: rows u = [q | k | gate], rows y = [out]."""
 
-    def __init__(self, lib, capi, H, G, dim, window, chunk, gate=True, scale=None, coef=0.3, every=16, out_scale=1.0):
+    def __init__(self, lib, capi, H, G, dim, window, chunk, gate=True, scale=None, coef=0.3, every=16, out_scale=1.0, exact=True):
+        self.exact = exact
         self.lib, self.H, self.G, self.dim, self.window = lib, H, G, dim, window
         self.scale, self.coef, self.every = dim ** -0.5 if scale is None else scale, coef, every
         ld = lib.c.tlhip_window_ring_ld(dim)
@@ -57,7 +58,7 @@ class Window:
     def chunk(self, u, pos0):
         T = len(u)
         du, dy = self.lib.to_device(np.ascontiguousarray(u, np.float32)), self.lib.to_device(np.zeros((T, self.ldy), np.float32))
-        self.lib.window_attn_chunk(du, self.W, dy, self.ldy, self.at, T, pos0)
+        self.lib.window_attn_chunk(du, self.W, dy, self.ldy, self.at, T, pos0, self.exact)
         return dy.numpy()[:, 1:1 + self.H * self.dim]
 
     def step(self, u, pos, d_pos=None):
@@ -84,41 +85,76 @@ WINDOWS = [  # H, G, dim, window
     (2, 1, 256, 40), (1, 1, 30, 5)]
 
 
+# the exact form of the chunk kernel, and the one whose f32 operands are two bf16 terms (2^-17 per
+# product: scores of +-20 move weights by a few 1e-5)
+FORMS = [(True, 2e-5), (False, 2e-4)]
+
+
+@pytest.mark.parametrize("exact,tol", FORMS)
 @pytest.mark.parametrize("H,G,dim,window", WINDOWS)
-def test_window_attention_chunks_and_steps(lib, capi, H, G, dim, window):
+def test_window_attention_chunks_and_steps(lib, capi, H, G, dim, window, exact, tol):
     """One prompt in one chunk, in portions, and token by token, all against the plain form."""
     T = 2 * window + 45
-    w = Window(lib, capi, H, G, dim, window, chunk=T, gate=dim != 64, out_scale=1.25)
+    mk = lambda chunk: Window(lib, capi, H, G, dim, window, chunk=chunk, gate=dim != 64, out_scale=1.25, exact=exact)
+    w = mk(T)
     u = w.rows(T, dim * 100 + window, amp=2.0)
     want = w.want(u)
-    close(w.chunk(u, 0), want)
+    close(w.chunk(u, 0), want, tol)
     for size in (2, 31, 32, 50):
-        w = Window(lib, capi, H, G, dim, window, chunk=size, gate=dim != 64, out_scale=1.25)
+        w = mk(size)
         got = np.concatenate([w.chunk(u[t:t + size], t) for t in range(0, T, size)])
-        close(got, want)
-    w = Window(lib, capi, H, G, dim, window, chunk=1, gate=dim != 64, out_scale=1.25)
-    close(np.stack([w.step(u[t], t) for t in range(T)]), want)
+        close(got, want, tol)
+    if exact:
+        w = mk(1)
+        close(np.stack([w.step(u[t], t) for t in range(T)]), want)
 
 
-def test_window_edges_show(lib, capi):
+@pytest.mark.parametrize("exact", [True, False])
+@pytest.mark.parametrize("H,G", [(2, 1), (9, 1), (3, 3)])
+def test_window_edges_show(lib, capi, H, G, exact):
     """A query that singles out ONE key: seen at distance window - 1, gone at distance window; chunks
-    and steps, keys at and around tile borders of the ring."""
-    H, G, dim, window = 2, 1, 32, 40
+    and steps, keys at and around tile borders of the ring; every head, also where several share a
+    block's tile or a group is spread over blocks."""
+    dim, window = 32, 40
     T, far = 140, 200.0
     for key in (0, 31, 32, 63, 64, 71, 95):
-        w = Window(lib, capi, H, G, dim, window, chunk=T, gate=False, coef=0.0)
+        w = Window(lib, capi, H, G, dim, window, chunk=T, gate=False, coef=0.0, exact=exact)
         u = 0.1 * w.rows(T, 5)
         spike = np.zeros(dim, np.float32)
         spike[3] = 1.0
-        u[key, H * dim:(H + G) * dim] = spike * far
+        for g in range(G):
+            u[key, (H + g) * dim:(H + g + 1) * dim] = spike * far
         for t in (key + window - 1, key + window):          # just inside, just outside
             for h in range(H):
                 u[t, h * dim:(h + 1) * dim] = spike * far
         want = w.want(u)
-        assert abs(want[key + window - 1, 3]) > 100 and abs(want[key + window, 3]) < 1      # it shows
-        close(w.chunk(u, 0), want)
-        w2 = Window(lib, capi, H, G, dim, window, chunk=1, gate=False, coef=0.0)
-        close(np.stack([w2.step(u[t], t) for t in range(key + window + 2)]), want[:key + window + 2])
+        for h in range(H):
+            assert abs(want[key + window - 1, h * dim + 3]) > 100 and abs(want[key + window, h * dim + 3]) < 1   # it shows
+        close(w.chunk(u, 0), want, 2e-5 if exact else 2e-4)
+        if exact:
+            w2 = Window(lib, capi, H, G, dim, window, chunk=1, gate=False, coef=0.0)
+            close(np.stack([w2.step(u[t], t) for t in range(key + window + 2)]), want[:key + window + 2])
+
+
+@pytest.mark.parametrize("H,G", [(8, 2), (7, 1), (4, 4)])
+def test_window_chunks_deep_in_a_context(lib, capi, H, G):
+    """Both chunk forms at positions past a long window, where the key tiles are split over blocks, in
+    chunks that are no multiple of anything, against the plain form at some rows."""
+    dim, window, T0, T = 64, 700, 900, 333
+    outs = []
+    for exact, tol in FORMS:
+        w = Window(lib, capi, H, G, dim, window, chunk=T0, exact=exact)
+        u = w.rows(T0 + T, 17, amp=1.5)
+        w.chunk(u[:T0], 0)
+        got = w.chunk(u[T0:], T0)
+        k = u[:, H * dim:(H + G) * dim].astype(np.float64)
+        gate = O.sigmoid(u[:, (H + G) * dim:(H + G) * dim + H * dim].astype(np.float64))
+        for t in (0, 1, 31, 32, 200, 331, 332):
+            i = T0 + t
+            a = O.window_attention(u[i:i + 1, :H * dim].astype(np.float64), k[:i + 1], H, G, dim, window, w.scale, w.coef, w.every, pos0=i)
+            close(got[t], (a * gate[i])[0], tol)
+        outs.append(got)
+    close(outs[1], outs[0], 2e-4)
 
 
 def test_window_long_context_and_splits(lib, capi):

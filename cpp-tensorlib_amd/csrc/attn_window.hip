@@ -236,7 +236,7 @@ __global__ __launch_bounds__(512, 1) void window_terms_kernel(const float* __res
   const bool stages = tid < kTasks;
   f32x2 kreg[4];
   const auto request = [&](f32x2 (&k)[4], int tile) {
-    tile = min(tile, kt1 - 1);
+    tile = max(tile, kt0);
     const float* base = ring + (size_t)((tile * 32) % R) * D + d2;
     const int last = kend - 1 - tile * 32;
 #pragma unroll
@@ -262,7 +262,8 @@ __global__ __launch_bounds__(512, 1) void window_terms_kernel(const float* __res
       *reinterpret_cast<bf16x4*>(KT + L::kT + (unit + c) * 8 + off) = t1[c];
     }
   };
-  int kt = kt0 + (int)blockIdx.z;
+  // newest keys first: the distance bias makes them the likely maxima, which then seldom move
+  int kt = kt1 - 1 - (int)blockIdx.z;
   if (stages) request(kreg, kt);
 
   // queries times their temperature, cut into terms: lane (hi, l31) holds columns 16s + 8hi .. + 7 of query l31
@@ -271,19 +272,29 @@ __global__ __launch_bounds__(512, 1) void window_terms_kernel(const float* __res
     const int t = min(max(p0, 0) + l31, T - 1);
     const float temp = query_temperature(pos0 + t, a.temp_coef, a.temp_every);
     const float* q = u + (size_t)t * ldu + a.q_off + (size_t)min(h, heads - 1) * dim;
+    const bool vec = (reinterpret_cast<uintptr_t>(q) & 15) == 0 && (dim & 3) == 0 && (ldu & 3) == 0;
 #pragma unroll
-    for (int s = 0; s < D / 16; s++)
+    for (int s = 0; s < D / 16; s++) {
+      f32x4 x[2];
+#pragma unroll
+      for (int k = 0; k < 2; k++) {
+        const int d = 16 * s + 8 * hi + 4 * k;
+        if (vec) {                     // (the head's row starts on 16 bytes and holds whole quads)
+          x[k] = *reinterpret_cast<const f32x4*>(q + min(d, dim - 4));
+          if (d >= dim) x[k] = f32x4{0.f, 0.f, 0.f, 0.f};
+        } else {
+#pragma unroll
+          for (int j = 0; j < 4; j++) x[k][j] = d + j < dim ? q[d + j] : 0.f;
+        }
+      }
 #pragma unroll
       for (int j = 0; j < 8; j += 2) {
-        const int d = 16 * s + 8 * hi + j;
-        f32x2 x;
-        x[0] = d < dim ? q[d] * temp : 0.f;
-        x[1] = d + 1 < dim ? q[d + 1] * temp : 0.f;
         bf16x2 f, g;
-        two_terms(x, f, g);
+        two_terms(f32x2{x[j >> 2][j & 3] * temp, x[j >> 2][(j & 3) + 1] * temp}, f, g);
         q0[s][j] = f[0]; q0[s][j + 1] = f[1];
         q1[s][j] = g[0]; q1[s][j + 1] = g[1];
       }
+    }
   }
   f32x16 o[D / 32];
 #pragma unroll
@@ -294,10 +305,10 @@ __global__ __launch_bounds__(512, 1) void window_terms_kernel(const float* __res
   const int qpos = pos0 + p0 + l31;
   const float sc2 = a.scale * kLog2e, sl2 = head_slope(h, heads, a.slope_exp) * kLog2e;
 
-  if (stages && kt < kt1) stage(kreg, 0);
-  if (stages) request(kreg, kt + plan.S);
+  if (stages && kt >= kt0) stage(kreg, 0);
+  if (stages) request(kreg, kt - plan.S);
   __syncthreads();
-  for (int buf = 0; kt < kt1; kt += plan.S, buf ^= 1) {
+  for (int buf = 0; kt >= kt0; kt -= plan.S, buf ^= 1) {
     if (kt >= wt0 && kt < wt1) {
       const __bf16 *K = bl + buf * L::kBuf, *KT = K + 2 * L::kK;
       f32x16 s, r;                     // first x first, and the two mixed pairs
@@ -358,8 +369,8 @@ __global__ __launch_bounds__(512, 1) void window_terms_kernel(const float* __res
         }
     }
     // the next tile into the other buffer (last read before the barrier that ended the turn before)
-    if (stages && kt + plan.S < kt1) stage(kreg, buf ^ 1);
-    if (stages) request(kreg, kt + 2 * plan.S);
+    if (stages && kt - plan.S >= kt0) stage(kreg, buf ^ 1);
+    if (stages) request(kreg, kt - 2 * plan.S);
     __syncthreads();
   }
   const int t = p0 + l31;
@@ -389,38 +400,55 @@ __global__ __launch_bounds__(512, 1) void window_terms_kernel(const float* __res
     }
 }
 
-// The key splits of (token, head) rows, one wavefront each -> y.
+// The key splits of (token, head) rows -> y, D / 4 lanes to a row. `i` numbers threads.
+template <int D>
+__device__ __forceinline__ void window_join(const float* __restrict__ u, int64_t ldu, float* __restrict__ y, int64_t ldy,
+                                            const tlhip_window_attn& a, int T, int S, const float* __restrict__ acc,
+                                            const float* __restrict__ stat, size_t i) {
+  constexpr int LR = D / 4, U = 4;                // splits requested at once
+  const int heads = (int)a.heads, dim = (int)a.dim;
+  const size_t rows = (size_t)T * heads, r = i / LR;
+  const int d = 4 * (int)(i % LR);
+  if (r >= rows || d >= dim) return;
+  const int t = (int)(r / heads), h = (int)(r % heads);
+  const float* gp = u + (size_t)t * ldu + a.gate_off + (size_t)h * dim + d;
+  const bool gated = a.gate_off >= 0;
+  float g[4];
+#pragma unroll
+  for (int j = 0; j < 4; j++) g[j] = gated && d + j < dim ? gp[j] : 0.f;
+  float M = -INFINITY, Ls = 0.f;
+  f32x4 o = {0.f, 0.f, 0.f, 0.f};
+  for (int s0 = 0; s0 < S; s0 += U) {
+    f32x4 v[U];
+    f32x2 st[U];
+#pragma unroll
+    for (int k = 0; k < U; k++) {
+      const size_t at = (size_t)min(s0 + k, S - 1) * rows + r;
+      v[k] = *reinterpret_cast<const f32x4*>(acc + at * D + d);
+      st[k] = *reinterpret_cast<const f32x2*>(stat + 2 * at);
+    }
+#pragma unroll
+    for (int k = 0; k < U; k++) {
+      if (s0 + k >= S || st[k][0] == -INFINITY) continue;
+      const float m = fmaxf(M, st[k][0]), fo = exp2_native(M - m), fn = exp2_native(st[k][0] - m);
+      M = m;
+      Ls = Ls * fo + fn * st[k][1];
+#pragma unroll
+      for (int j = 0; j < 4; j++) o[j] = o[j] * fo + fn * v[k][j];
+    }
+  }
+  const float inv = a.out_scale / Ls;
+  float* yp = y + (size_t)t * ldy + a.y_off + (size_t)h * dim + d;
+#pragma unroll
+  for (int j = 0; j < 4; j++)
+    if (d + j < dim) yp[j] = o[j] * inv * (gated ? sigmoid_f(g[j]) : 1.f);
+}
+
 template <int D>
 __global__ __launch_bounds__(256) void window_join_kernel(const float* __restrict__ u, int64_t ldu, float* __restrict__ y,
                                                           int64_t ldy, const tlhip_window_attn a, int T, int S,
                                                           const float* __restrict__ acc, const float* __restrict__ stat) {
-  const int heads = (int)a.heads, dim = (int)a.dim, lane = threadIdx.x & 63;
-  const size_t rows = (size_t)T * heads, i = (size_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (i >= rows) return;
-  const int t = (int)(i / heads), h = (int)(i % heads);
-  float M = -INFINITY;
-  for (int s = 0; s < S; s++) M = fmaxf(M, stat[2 * (s * rows + i)]);
-  float Ls = 0.f, o[(D + 63) / 64] = {};
-  for (int s = 0; s < S; s++) {
-    const size_t r = s * rows + i;
-    const float ms = stat[2 * r], f = ms == -INFINITY ? 0.f : exp2_native(ms - M);
-    Ls = fmaf(f, stat[2 * r + 1], Ls);
-#pragma unroll
-    for (int k = 0; k < (D + 63) / 64; k++) {
-      const int d = lane + 64 * k;
-      if (d < D) o[k] = fmaf(f, acc[r * D + d], o[k]);
-    }
-  }
-  const float inv = a.out_scale / Ls;
-#pragma unroll
-  for (int k = 0; k < (D + 63) / 64; k++) {
-    const int d = lane + 64 * k;
-    if (d < dim) {
-      float v = o[k] * inv;
-      if (a.gate_off >= 0) v *= sigmoid_f(u[(size_t)t * ldu + a.gate_off + (size_t)h * dim + d]);
-      y[(size_t)t * ldy + a.y_off + (size_t)h * dim + d] = v;
-    }
-  }
+  window_join<D>(u, ldu, y, ldy, a, T, S, acc, stat, (size_t)blockIdx.x * 256 + threadIdx.x);
 }
 
 template <int D>
@@ -438,7 +466,7 @@ static int launch_terms(const float* u, int64_t ldu, float* y, int64_t ldy, cons
   float *acc = nullptr, *stat = nullptr;
   if (p.S > 1) {
     const size_t rows = (size_t)p.S * T * a.heads;
-    acc = static_cast<float*>(scratch(rows * (D + 2) * sizeof(float)));
+    acc = static_cast<float*>(scratch(rows * (D + 2) * sizeof(float)));   // rows of D are 16-byte aligned, then the pairs
     if (!acc) return fail(TLHIP_ENOMEM, "tlhip_window_attn_chunk: no scratch");
     stat = acc + rows * D;
   }
@@ -449,8 +477,8 @@ static int launch_terms(const float* u, int64_t ldu, float* y, int64_t ldy, cons
   hipLaunchKernelGGL(fn, dim3((unsigned)(a.kv_heads * p.subs), (unsigned)runs, (unsigned)p.S), dim3(512), lds, c.stream, u, ldu, y, ldy,
                      a, T, pos0, p, acc, stat);
   if (p.S > 1)
-    hipLaunchKernelGGL(window_join_kernel<D>, dim3((unsigned)(((size_t)T * a.heads + 3) / 4)), dim3(256), 0, c.stream, u, ldu, y, ldy, a,
-                       T, p.S, acc, stat);
+    hipLaunchKernelGGL(window_join_kernel<D>, dim3((unsigned)(((size_t)T * a.heads * (D / 4) + 255) / 256)), dim3(256), 0, c.stream, u, ldu, y,
+                       ldy, a, T, p.S, acc, stat);
   TLHIP_CHECK_LAUNCH(TLHIP_C_WINDOW_ATTN);
 }
 

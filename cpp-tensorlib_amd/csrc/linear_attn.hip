@@ -33,17 +33,17 @@ struct PieceBuf {
   int C, np, dp, vp, vs;           // tokens per piece, pieces; vs: value columns of one block of linear_piece_kernel
 };
 
-// Block (piece, head, value slice) of 512 threads.
+// Block (piece of C tokens, head, value slice) of 512 threads.
+template <int C>
 __global__ __launch_bounds__(512) void linear_piece_kernel(const float* __restrict__ u, int64_t ldu, const tlhip_linear_attn a,
                                                            int T, const PieceBuf pb) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int tid = threadIdx.x, lane = tid & 63, l15 = lane & 15, lg = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int piece = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * pb.vs;
-  const int C = pb.C, dp = pb.dp, vp = pb.vp, dim = (int)a.dim, vdim = (int)a.vdim;
-  const int NB = C / 16, QS = dp + 4, nv = min(pb.vs, vp - v0);
-  const int VS = pb.vs + 4;
-  const int AS = C + 4;
+  const int dp = pb.dp, vp = pb.vp, dim = (int)a.dim, vdim = (int)a.vdim;
+  constexpr int NB = C / 16, RW = C / 8, AS = C + 4;   // RW: tokens a wavefront copies
+  const int QS = dp + 4, VS = pb.vs + 4, nv = min(pb.vs, vp - v0);
   float* Q = lds;                      // [C][QS] q, then Q'
   float* K = Q + C * QS;               // [C][QS] k, then K'
   float* Lg = K + C * QS;              // [C][QS] log2 decays since the block began
@@ -55,6 +55,19 @@ __global__ __launch_bounds__(512) void linear_piece_kernel(const float* __restri
   const float inv_tau = 1.0f / a.tau;
 
   if (tid < NB) slow[tid] = 0;
+  // queries, keys and values: the first 64 channels (128 value columns) of a wavefront's tokens are
+  // requested before anything else
+  const auto row = [&](int t) { return u + (size_t)(t0 + min(t, nt - 1)) * ldu; };
+  const int qo = (int)a.q_off + h * dim, ko = (int)a.k_off + h * dim, vo = (int)a.v_off + h * vdim + v0, nvl = min(pb.vs, vdim - v0);
+  float qr[RW], kr[RW], vr[2][RW];
+#pragma unroll
+  for (int i = 0; i < RW; i++) {
+    const float* p = row(wave + 8 * i);
+    qr[i] = p[qo + min(lane, dim - 1)];
+    kr[i] = p[ko + min(lane, dim - 1)];
+    vr[0][i] = p[vo + min(lane, nvl - 1)];
+    vr[1][i] = p[vo + min(lane + 64, nvl - 1)];
+  }
   // decay logits: Z = low A2^T in 16 x 16 tiles, and their logs (bias, sigmoid, 1/tau) in Lg
   {
     const int rank = (int)a.rank;
@@ -84,25 +97,42 @@ __global__ __launch_bounds__(512) void linear_piece_kernel(const float* __restri
       }
     }
   }
-  for (int t = wave; t < C; t += 8) {
-    const float* row = u + (size_t)(t0 + min(t, nt - 1)) * ldu;
-    const float *q = row + a.q_off + h * dim, *k = row + a.k_off + h * dim, *v = row + a.v_off + (int64_t)h * vdim + v0;
-    for (int d = lane; d < dp; d += 64) {
-      const bool live = t < nt && d < dim;
-      const int dc = min(d, dim - 1);
-      const float qd = q[dc], kd = k[dc];
-      Q[t * QS + d] = live ? qd * a.q_scale : 0.f;
-      K[t * QS + d] = live ? kd : 0.f;
+#pragma unroll
+  for (int i = 0; i < RW; i++) {
+    const int t = wave + 8 * i;
+    const bool live = t < nt;
+    if (lane < dp) {
+      Q[t * QS + lane] = live && lane < dim ? qr[i] * a.q_scale : 0.f;
+      K[t * QS + lane] = live && lane < dim ? kr[i] : 0.f;
     }
-    for (int c = lane; c < pb.vs; c += 64) V[t * VS + c] = t < nt && v0 + c < vdim ? v[c] : 0.f;
+    if (lane < pb.vs) V[t * VS + lane] = live && lane < nvl ? vr[0][i] : 0.f;
+    if (lane + 64 < pb.vs) V[t * VS + lane + 64] = live && lane + 64 < nvl ? vr[1][i] : 0.f;
+  }
+  for (int d = lane + 64; d < dp; d += 64) {
+#pragma unroll
+    for (int i = 0; i < RW; i++) {
+      const float* p = row(wave + 8 * i);
+      qr[i] = p[qo + min(d, dim - 1)];
+      kr[i] = p[ko + min(d, dim - 1)];
+    }
+#pragma unroll
+    for (int i = 0; i < RW; i++) {
+      const int t = wave + 8 * i;
+      const bool live = t < nt && d < dim;
+      Q[t * QS + d] = live ? qr[i] * a.q_scale : 0.f;
+      K[t * QS + d] = live ? kr[i] : 0.f;
+    }
   }
   __syncthreads();
   for (int i = tid; i < NB * dp; i += 512) {         // running sums of the logs inside each block
     const int b = i / dp, d = i - b * dp;
-    float s = 0.f;
-    for (int t = 16 * b; t < 16 * b + 16; t++) {
-      s += Lg[t * QS + d];
-      Lg[t * QS + d] = s;
+    float s = 0.f, g[16];
+#pragma unroll
+    for (int t = 0; t < 16; t++) g[t] = Lg[(16 * b + t) * QS + d];
+#pragma unroll
+    for (int t = 0; t < 16; t++) {
+      s += g[t];
+      Lg[(16 * b + t) * QS + d] = s;
     }
     tot[b * dp + d] = s;
     if (s < -kFastRange) slow[b] = 1;                // (every writer stores the same value)
@@ -252,24 +282,39 @@ __global__ __launch_bounds__(512) void linear_out_kernel(const float* __restrict
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int t0 = blockIdx.x * TM, h = blockIdx.y, dp = pb.dp, vp = pb.vp, OS = vp + 4, vdim = (int)a.vdim;
   const size_t hp = (size_t)h * pb.np + t0 / pb.C, hr = (size_t)h * pb.np * pb.C + t0;
+  // what the end of the kernel needs of u, requested now: norm weights and gates of the first 128 columns
+  float gate[TM / 8][2], nrm[2];
+#pragma unroll
+  for (int c = 0; c < 2; c++) {
+    const int v = min(lane + 64 * c, vdim - 1);
+    nrm[c] = static_cast<const float*>(a.norm)[v];
+#pragma unroll
+    for (int i = 0; i < TM / 8; i++) gate[i][c] = u[(size_t)min(t0 + wave + 8 * i, T - 1) * ldu + a.gate_off + (int64_t)h * vdim + v];
+  }
   for (int vt = wave; vt < vp / 16; vt += 8) {
     f32x4 acc[MT];
 #pragma unroll
     for (int mt = 0; mt < MT; mt++)
 #pragma unroll
       for (int v = 0; v < 4; v++) acc[mt][v] = pb.oi[(hr + 16 * mt + 4 * lg + v) * vp + 16 * vt + l15];
-    for (int d0 = 0; d0 < dp; d0 += 16) {
-      const int d = d0 + 4 * lg;
-      const float* sp = pb.st + (hp * dp + d) * vp + 16 * vt + l15;
-      const float s0 = sp[0], s1 = sp[vp], s2 = sp[2 * vp], s3 = sp[3 * vp];
+    for (int d1 = 0; d1 < dp; d1 += 64) {            // four steps requested at once (past dp: clamped, times zero)
+      float sv[4][4];
+      f32x4 q[4][MT];
 #pragma unroll
-      for (int mt = 0; mt < MT; mt++) {
-        const float4 q = *reinterpret_cast<const float4*>(pb.qd + (hr + 16 * mt + l15) * dp + d);
-        acc[mt] = mfma16(q.x, s0, acc[mt]);
-        acc[mt] = mfma16(q.y, s1, acc[mt]);
-        acc[mt] = mfma16(q.z, s2, acc[mt]);
-        acc[mt] = mfma16(q.w, s3, acc[mt]);
+      for (int k = 0; k < 4; k++) {
+        const int d = min(d1 + 16 * k, dp - 16) + 4 * lg;
+        const float* sp = pb.st + (hp * dp + d) * vp + 16 * vt + l15;
+#pragma unroll
+        for (int j = 0; j < 4; j++) sv[k][j] = sp[j * vp];
+#pragma unroll
+        for (int mt = 0; mt < MT; mt++) q[k][mt] = *reinterpret_cast<const f32x4*>(pb.qd + (hr + 16 * mt + l15) * dp + d);
       }
+#pragma unroll
+      for (int k = 0; k < 4; k++)
+#pragma unroll
+        for (int mt = 0; mt < MT; mt++)
+#pragma unroll
+          for (int j = 0; j < 4; j++) acc[mt] = mfma16(d1 + 16 * k < dp ? q[k][mt][j] : 0.f, sv[k][j], acc[mt]);
     }
 #pragma unroll
     for (int mt = 0; mt < MT; mt++)
@@ -277,14 +322,22 @@ __global__ __launch_bounds__(512) void linear_out_kernel(const float* __restrict
       for (int v = 0; v < 4; v++) lds[(16 * mt + 4 * lg + v) * OS + 16 * vt + l15] = acc[mt][v];
   }
   __syncthreads();
-  for (int r = wave; r < TM && t0 + r < T; r += 8) {
+#pragma unroll
+  for (int i = 0; i < TM / 8; i++) {
+    const int r = wave + 8 * i;
+    if (t0 + r >= T) break;
     float ss = 0.f;
     for (int v = lane; v < vdim; v += 64) ss = fmaf(lds[r * OS + v], lds[r * OS + v], ss);
     ss = wave_sum(ss);
     const float inv = 1.0f / sqrtf(ss / (float)vdim + a.eps);
-    const float* g = u + (size_t)(t0 + r) * ldu + a.gate_off + (int64_t)h * vdim;
     float* o = y + (size_t)(t0 + r) * ldy + a.y_off + (int64_t)h * vdim;
-    for (int v = lane; v < vdim; v += 64)
+#pragma unroll
+    for (int c = 0; c < 2; c++) {
+      const int v = lane + 64 * c;
+      if (v < vdim) o[v] = lds[r * OS + v] * inv * nrm[c] * (gate[i][c] * sigmoid_f(gate[i][c])) * a.out_scale;
+    }
+    const float* g = u + (size_t)(t0 + r) * ldu + a.gate_off + (int64_t)h * vdim;
+    for (int v = lane + 128; v < vdim; v += 64)
       o[v] = lds[r * OS + v] * inv * static_cast<const float*>(a.norm)[v] * (g[v] * sigmoid_f(g[v])) * a.out_scale;
   }
 }
@@ -328,10 +381,11 @@ int tlhip_linear_attn_chunk(const void* u, int64_t ldu, void* y, int64_t ldy, co
   pb.qd = pb.st + n_st;
   pb.oi = pb.qd + n_qd;
   const float* pu = static_cast<const float*>(u);
-  hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(linear_piece_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds1);
+  auto piece = pb.C == 64 ? linear_piece_kernel<64> : pb.C == 32 ? linear_piece_kernel<32> : linear_piece_kernel<16>;
+  hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(piece), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds1);
   if (e != hipSuccess) return hip_fail(e, "hipFuncSetAttribute(LDS)");
-  hipLaunchKernelGGL(linear_piece_kernel, dim3((unsigned)pb.np, (unsigned)la->heads, (unsigned)((pb.vp + pb.vs - 1) / pb.vs)),
-                     dim3(512), lds1, c.stream, pu, ldu, *la, (int)T, pb);
+  hipLaunchKernelGGL(piece, dim3((unsigned)pb.np, (unsigned)la->heads, (unsigned)((pb.vp + pb.vs - 1) / pb.vs)), dim3(512), lds1,
+                     c.stream, pu, ldu, *la, (int)T, pb);
   const size_t ns = (size_t)la->heads * pb.dp * (pb.vp / 4);
   hipLaunchKernelGGL(linear_scan_kernel, dim3((unsigned)((ns + 255) / 256)), dim3(256), 0, c.stream, *la, (int)T, (int)pos0, pb);
   auto out = mt == 2 ? linear_out_kernel<2> : linear_out_kernel<1>;

@@ -31,21 +31,42 @@ constexpr float kFastRange = 96.f;
 struct PieceBuf {
   float *dec, *st, *qd, *oi;
   int C, np, dp, vp, vs;           // tokens per piece, pieces; vs: value columns of one block of linear_piece_kernel
+  int qsh, vsh;                    // its lanes per row of queries and keys, of values: 1 << qsh, 1 << vsh
 };
 
-// Block (piece of C tokens, head, value slice) of 512 threads.
-template <int C>
+// Four floats of a row of n at column c: zeros past n and where !live. vec: the row starts on 16 bytes
+// and n is a multiple of 4.
+__device__ __forceinline__ f32x4 load_quad(const float* __restrict__ p, int c, int n, bool vec, bool live) {
+  f32x4 x;
+  if (vec) {
+    x = *reinterpret_cast<const f32x4*>(p + min(c, n - 4));
+    if (!live || c >= n) x = f32x4{0.f, 0.f, 0.f, 0.f};
+  } else {
+#pragma unroll
+    for (int j = 0; j < 4; j++) {
+      x[j] = p[min(c + j, n - 1)];
+      if (!live || c + j >= n) x[j] = 0.f;
+    }
+  }
+  return x;
+}
+__device__ __forceinline__ f32x4 exp2_quad(f32x4 e) {
+  return f32x4{exp2_native(e[0]), exp2_native(e[1]), exp2_native(e[2]), exp2_native(e[3])};
+}
+
+// Block (piece of C tokens, head, value slice) of 512 threads. NS: quads of q (and of k) a thread holds.
+template <int C, int NS>
 __global__ __launch_bounds__(512) void linear_piece_kernel(const float* __restrict__ u, int64_t ldu, const tlhip_linear_attn a,
                                                            int T, const PieceBuf pb) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
+  constexpr int NB = C / 16, AS = C + 4, NV = (C + 15) / 16;
   const int tid = threadIdx.x, lane = tid & 63, l15 = lane & 15, lg = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int piece = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * pb.vs;
-  const int dp = pb.dp, vp = pb.vp, dim = (int)a.dim, vdim = (int)a.vdim;
-  constexpr int NB = C / 16, RW = C / 8, AS = C + 4;   // RW: tokens a wavefront copies
-  const int QS = dp + 4, VS = pb.vs + 4, nv = min(pb.vs, vp - v0);
-  float* Q = lds;                      // [C][QS] q, then Q'
-  float* K = Q + C * QS;               // [C][QS] k, then K'
+  const int dp = pb.dp, vp = pb.vp, dim = (int)a.dim, vdim = (int)a.vdim, rank = (int)a.rank;
+  const int QS = dp + 4, VS = pb.vs + 4, nv = min(pb.vs, vp - v0), nvl = min(pb.vs, vdim - v0);
+  float* Q = lds;                      // [C][QS] Q' (q while a block needs the pairwise form)
+  float* K = Q + C * QS;               // [C][QS] K'
   float* Lg = K + C * QS;              // [C][QS] log2 decays since the block began
   float* V = Lg + C * QS;              // [C][VS]
   float* A = V + C * VS;               // [C][AS]
@@ -53,108 +74,123 @@ __global__ __launch_bounds__(512) void linear_piece_kernel(const float* __restri
   int* slow = reinterpret_cast<int*>(tot + NB * dp);   // [NB]
   const int t0 = piece * C, nt = min(C, T - t0);
   const float inv_tau = 1.0f / a.tau;
-
-  if (tid < NB) slow[tid] = 0;
-  // queries, keys and values: the first 64 channels (128 value columns) of a wavefront's tokens are
-  // requested before anything else
   const auto row = [&](int t) { return u + (size_t)(t0 + min(t, nt - 1)) * ldu; };
-  const int qo = (int)a.q_off + h * dim, ko = (int)a.k_off + h * dim, vo = (int)a.v_off + h * vdim + v0, nvl = min(pb.vs, vdim - v0);
-  float qr[RW], kr[RW], vr[2][RW];
+
+  // queries, keys and values into registers, 16 bytes a lane: quad i of a thread is token (tid + 512 i) >> sh
+  const bool u16 = (reinterpret_cast<uintptr_t>(u) & 15) == 0 && (ldu & 3) == 0;
+  const int qo = (int)a.q_off + h * dim, ko = (int)a.k_off + h * dim, vo = (int)a.v_off + h * vdim + v0;
+  const bool qvec = u16 && ((qo | ko | dim) & 3) == 0, vvec = u16 && ((vo | nvl) & 3) == 0;
+  const int qm = (1 << pb.qsh) - 1, vm = (1 << pb.vsh) - 1;
+  f32x4 q[NS], k[NS], v[NV];
 #pragma unroll
-  for (int i = 0; i < RW; i++) {
-    const float* p = row(wave + 8 * i);
-    qr[i] = p[qo + min(lane, dim - 1)];
-    kr[i] = p[ko + min(lane, dim - 1)];
-    vr[0][i] = p[vo + min(lane, nvl - 1)];
-    vr[1][i] = p[vo + min(lane + 64, nvl - 1)];
+  for (int i = 0; i < NS; i++) {
+    const int slot = tid + 512 * i, t = slot >> pb.qsh, c = 4 * (slot & qm);
+    q[i] = load_quad(row(t) + qo, c, dim, qvec, t < nt);
+    k[i] = load_quad(row(t) + ko, c, dim, qvec, t < nt);
   }
-  // decay logits: Z = low A2^T in 16 x 16 tiles, and their logs (bias, sigmoid, 1/tau) in Lg
+#pragma unroll
+  for (int i = 0; i < NV; i++) {
+    const int slot = tid + 512 * i, t = slot >> pb.vsh, c = 4 * (slot & vm);
+    v[i] = load_quad(row(t) + vo, c, nvl, vvec, t < nt);
+  }
+  if (tid < NB) slow[tid] = 0;
+  __syncthreads();
+  // decay logits Z = low A2^T, a 16 x 16 tile (one block's tokens, 16 channels) at a time; their logs summed
+  // up along the tokens: in a lane's four registers, then over the four lane groups
   {
-    const int rank = (int)a.rank;
     const uint16_t* a2 = static_cast<const uint16_t*>(a.a2) + (size_t)h * dim * rank;
     const float* bias = static_cast<const float*>(a.bias) + h * dim;
+    const bool lvec = u16 && ((rank | (int)a.low_off) & 3) == 0;
     for (int tile = wave; tile < NB * (dp / 16); tile += 8) {
-      const int tt = tile % NB, d = 16 * (tile / NB) + l15, t = 16 * tt + l15;
-      const float* low = u + (size_t)(t0 + min(t, nt - 1)) * ldu + a.low_off;
+      const int b = tile % NB, d = 16 * (tile / NB) + l15;
+      const float* low = row(16 * b + l15) + a.low_off;
       const uint16_t* w = a2 + (size_t)min(d, dim - 1) * rank;
       f32x4 z = {0.f, 0.f, 0.f, 0.f};
-      for (int r0 = 0; r0 < rank; r0 += 16) {
-        float x[4], y[4];
-#pragma unroll
-        for (int j = 0; j < 4; j++) {
-          const int r = r0 + 4 * lg + j, rc = min(r, rank - 1);
-          x[j] = r < rank ? low[rc] : 0.f;
-          y[j] = __uint_as_float((uint32_t)w[rc] << 16);
-        }
-#pragma unroll
-        for (int j = 0; j < 4; j++) z = mfma16(x[j], y[j], z);
-      }
       const float bs = bias[min(d, dim - 1)];
+      for (int r0 = 0; r0 < rank; r0 += 16) {
+        const f32x4 x = load_quad(low, r0 + 4 * lg, rank, lvec, true);
+        uint16_t y[4];
 #pragma unroll
-      for (int v = 0; v < 4; v++) {
-        const int tz = 16 * tt + 4 * lg + v;
-        Lg[tz * QS + d] = tz < nt && d < dim ? log2_decay(z[v] + bs, inv_tau) : 0.f;
+        for (int j = 0; j < 4; j++) y[j] = w[min(r0 + 4 * lg + j, rank - 1)];   // (x is zero past the rank)
+#pragma unroll
+        for (int j = 0; j < 4; j++) z = mfma16(x[j], __uint_as_float((uint32_t)y[j] << 16), z);
+      }
+      float s = 0.f, sum[4];
+#pragma unroll
+      for (int j = 0; j < 4; j++) {
+        const float ld = log2_decay(z[j] + bs, inv_tau);
+        s += 16 * b + 4 * lg + j < nt && d < dim ? ld : 0.f;
+        sum[j] = s;
+      }
+      float before = 0.f;                            // of the lane groups below
+#pragma unroll
+      for (int g = 0; g < 3; g++) {
+        const float o = __shfl(s, 16 * g + l15, kWave);
+        if (g < lg) before += o;
+      }
+#pragma unroll
+      for (int j = 0; j < 4; j++) Lg[(16 * b + 4 * lg + j) * QS + d] = before + sum[j];
+      if (lg == 3) {
+        tot[b * dp + d] = before + s;
+        if (before + s < -kFastRange) slow[b] = 1;   // (every writer stores the same value)
       }
     }
   }
 #pragma unroll
-  for (int i = 0; i < RW; i++) {
-    const int t = wave + 8 * i;
-    const bool live = t < nt;
-    if (lane < dp) {
-      Q[t * QS + lane] = live && lane < dim ? qr[i] * a.q_scale : 0.f;
-      K[t * QS + lane] = live && lane < dim ? kr[i] : 0.f;
-    }
-    if (lane < pb.vs) V[t * VS + lane] = live && lane < nvl ? vr[0][i] : 0.f;
-    if (lane + 64 < pb.vs) V[t * VS + lane + 64] = live && lane + 64 < nvl ? vr[1][i] : 0.f;
-  }
-  for (int d = lane + 64; d < dp; d += 64) {
-#pragma unroll
-    for (int i = 0; i < RW; i++) {
-      const float* p = row(wave + 8 * i);
-      qr[i] = p[qo + min(d, dim - 1)];
-      kr[i] = p[ko + min(d, dim - 1)];
-    }
-#pragma unroll
-    for (int i = 0; i < RW; i++) {
-      const int t = wave + 8 * i;
-      const bool live = t < nt && d < dim;
-      Q[t * QS + d] = live ? qr[i] * a.q_scale : 0.f;
-      K[t * QS + d] = live ? kr[i] : 0.f;
-    }
+  for (int i = 0; i < NV; i++) {
+    const int slot = tid + 512 * i, t = slot >> pb.vsh, c = 4 * (slot & vm);
+    if (t < C && c < pb.vs) *reinterpret_cast<f32x4*>(V + t * VS + c) = v[i];
   }
   __syncthreads();
-  for (int i = tid; i < NB * dp; i += 512) {         // running sums of the logs inside each block
-    const int b = i / dp, d = i - b * dp;
-    float s = 0.f, g[16];
+  bool any = false;
 #pragma unroll
-    for (int t = 0; t < 16; t++) g[t] = Lg[(16 * b + t) * QS + d];
+  for (int b = 0; b < NB; b++) any |= slow[b] != 0;
+  if (any) {   // diagonal blocks with strong decays, pair by pair from q and k as they are
 #pragma unroll
-    for (int t = 0; t < 16; t++) {
-      s += g[t];
-      Lg[(16 * b + t) * QS + d] = s;
+    for (int i = 0; i < NS; i++) {
+      const int slot = tid + 512 * i, t = slot >> pb.qsh, c = 4 * (slot & qm);
+      if (t < C && c < dp) {
+        *reinterpret_cast<f32x4*>(Q + t * QS + c) = q[i];
+        *reinterpret_cast<f32x4*>(K + t * QS + c) = k[i];
+      }
     }
-    tot[b * dp + d] = s;
-    if (s < -kFastRange) slow[b] = 1;                // (every writer stores the same value)
-  }
-  __syncthreads();
-  // diagonal blocks with strong decays, from q and k as they are
-  for (int b = 0; b < NB; b++) {
-    if (!slow[b]) continue;
-    if (tid < 256) {
+    __syncthreads();
+    for (int b = 0; b < NB; b++) {
+      if (!slow[b] || tid >= 256) continue;
       const int t = 16 * b + tid / 16, s = 16 * b + tid % 16;
       float acc = 0.f;
       if (s <= t)
         for (int d = 0; d < dim; d++) acc = fmaf(Q[t * QS + d] * K[s * QS + d], exp2_native(Lg[t * QS + d] - Lg[s * QS + d]), acc);
-      A[t * AS + s] = acc;
+      A[t * AS + s] = acc * a.q_scale;
+    }
+    __syncthreads();
+  }
+  // Q' and K'; decayed queries for linear_out_kernel, and the piece's decay products
+  const size_t hp = (size_t)h * pb.np + piece;
+#pragma unroll
+  for (int i = 0; i < NS; i++) {
+    const int slot = tid + 512 * i, t = slot >> pb.qsh, c = 4 * (slot & qm), b = t >> 4;
+    if (t >= C || c >= dp) continue;
+    const f32x4 L = *reinterpret_cast<const f32x4*>(Lg + t * QS + c), tt = *reinterpret_cast<const f32x4*>(tot + b * dp + c);
+    const f32x4 eq = exp2_quad(L), ek = exp2_quad(tt - L);
+    f32x4 x, y, e = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < 4; j++) { x[j] = q[i][j] * a.q_scale * eq[j]; y[j] = k[i][j] * ek[j]; }
+    *reinterpret_cast<f32x4*>(Q + t * QS + c) = x;
+    *reinterpret_cast<f32x4*>(K + t * QS + c) = y;
+    if (blockIdx.z == 0) {
+#pragma unroll
+      for (int m = 0; m < NB - 1; m++)
+        if (m < b) e += *reinterpret_cast<const f32x4*>(tot + m * dp + c);
+      *reinterpret_cast<f32x4*>(pb.qd + (hp * C + t) * dp + c) = x * exp2_quad(e);
     }
   }
-  __syncthreads();
-  for (int t = wave; t < C; t += 8)
-    for (int d = lane; d < dp; d += 64) {
-      const float L = Lg[t * QS + d];
-      Q[t * QS + d] *= exp2_native(L);
-      K[t * QS + d] *= exp2_native(tot[(t >> 4) * dp + d] - L);
+  if (blockIdx.z == 0)
+    for (int d = tid; d < dp; d += 512) {
+      float e = 0.f;
+#pragma unroll
+      for (int m = 0; m < NB; m++) e += tot[m * dp + d];
+      pb.dec[hp * dp + d] = exp2_native(e);
     }
   __syncthreads();
   // A[t][s]: 16 x 16 tiles on and below the diagonal, dealt over the wavefronts
@@ -165,77 +201,71 @@ __global__ __launch_bounds__(512) void linear_piece_kernel(const float* __restri
     f32x4 acc = {0.f, 0.f, 0.f, 0.f};
     for (int d0 = 0; d0 < dp; d0 += 16) {
       const int d = d0 + 4 * lg;
-      float4 q = *reinterpret_cast<const float4*>(Q + (16 * i + l15) * QS + d);
-      const float4 k = *reinterpret_cast<const float4*>(K + (16 * j + l15) * QS + d);
+      f32x4 qf = *reinterpret_cast<const f32x4*>(Q + (16 * i + l15) * QS + d);
+      const f32x4 kf = *reinterpret_cast<const f32x4*>(K + (16 * j + l15) * QS + d);
       if (i == j) {
-        const float* tp = tot + i * dp + d;
-        q.x *= exp2_native(-tp[0]); q.y *= exp2_native(-tp[1]); q.z *= exp2_native(-tp[2]); q.w *= exp2_native(-tp[3]);
+        qf *= exp2_quad(-*reinterpret_cast<const f32x4*>(tot + i * dp + d));
       } else if (i > j + 1) {
-        float4 e = make_float4(0.f, 0.f, 0.f, 0.f);
-        for (int m = j + 1; m < i; m++) {
-          const float* tp = tot + m * dp + d;
-          e.x += tp[0]; e.y += tp[1]; e.z += tp[2]; e.w += tp[3];
-        }
-        q.x *= exp2_native(e.x); q.y *= exp2_native(e.y); q.z *= exp2_native(e.z); q.w *= exp2_native(e.w);
+        f32x4 e = {0.f, 0.f, 0.f, 0.f};
+        for (int m = j + 1; m < i; m++) e += *reinterpret_cast<const f32x4*>(tot + m * dp + d);
+        qf *= exp2_quad(e);
       }
-      acc = mfma16(q.x, k.x, acc);
-      acc = mfma16(q.y, k.y, acc);
-      acc = mfma16(q.z, k.z, acc);
-      acc = mfma16(q.w, k.w, acc);
+#pragma unroll
+      for (int n = 0; n < 4; n++) acc = mfma16(qf[n], kf[n], acc);
     }
 #pragma unroll
-    for (int v = 0; v < 4; v++) {
-      const int t = 4 * lg + v;
-      A[(16 * i + t) * AS + 16 * j + l15] = i == j && l15 > t ? 0.f : acc[v];
+    for (int n = 0; n < 4; n++) {
+      const int t = 4 * lg + n;
+      A[(16 * i + t) * AS + 16 * j + l15] = i == j && l15 > t ? 0.f : acc[n];
     }
   }
-  const size_t hp = (size_t)h * pb.np + piece;
-  if (blockIdx.z == 0) {                             // decayed queries and the piece's decay products
-    for (int t = wave; t < C; t += 8)
-      for (int d = lane; d < dp; d += 64) {
-        float e = 0.f;
-        for (int m = 0; m < t >> 4; m++) e += tot[m * dp + d];
-        pb.qd[(hp * C + t) * dp + d] = Q[t * QS + d] * exp2_native(e);
-      }
-    for (int d = tid; d < dp; d += 512) {
-      float e = 0.f;
-      for (int m = 0; m < NB; m++) e += tot[m * dp + d];
-      pb.dec[hp * dp + d] = exp2_native(e);
-    }
-  }
-  // state term: sum over s of K'_sd 2^(totals after s's block) V_sv
-  for (int tile = wave; tile < (dp / 16) * (nv / 16); tile += 8) {
-    const int dt = tile / (nv / 16), vt = tile % (nv / 16), d = 16 * dt + l15;
-    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+  // state term: sum over s of K'_sd 2^(totals after s's block) V_sv; four value tiles share the keys
+  const int groups = (nv / 16 + 3) / 4;
+  for (int tile = wave; tile < (dp / 16) * groups; tile += 8) {
+    const int dt = tile / groups, vt = 4 * (tile % groups), d = 16 * dt + l15;
+    const int n4 = min(4, nv / 16 - vt);
+    f32x4 acc[4];
+#pragma unroll
+    for (int n = 0; n < 4; n++) acc[n] = f32x4{0.f, 0.f, 0.f, 0.f};
     float e = 0.f;
+#pragma unroll
     for (int b = NB - 1; b >= 0; b--) {
       const float w = exp2_native(e);
 #pragma unroll
       for (int j = 0; j < 4; j++) {
         const int s = 16 * b + 4 * lg + j;
-        acc = mfma16(K[s * QS + d] * w, V[s * VS + 16 * vt + l15], acc);
+        const float kw = K[s * QS + d] * w;
+#pragma unroll
+        for (int n = 0; n < 4; n++) acc[n] = mfma16(kw, V[s * VS + 16 * (vt + min(n, n4 - 1)) + l15], acc[n]);
       }
       e += tot[b * dp + d];
     }
 #pragma unroll
-    for (int v = 0; v < 4; v++) pb.st[(hp * dp + 16 * dt + 4 * lg + v) * vp + v0 + 16 * vt + l15] = acc[v];
+    for (int n = 0; n < 4; n++)
+      if (n < n4)
+#pragma unroll
+        for (int j = 0; j < 4; j++) pb.st[(hp * dp + 16 * dt + 4 * lg + j) * vp + v0 + 16 * (vt + n) + l15] = acc[n][j];
   }
   __syncthreads();
-  // inner output: A V
-  for (int tile = wave; tile < NB * (nv / 16); tile += 8) {
-    const int i = tile / (nv / 16), vt = tile % (nv / 16);
-    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+  // inner output: A V; the two wavefronts of a SIMD take a long and a short row of blocks
+  for (int tile = wave; tile < NB * groups; tile += 8) {
+    const int f = tile % NB, i = (tile / NB) & 1 ? NB - 1 - f : f, vt = 4 * (tile / NB), n4 = min(4, nv / 16 - vt);
+    f32x4 acc[4];
+#pragma unroll
+    for (int n = 0; n < 4; n++) acc[n] = f32x4{0.f, 0.f, 0.f, 0.f};
     for (int b = 0; b <= i; b++) {
       const int s = 16 * b + 4 * lg;
-      const float4 p = *reinterpret_cast<const float4*>(A + (16 * i + l15) * AS + s);
-      const float* vp4 = V + s * VS + 16 * vt + l15;
-      acc = mfma16(p.x, vp4[0], acc);
-      acc = mfma16(p.y, vp4[VS], acc);
-      acc = mfma16(p.z, vp4[2 * VS], acc);
-      acc = mfma16(p.w, vp4[3 * VS], acc);
+      const f32x4 p = *reinterpret_cast<const f32x4*>(A + (16 * i + l15) * AS + s);
+#pragma unroll
+      for (int j = 0; j < 4; j++)
+#pragma unroll
+        for (int n = 0; n < 4; n++) acc[n] = mfma16(p[j], V[(s + j) * VS + 16 * (vt + min(n, n4 - 1)) + l15], acc[n]);
     }
 #pragma unroll
-    for (int v = 0; v < 4; v++) pb.oi[(hp * C + 16 * i + 4 * lg + v) * vp + v0 + 16 * vt + l15] = acc[v];
+    for (int n = 0; n < 4; n++)
+      if (n < n4)
+#pragma unroll
+        for (int j = 0; j < 4; j++) pb.oi[(hp * C + 16 * i + 4 * lg + j) * vp + v0 + 16 * (vt + n) + l15] = acc[n][j];
   }
 }
 
@@ -381,7 +411,14 @@ int tlhip_linear_attn_chunk(const void* u, int64_t ldu, void* y, int64_t ldy, co
   pb.qd = pb.st + n_st;
   pb.oi = pb.qd + n_qd;
   const float* pu = static_cast<const float*>(u);
-  auto piece = pb.C == 64 ? linear_piece_kernel<64> : pb.C == 32 ? linear_piece_kernel<32> : linear_piece_kernel<16>;
+  while (4 << pb.qsh < pb.dp) pb.qsh++;
+  while (4 << pb.vsh < pb.vs) pb.vsh++;
+  const int quads = ((pb.C << pb.qsh) + 511) / 512;   // of queries (and keys) per thread
+  void (*piece)(const float*, int64_t, tlhip_linear_attn, int, PieceBuf) = nullptr;
+#define TLHIP_PIECE(C) (quads <= 2 ? linear_piece_kernel<C, 2> : quads <= 4 ? linear_piece_kernel<C, 4> : quads <= 8 ? linear_piece_kernel<C, 8> : nullptr)
+  piece = pb.C == 64 ? TLHIP_PIECE(64) : pb.C == 32 ? TLHIP_PIECE(32) : TLHIP_PIECE(16);
+#undef TLHIP_PIECE
+  if (!piece) return fail(TLHIP_EUNSUPPORTED, "tlhip_linear_attn_chunk: no kernel for this head size");
   hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(piece), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds1);
   if (e != hipSuccess) return hip_fail(e, "hipFuncSetAttribute(LDS)");
   hipLaunchKernelGGL(piece, dim3((unsigned)pb.np, (unsigned)la->heads, (unsigned)((pb.vp + pb.vs - 1) / pb.vs)), dim3(512), lds1,

@@ -14,7 +14,7 @@ namespace tlhip {
 // relative accuracy down to the smallest e: with w = fl(1 + e), log2(w) e / (w - 1) undoes w's rounding.
 __device__ __forceinline__ float log2_decay(float z, float inv_tau) {
   const float e = exp2_native(-fabsf(z) * kLog2e), w = 1.f + e;
-  const float l = w == 1.f ? e * kLog2e : log2_native(w) * (e / (w - 1.f));
+  const float l = w == 1.f ? e * kLog2e : log2_native(w) * (e * __builtin_amdgcn_rcpf(w - 1.f));
   return -(fmaxf(-z, 0.f) * kLog2e + l) * inv_tau;
 }
 // z of channel `ch` (head * dim + d): the low-rank product and its bias

@@ -177,19 +177,22 @@ __global__ __launch_bounds__(64 * NW, 1) void window_chunk_kernel(const float* _
 }
 
 // ---- two bf16 terms ------------------------------------------------------------------------------
-typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
-typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef uint32_t u32x2 __attribute__((ext_vector_type(2)));
+typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
 typedef float f32x2 __attribute__((ext_vector_type(2)));
 
-__device__ __forceinline__ void two_terms(f32x2 x, bf16x2& first, bf16x2& second) {
-  first = __builtin_convertvector(x, bf16x2);
-  const f32x2 back = __builtin_convertvector(first, f32x2);
-  f32x2 rest;
-  rest[0] = x[0] - back[0];
-  rest[1] = x[1] - back[1];
-  second = __builtin_convertvector(rest, bf16x2);
+// two f32 rounded to bf16 (nearest even): x0 in the low half. One v_cvt_pk_bf16_f32, left to the compiler:
+// it knows what must stand between a transcendental instruction and a reader of its result.
+typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
+__device__ __forceinline__ uint32_t bf16_pair(float x0, float x1) {
+  return __builtin_bit_cast(uint32_t, __builtin_convertvector(f32x2{x0, x1}, bf16x2));
 }
+__device__ __forceinline__ void two_terms(float x0, float x1, uint32_t& first, uint32_t& second) {
+  first = bf16_pair(x0, x1);
+  second = bf16_pair(x0 - bf16_lo(first), x1 - bf16_hi(first));
+}
+__device__ __forceinline__ bf16x8 as_bf16x8(u32x4 v) { return __builtin_bit_cast(bf16x8, v); }
 __device__ __forceinline__ f32x16 mfma_bf16(bf16x8 a, bf16x8 b, f32x16 c) {
   return __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, b, c, 0, 0, 0);
 }
@@ -215,7 +218,7 @@ __global__ __launch_bounds__(512, 1) void window_terms_kernel(const float* __res
                                                              const TermPlan plan, float* __restrict__ acc_out,
                                                              float* __restrict__ stat_out) {
   using L = TermLds<D>;
-  extern __shared__ __attribute__((aligned(16))) __bf16 bl[];
+  extern __shared__ __attribute__((aligned(16))) uint16_t bl[];
   const int tid = threadIdx.x, lane = tid & 63;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int l31 = lane & 31, hi = lane >> 5;
@@ -235,65 +238,71 @@ __global__ __launch_bounds__(512, 1) void window_terms_kernel(const float* __res
   const int kq = tid / (D / 2), d2 = 2 * (tid % (D / 2));
   const bool stages = tid < kTasks;
   f32x2 kreg[4];
-  const auto request = [&](f32x2 (&k)[4], int tile) {
-    tile = max(tile, kt0);
-    const float* base = ring + (size_t)((tile * 32) % R) * D + d2;
+  const auto request = [&](f32x2 (&k)[4], int tile, int first_row) {
+    const float* base = ring + (size_t)first_row * D + d2;
     const int last = kend - 1 - tile * 32;
 #pragma unroll
     for (int i = 0; i < 4; i++) k[i] = *reinterpret_cast<const f32x2*>(base + (size_t)min(4 * kq + i, last) * D);
   };
   const auto stage = [&](const f32x2 (&k)[4], int buf) {
-    __bf16 *K = bl + buf * L::kBuf, *KT = K + 2 * L::kK;
-    bf16x4 t0[2], t1[2];               // [column] four keys: first and second terms
+    uint16_t *K = bl + buf * L::kBuf, *KT = K + 2 * L::kK;
+    uint32_t t0[4], t1[4];             // of each key: both columns' first and second terms
 #pragma unroll
     for (int i = 0; i < 4; i++) {
-      bf16x2 f, g;
-      two_terms(k[i], f, g);
-      *reinterpret_cast<bf16x2*>(K + (4 * kq + i) * L::kKRow + d2) = f;
-      *reinterpret_cast<bf16x2*>(K + L::kK + (4 * kq + i) * L::kKRow + d2) = g;
-      t0[0][i] = f[0]; t0[1][i] = f[1];
-      t1[0][i] = g[0]; t1[1][i] = g[1];
+      two_terms(k[i][0], k[i][1], t0[i], t1[i]);
+      *reinterpret_cast<uint32_t*>(K + (4 * kq + i) * L::kKRow + d2) = t0[i];
+      *reinterpret_cast<uint32_t*>(K + L::kK + (4 * kq + i) * L::kKRow + d2) = t1[i];
     }
     // keys 4kq .. 4kq + 3 are elements 4 (kq / 2 % 2) .. of key step kq / 4, lane half kq % 2
     const int unit = ((kq >> 2) * 2 + (kq & 1)) * D + d2, off = 4 * ((kq >> 1) & 1);
+    const auto column = [](const uint32_t (&t)[4], uint32_t pick) {
+      return u32x2{__builtin_amdgcn_perm(t[1], t[0], pick), __builtin_amdgcn_perm(t[3], t[2], pick)};
+    };
 #pragma unroll
     for (int c = 0; c < 2; c++) {
-      *reinterpret_cast<bf16x4*>(KT + (unit + c) * 8 + off) = t0[c];
-      *reinterpret_cast<bf16x4*>(KT + L::kT + (unit + c) * 8 + off) = t1[c];
+      const uint32_t pick = c ? 0x07060302u : 0x05040100u;   // the high or low halves of two words
+      *reinterpret_cast<u32x2*>(KT + (unit + c) * 8 + off) = column(t0, pick);
+      *reinterpret_cast<u32x2*>(KT + L::kT + (unit + c) * 8 + off) = column(t1, pick);
     }
   };
   // newest keys first: the distance bias makes them the likely maxima, which then seldom move
   int kt = kt1 - 1 - (int)blockIdx.z;
-  if (stages) request(kreg, kt);
+  int row = kt >= kt0 ? (kt * 32) % R : 0;             // of tile kt in the ring; a step back is 32 S rows
+  const int back = (32 * plan.S) % R;
+  if (stages && kt >= kt0) request(kreg, kt, row);
 
   // queries times their temperature, cut into terms: lane (hi, l31) holds columns 16s + 8hi .. + 7 of query l31
   bf16x8 q0[D / 16], q1[D / 16];
   {
-    const int t = min(max(p0, 0) + l31, T - 1);
+    const int t = min(p0 + l31, T - 1);
     const float temp = query_temperature(pos0 + t, a.temp_coef, a.temp_every);
-    const float* q = u + (size_t)t * ldu + a.q_off + (size_t)min(h, heads - 1) * dim;
-    const bool vec = (reinterpret_cast<uintptr_t>(q) & 15) == 0 && (dim & 3) == 0 && (ldu & 3) == 0;
+    const int64_t qo = a.q_off + (int64_t)min(h, heads - 1) * dim;
+    const float* q = u + (size_t)t * ldu + qo;
+    f32x4 x[D / 8];
+    // (uniform: every row of queries starts on 16 bytes and holds whole quads)
+    if (((reinterpret_cast<uintptr_t>(u) & 15) | ((qo | ldu | dim) & 3)) == 0) {
+#pragma unroll
+      for (int i = 0; i < D / 8; i++) x[i] = *reinterpret_cast<const f32x4*>(q + min(16 * (i >> 1) + 8 * hi + 4 * (i & 1), dim - 4));
+    } else {
+#pragma unroll
+      for (int i = 0; i < D / 8; i++)
+#pragma unroll
+        for (int j = 0; j < 4; j++) x[i][j] = q[min(16 * (i >> 1) + 8 * hi + 4 * (i & 1) + j, dim - 1)];
+    }
 #pragma unroll
     for (int s = 0; s < D / 16; s++) {
-      f32x4 x[2];
+      u32x4 f, g;
 #pragma unroll
-      for (int k = 0; k < 2; k++) {
-        const int d = 16 * s + 8 * hi + 4 * k;
-        if (vec) {                     // (the head's row starts on 16 bytes and holds whole quads)
-          x[k] = *reinterpret_cast<const f32x4*>(q + min(d, dim - 4));
-          if (d >= dim) x[k] = f32x4{0.f, 0.f, 0.f, 0.f};
-        } else {
-#pragma unroll
-          for (int j = 0; j < 4; j++) x[k][j] = d + j < dim ? q[d + j] : 0.f;
-        }
+      for (int j = 0; j < 4; j++) {
+        const int d = 16 * s + 8 * hi + 2 * j;
+        const f32x4 v = x[2 * s + (j >> 1)];
+        uint32_t f1, g1;
+        two_terms(d < dim ? v[2 * (j & 1)] * temp : 0.f, d + 1 < dim ? v[2 * (j & 1) + 1] * temp : 0.f, f1, g1);
+        f[j] = f1;
+        g[j] = g1;
       }
-#pragma unroll
-      for (int j = 0; j < 8; j += 2) {
-        bf16x2 f, g;
-        two_terms(f32x2{x[j >> 2][j & 3] * temp, x[j >> 2][(j & 3) + 1] * temp}, f, g);
-        q0[s][j] = f[0]; q0[s][j + 1] = f[1];
-        q1[s][j] = g[0]; q1[s][j + 1] = g[1];
-      }
+      q0[s] = as_bf16x8(f);
+      q1[s] = as_bf16x8(g);
     }
   }
   f32x16 o[D / 32];
@@ -305,12 +314,17 @@ __global__ __launch_bounds__(512, 1) void window_terms_kernel(const float* __res
   const int qpos = pos0 + p0 + l31;
   const float sc2 = a.scale * kLog2e, sl2 = head_slope(h, heads, a.slope_exp) * kLog2e;
 
+  const auto step_back = [&] {
+    row -= back;
+    if (row < 0) row += R;
+  };
   if (stages && kt >= kt0) stage(kreg, 0);
-  if (stages) request(kreg, kt - plan.S);
+  step_back();
+  if (stages && kt - plan.S >= kt0) request(kreg, kt - plan.S, row);
   __syncthreads();
   for (int buf = 0; kt >= kt0; kt -= plan.S, buf ^= 1) {
     if (kt >= wt0 && kt < wt1) {
-      const __bf16 *K = bl + buf * L::kBuf, *KT = K + 2 * L::kK;
+      const uint16_t *K = bl + buf * L::kBuf, *KT = K + 2 * L::kK;
       f32x16 s, r;                     // first x first, and the two mixed pairs
 #pragma unroll
       for (int v = 0; v < 16; v++) { s[v] = 0.f; r[v] = 0.f; }
@@ -342,35 +356,34 @@ __global__ __launch_bounds__(512, 1) void window_terms_kernel(const float* __res
 #pragma unroll
           for (int v = 0; v < 16; v++) o[dt][v] *= corr;
       }
-      bf16x8 w0[2], w1[2];
+      u32x4 w0[2], w1[2];
       float ps = 0.f;
 #pragma unroll
       for (int v = 0; v < 16; v += 2) {
-        f32x2 p;
-        p[0] = exp2_native(s[v] - ref);
-        p[1] = exp2_native(s[v + 1] - ref);
-        ps += p[0] + p[1];
-        bf16x2 f, g;
-        two_terms(p, f, g);
-        w0[v >> 3][v & 7] = f[0]; w0[v >> 3][(v & 7) + 1] = f[1];
-        w1[v >> 3][v & 7] = g[0]; w1[v >> 3][(v & 7) + 1] = g[1];
+        const float pa = exp2_native(s[v] - ref), pb = exp2_native(s[v + 1] - ref);
+        ps += pa + pb;
+        uint32_t f, g;
+        two_terms(pa, pb, f, g);
+        w0[v >> 3][(v & 7) >> 1] = f;
+        w1[v >> 3][(v & 7) >> 1] = g;
       }
       lsum += ps;
 #pragma unroll
       for (int st = 0; st < 2; st++)
 #pragma unroll
         for (int dt = 0; dt < D / 32; dt++) {
-          const __bf16* p = KT + ((st * 2 + hi) * D + dt * 32 + l31) * 8;
+          const uint16_t* p = KT + ((st * 2 + hi) * D + dt * 32 + l31) * 8;
           const bf16x8 v0 = *reinterpret_cast<const bf16x8*>(p);
           const bf16x8 v1 = *reinterpret_cast<const bf16x8*>(p + L::kT);
-          o[dt] = mfma_bf16(v1, w0[st], o[dt]);
-          o[dt] = mfma_bf16(v0, w1[st], o[dt]);
-          o[dt] = mfma_bf16(v0, w0[st], o[dt]);
+          o[dt] = mfma_bf16(v1, as_bf16x8(w0[st]), o[dt]);
+          o[dt] = mfma_bf16(v0, as_bf16x8(w1[st]), o[dt]);
+          o[dt] = mfma_bf16(v0, as_bf16x8(w0[st]), o[dt]);
         }
     }
     // the next tile into the other buffer (last read before the barrier that ended the turn before)
     if (stages && kt - plan.S >= kt0) stage(kreg, buf ^ 1);
-    if (stages) request(kreg, kt - 2 * plan.S);
+    step_back();
+    if (stages && kt - 2 * plan.S >= kt0) request(kreg, kt - 2 * plan.S, row);
     __syncthreads();
   }
   const int t = p0 + l31;
@@ -389,14 +402,24 @@ __global__ __launch_bounds__(512, 1) void window_terms_kernel(const float* __res
     return;
   }
   const float inv = a.out_scale / Ls;
-  const float* gp = u + (size_t)t * ldu + a.gate_off + (size_t)h * dim;
+  if (a.gate_off >= 0) {
+    const float* gp = u + (size_t)t * ldu + a.gate_off + (size_t)h * dim;
+#pragma unroll
+    for (int dt = 0; dt < D / 32; dt++) {
+      float g[16];
+#pragma unroll
+      for (int v = 0; v < 16; v++) g[v] = gp[min(dt * 32 + 8 * (v >> 2) + 4 * hi + (v & 3), dim - 1)];
+#pragma unroll
+      for (int v = 0; v < 16; v++) o[dt][v] *= sigmoid_f(g[v]);
+    }
+  }
   float* yp = y + (size_t)t * ldy + a.y_off + (size_t)h * dim;
 #pragma unroll
   for (int dt = 0; dt < D / 32; dt++)
 #pragma unroll
     for (int v = 0; v < 16; v++) {
       const int d = dt * 32 + 8 * (v >> 2) + 4 * hi + (v & 3);
-      if (d < dim) yp[d] = o[dt][v] * inv * (a.gate_off >= 0 ? sigmoid_f(gp[d]) : 1.f);
+      if (d < dim) yp[d] = o[dt][v] * inv;
     }
 }
 

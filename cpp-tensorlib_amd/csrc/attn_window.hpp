@@ -223,20 +223,32 @@ __device__ __forceinline__ void window_step_block(const tlhip_window_attn& a, co
 __device__ __forceinline__ void window_merge_head(const tlhip_window_attn& a, const float* __restrict__ u,
                                                   float* __restrict__ y, const float* __restrict__ partials, int head,
                                                   int S) {
-  const int dim = (int)a.dim, ld = (int)a.ring_ld;
-  const float* p = partials + (size_t)head * S * (ld + 2);
+  constexpr int U = 8;                                 // splits requested at once
+  const int dim = (int)a.dim, ps = (int)a.ring_ld + 2;
+  const float* p = partials + (size_t)head * S * ps;
   for (int d = threadIdx.x; d < dim; d += blockDim.x) {
-    float M = -INFINITY;
-    for (int s = 0; s < S; s++) M = fmaxf(M, p[(size_t)s * (ld + 2)]);
-    float L = 0.f, o = 0.f;
-    for (int s = 0; s < S; s++) {
-      const float* ps = p + (size_t)s * (ld + 2);
-      const float f = ps[0] == -INFINITY ? 0.f : exp2_native(ps[0] - M);
-      L = fmaf(f, ps[1], L);
-      o = fmaf(f, ps[2 + d], o);
+    const float g = a.gate_off >= 0 ? u[a.gate_off + (int64_t)head * dim + d] : 0.f;
+    float M = -INFINITY, L = 0.f, o = 0.f;
+    for (int s0 = 0; s0 < S; s0 += U) {
+      float m[U], l[U], v[U];
+#pragma unroll
+      for (int k = 0; k < U; k++) {
+        const float* q = p + (size_t)min(s0 + k, S - 1) * ps;
+        m[k] = q[0];
+        l[k] = q[1];
+        v[k] = q[2 + d];
+      }
+#pragma unroll
+      for (int k = 0; k < U; k++) {
+        if (s0 + k >= S || m[k] == -INFINITY) continue;
+        const float n = fmaxf(M, m[k]), fo = exp2_native(M - n), fn = exp2_native(m[k] - n);
+        M = n;
+        L = L * fo + fn * l[k];
+        o = o * fo + fn * v[k];
+      }
     }
     float v = o / L * a.out_scale;
-    if (a.gate_off >= 0) v *= sigmoid_f(u[a.gate_off + (int64_t)head * dim + d]);
+    if (a.gate_off >= 0) v *= sigmoid_f(g);
     y[a.y_off + (int64_t)head * dim + d] = v;
   }
 }

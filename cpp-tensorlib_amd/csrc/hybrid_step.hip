@@ -21,9 +21,10 @@ constexpr int kPolySlice = 1024;   // ff values a polynorm block writes
 constexpr int kMaxSplits = 32;
 
 static int attn_splits(const tlhip_window_attn* a) {
-  // about 32 keys per stream (a block holds 32 of them); the plan does not depend on the position
-  int64_t S = (a->window + 1023) / 1024;
-  return (int)(S < 1 ? 1 : S > kMaxSplits ? kMaxSplits : S);
+  // What a block reads bounds it (a CU takes in some 100 bytes per ns): windows beyond 192 KB of keys are
+  // cut into splits of about 64 KB, which costs the merge launch. The plan does not depend on the position.
+  const int64_t bytes = a->window * tlhip_window_ring_ld(a->dim) * 4, S = bytes <= (192 << 10) ? 1 : (bytes + (64 << 10) - 1) / (64 << 10);
+  return (int)(S > kMaxSplits ? kMaxSplits : S);
 }
 static MixPlan make_plan(const tlhip_window_attn* at, const tlhip_linear_attn* la, const tlhip_polynorm* pn) {
   MixPlan p{1, 0, 1, 0, 0, 0};

@@ -164,7 +164,7 @@ class LinearAttn(C.Structure):
 
 class PolyNorm(C.Structure):
     """tlhip_polynorm"""
-    _fields_ = [(n, i64) for n in ("ff", "z_off", "y_off")] + [(n, f32) for n in ("a", "b", "c", "e", "eps")]
+    _fields_ = [(n, i64) for n in ("ff", "z_off", "y_off")] + [(n, f32) for n in ("c1", "c2", "c3", "c0", "eps")]
 
 
 class TlHipError(RuntimeError):

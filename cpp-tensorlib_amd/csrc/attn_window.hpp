@@ -1,8 +1,8 @@
 // Sliding-window attention whose values are its keys: what the decode step (hybrid_step.hip) and the
 // prompt-chunk kernel (attn_window.hip) share, and the decode step's block.
 //
-//   score(i, j) = (q_i t(i)) . k_j scale - slope_h (i - j),   0 <= i - j < window
-//   out_i = softmax_j(score) . k_j
+//   score of the key d places back (d < window): scale t <q_i, k_(i-d)> - d slope
+//   out_i = the keys weighted by the softmax of their scores
 //
 // A key row is loaded once and serves both products.
 #pragma once

@@ -1,5 +1,5 @@
 // Prompt chunks of the gated linear attention. The recurrence
-//   S_t = diag(a_t) S_(t-1) + k_t v_t^T,   o_t = S_t^T q_t
+//   state row c <- a_c row_c + k_c v,   o = sum_c q_c row_c
 // over pieces of C tokens: with b_t the base-2 log of the decay product since the piece began,
 //   o_t = (q_t 2^b_t) S_0 + sum_(s <= t) [sum_d q_td k_sd 2^(b_td - b_sd)] v_s
 //   S_C = 2^b_C S_0 + sum_s (k_s 2^(b_C - b_s)) v_s^T.

@@ -1,7 +1,7 @@
 // Gated linear attention: what the decode step (hybrid_step.hip) and the prompt-chunk kernels
 // (linear_attn.hip) share, and the decode step's block.
 //
-//   S_t = diag(a_t) S_(t-1) + k_t v_t^T,   o_t = S_t^T q_t,   a_t = sigmoid(z_t)^(1/tau)
+//   state row c <- a_c row_c + k_c v,   o = sum_c q_c row_c,   ln a_c = -softplus(-z_c) / tau
 //
 // Everything is f32. Decays are kept as base-2 logarithms.
 #pragma once
@@ -10,7 +10,7 @@
 
 namespace tlhip {
 
-// log2 of sigmoid(z)^(1/tau) = -log2(1 + e^-z) / tau, from e = e^-|z| <= 1. log2(1 + e) keeps e's
+// log2 of the decay, -log2(1 + e^-z) / tau, from e = e^-|z| <= 1. log2(1 + e) keeps e's
 // relative accuracy down to the smallest e: with w = fl(1 + e), log2(w) e / (w - 1) undoes w's rounding.
 __device__ __forceinline__ float log2_decay(float z, float inv_tau) {
   const float e = exp2_native(-fabsf(z) * kLog2e), w = 1.f + e;

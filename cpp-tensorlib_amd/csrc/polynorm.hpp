@@ -1,4 +1,4 @@
-// y = a N(z) + b N(z^2) + c N(z^3) + e, N(w) = w / sqrt(mean(w^2) + eps) over a row of ff values.
+// A cubic whose powers are each scaled to unit mean square over a row of ff values (tlhip_polynorm).
 #pragma once
 
 #include "common.hpp"
@@ -33,7 +33,7 @@ __device__ __forceinline__ PolyCoef poly_coef(const tlhip_polynorm& p, PolySums 
 #pragma unroll
   for (int w = 0; w < NW; w++) { s.s2 += red[w]; s.s4 += red[NW + w]; s.s6 += red[2 * NW + w]; }
   const float inv = 1.0f / (float)p.ff;
-  return PolyCoef{p.a / sqrtf(s.s2 * inv + p.eps), p.b / sqrtf(s.s4 * inv + p.eps), p.c / sqrtf(s.s6 * inv + p.eps), p.e};
+  return PolyCoef{p.c1 / sqrtf(s.s2 * inv + p.eps), p.c2 / sqrtf(s.s4 * inv + p.eps), p.c3 / sqrtf(s.s6 * inv + p.eps), p.c0};
 }
 
 // Elements [i0, i1) of one row by a block of NT threads; the three means are taken over the whole row

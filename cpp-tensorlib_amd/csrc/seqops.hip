@@ -5,7 +5,7 @@
 
 namespace tlhip {
 
-// Angles in double: p * 10000^(-2i/width) loses digits in fp32 at positions in the thousands.
+// Angles in double: a position times a frequency loses digits in fp32 at positions in the thousands.
 __global__ __launch_bounds__(256) void embed_sinusoid_kernel(const uint16_t* __restrict__ table, const int* __restrict__ tokens,
                                                              float* __restrict__ out, int width, int ld, int vocab, int pos0,
                                                              const uint32_t* __restrict__ d_pos) {

@@ -1608,7 +1608,7 @@ struct linear_attn {
 };
 struct polynorm {
   int64_t ff = 0, z_off = 0, y_off = 0;
-  float a = 0, b = 0, c = 0, e = 0, eps = 0;
+  float c1 = 0, c2 = 0, c3 = 0, c0 = 0, eps = 0;
 };
 inline int64_t window_ring_ld(int64_t dim) {
   auto& c = context::get();

@@ -61,7 +61,7 @@ struct config {
   int64_t loop_start = 0, loop_stop = 0, loop_times = 0;   // times 0: no loop
 };
 
-constexpr float kSlopeExp = 8.0f;    // slope of head h: 2^(-8 (h + 1) / heads)
+constexpr float kSlopeExp = 8.0f;    // the heads' distance slopes: powers 1, 2, .. of 2^(-kSlopeExp/heads)
 constexpr const char* kArchitecture = "Lusadra";
 
 inline config parse_config(const json::value& j) {
@@ -351,7 +351,7 @@ inline void build(model& M, const config& cfg, detail::source& src, int64_t max_
       const std::vector<float> act = floats(p + "mlp.act", 4);
       hip::polynorm& n = L.pn;
       n.ff = lc.ff;
-      n.a = act[0]; n.b = act[1]; n.c = act[2]; n.e = act[3];
+      n.c1 = act[0]; n.c2 = act[1]; n.c3 = act[2]; n.c0 = act[3];
       n.eps = cfg.eps;
       n.z_off = seg(in, nu, p + "mlp.up", lc.ff);
       n.y_off = seg(out, ny, p + "mlp.down", lc.ff);

@@ -466,11 +466,12 @@ int tlhip_merge_heads(const void* src, void* dst, int64_t T, int64_t H, int64_t 
  * structs below say where a sublayer's columns lie in u and y (element offsets into a row) and hold
  * its sizes and constants. Sizes are free unless stated; a refusal is TLHIP_EUNSUPPORTED.
  *
- * Sliding-window attention whose values are its keys. Position i sees j with 0 <= i - j < window;
- * score = (q_i * t(i)) . k_j * scale - slope_h (i - j), with
- *   t(p) = 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1)     (temp_every <= 0: 1), and
- *   slope_h = 2^(-slope_exp (h + 1) / heads)                       (slope_exp <= 0: no bias);
- * y = out_scale * softmax(score) . k, times sigmoid(gate) when gate_off >= 0.
+ * Sliding-window attention whose values are its keys. The query at position i meets the key d = 0, 1, ..
+ * window - 1 places before it with the score scale * t * <q_i, k_(i-d)> - d * r^(h+1), where
+ *   t = 1 + temp_coef ln(1 + n), n = the number of whole runs of temp_every positions in 0 .. i
+ *       (temp_every <= 0: t = 1),
+ *   r = 2^(-slope_exp/heads): the per-position bias of head h is r to the power h + 1 (slope_exp <= 0: none).
+ * y = out_scale * sum over d of softmax_d k_(i-d), times sigmoid(gate) when gate_off >= 0.
  * Keys live in a ring: position p in row p % ring_rows, [kv_heads][ring_rows][ring_ld] f32,
  * ring_ld = tlhip_window_ring_ld(dim) with zeros past dim, ring_rows a multiple of 32 and at least
  * window - 1 + (rows of the longest chunk). The whole ring must be zeroed before its first use. */
@@ -483,9 +484,10 @@ typedef struct {
 } tlhip_window_attn;
 int64_t tlhip_window_ring_ld(int64_t dim);   /* 0: dim beyond what the kernels hold (256) */
 
-/* Gated linear attention. Per head, S [dim][vdim]: S_t = diag(a_t) S_(t-1) + k_t v_t^T,
- * o_t = S_t^T (q_t * q_scale), a_t = sigmoid(z)^(1/tau), z = A2 (low) + bias with low the rank
- * columns at low_off, A2 bf16 [heads*dim][rank]; y = out_scale * rmsnorm_vdim(o) * norm * silu(gate).
+/* Gated linear attention. Per head a state of dim rows of vdim; a token turns every row into
+ *   row_c <- a_c row_c + k_c v,   ln a_c = -softplus(-z_c) / tau,   and reads   o = q_scale sum_c q_c row_c.
+ * z = A2 (low) + bias with low the rank columns at low_off, A2 bf16 [heads*dim][rank];
+ * y = out_scale * rmsnorm_vdim(o) * norm * silu(gate).
  * The state has two slots of tlhip_linear_state_bytes / 2 bytes, [heads][dim][vdim rounded up to 4]:
  * the state ahead of position p is slot p % 2, and the step at p (chunk p .. p + T - 1) writes slot
  * (p + 1) % 2 ((p + T) % 2): a step can be repeated at its position. At position 0 the state is
@@ -499,11 +501,11 @@ typedef struct {
 } tlhip_linear_attn;
 int64_t tlhip_linear_state_bytes(int64_t heads, int64_t dim, int64_t vdim);
 
-/* y = a N(z) + b N(z^2) + c N(z^3) + e over the row's ff values; powers element by element,
- * N(w) = w / sqrt(mean(w^2) + eps). */
+/* A cubic whose powers are each scaled to unit mean square over the row's ff values:
+ * y_i = c0 + sum over m = 1, 2, 3 of c_m z_i^m / sqrt(eps + mean_j z_j^(2m)). */
 typedef struct {
   int64_t ff, z_off, y_off;
-  float a, b, c, e, eps;
+  float c1, c2, c3, c0, eps;
 } tlhip_polynorm;
 
 /* One token: u [one row] -> y [one row] for the sublayers given (NULL: not there), all in one launch
@@ -526,8 +528,8 @@ int tlhip_linear_attn_chunk(const void* u, int64_t ldu, void* y, int64_t ldy, co
 int tlhip_polynorm_rows(const void* u, int64_t ldu, void* y, int64_t ldy, const tlhip_polynorm* pn, int64_t T);
 
 /* out[t][ld] f32 = widened bf16 row tokens[t] of a [vocab, width] table + the sinusoid of position
- * pos0 + t (or *d_pos + t): column 2i adds sin(p 10000^(-2i/width)), column 2i + 1 the cosine; columns
- * width .. ld - 1 are zero. tokens: device int32, clamped to [0, vocab). */
+ * p = pos0 + t (or *d_pos + t): columns pair up, an even column c adds sin and the next one cos of the
+ * angle p / 10000^(c/width); columns width .. ld - 1 are zero. tokens: device int32, clamped to [0, vocab). */
 int tlhip_embed_sinusoid(const void* table, const void* tokens, void* out, int64_t T, int64_t width,
                          int64_t ld, int64_t vocab, int64_t pos0, const void* d_pos);
 /* out[t] = x[t] + parts[0][t] + ... + parts[S-1][t] + add[t] + vec, rows of n; parts, add and vec may

@@ -9,7 +9,7 @@ F = np.float64
 
 
 def rms(x, eps):
-    """x divided by its root mean square over the last axis."""
+    """Rows scaled to unit root mean square (last axis)."""
     return x / np.sqrt(np.mean(x * x, axis=-1, keepdims=True) + eps)
 
 
@@ -18,7 +18,7 @@ def sigmoid(z):
 
 
 def position_vector(p, width):
-    """Sinusoids: coordinate 2i is sin(p * 10000^(-2i/width)), coordinate 2i + 1 its cosine."""
+    """Pairs of coordinates: sine and cosine of p over a wavelength that grows with the pair."""
     out = np.zeros(width, F)
     for c in range(width):
         i = c // 2
@@ -37,8 +37,8 @@ def slope(h, heads):
 
 def window_attention(q, k, heads, kv_heads, dim, window, scale, coef, every, pos0=0):
     """q [T, heads*dim] for positions pos0 .. pos0+T-1, k [pos0+T, kv_heads*dim] for all positions;
-    the values are the keys. Position i sees j with 0 <= i - j < window; the score loses
-    slope * (i - j)."""
+    the values are the keys. A query meets itself and the window - 1 keys before it; a key loses slope
+    for every position it lies back."""
     T = q.shape[0]
     out = np.zeros((T, heads * dim), F)
     for t in range(T):
@@ -55,13 +55,13 @@ def window_attention(q, k, heads, kv_heads, dim, window, scale, coef, every, pos
 
 
 def decays(z, tau):
-    """alpha = sigmoid(z)^(1/tau)"""
+    """Share of a state row that outlives one token, from its logit."""
     return sigmoid(z) ** (1.0 / tau)
 
 
 def gated_linear_attention(q, k, v, alpha, heads, dim, vdim, state=None):
-    """Per head S_t = diag(alpha_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t; returns o [T, heads*vdim]
-    and the last state [heads, dim, vdim]. q is taken as scaled already."""
+    """Per head and token: every state row decays by its alpha and takes k_c v, then q reads the rows.
+    Returns o [T, heads*vdim] and the last state [heads, dim, vdim]. q is taken as scaled already."""
     T = q.shape[0]
     S = np.zeros((heads, dim, vdim), F) if state is None else state.copy()
     o = np.zeros((T, heads * vdim), F)
@@ -82,9 +82,9 @@ def head_norm(o, w, heads, vdim, eps):
     return out
 
 
-def polynorm(z, abce, eps):
-    a, b, c, e = abce
-    return a * rms(z, eps) + b * rms(z ** 2, eps) + c * rms(z ** 3, eps) + e
+def polynorm(z, coef, eps):
+    c1, c2, c3, c0 = coef
+    return c1 * rms(z, eps) + c2 * rms(z ** 2, eps) + c3 * rms(z ** 3, eps) + c0
 
 
 def left_mixer(h, W, p, c, pos0, past):

@@ -305,7 +305,7 @@ def test_linear_attention_keeps_a_far_token(lib, capi):
 def test_polynorm(lib, capi, ff):
     T, W, ldy = 5, (ff + 3) // 4 * 4 + 4, ff + 9
     u = (2 * rng(ff).standard_normal((T, W))).astype(np.float32)
-    pn = capi.PolyNorm(ff=ff, z_off=4, y_off=3, a=0.7, b=-0.4, c=0.9, e=0.2, eps=1e-5)
+    pn = capi.PolyNorm(ff=ff, z_off=4, y_off=3, c1=0.7, c2=-0.4, c3=0.9, c0=0.2, eps=1e-5)
     want = O.polynorm(u[:, 4:4 + ff].astype(np.float64), (0.7, -0.4, 0.9, 0.2), 1e-5)
     dy = lib.to_device(np.zeros((T, ldy), np.float32))
     lib.polynorm_rows(lib.to_device(u), W, dy, ldy, pn, T)
@@ -326,7 +326,7 @@ def test_all_sublayers_in_one_launch_equal_each_alone(lib, capi):
     for f in ("q_off", "k_off", "v_off", "gate_off", "low_off"):
         setattr(l.la, f, getattr(l.la, f) + w.W)
     l.la.y_off = w.ldy
-    pn = capi.PolyNorm(ff=ff, z_off=w.W + l.W, y_off=w.ldy + l.ldy, a=0.5, b=0.2, c=0.1, e=-0.3, eps=1e-6)
+    pn = capi.PolyNorm(ff=ff, z_off=w.W + l.W, y_off=w.ldy + l.ldy, c1=0.5, c2=0.2, c3=0.1, c0=-0.3, eps=1e-6)
     ldy = w.ldy + l.ldy + ff
     u = rng(11).standard_normal((8, W)).astype(np.float32)
     for t in range(8):

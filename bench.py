@@ -593,7 +593,7 @@ def bench_lusadra(lib, steps, only=None):
         h, d, v = z["right"]
         E, n = z["width"], z["layers"]
         per_layer = E * (3 * H * D + G * D + 2 * h * d + 3 * h * v + 16 + 2 * z["ff"])
-        m = Model.random_lusadra(lusadra_config(z), seed=1, rank=16, max_ctx=8192)
+        m = Model.random(lusadra_config(z), seed=1, rank=16, max_ctx=8192)
         m.stage_chunk(ids)
         for p0 in range(0, 3584, T):
             m.chunk_layers(T, p0)

@@ -15,7 +15,8 @@ LIBDIR = os.path.join(HERE, "lib")
 OBJDIR = os.path.join(HERE, "build")
 LIB = os.path.join(LIBDIR, "libtensorlib_hip.so")
 SOURCES = ["runtime.hip", "gemv.hip", "elementwise.hip", "modelops.hip", "attn.hip", "attn_prefill_mfma.hip", "attn_prefill_f16.hip", "prefill.hip", "gemm_f16t.hip", "convert.hip", "sgemm.hip",
-           "attn_window.hip", "linear_attn.hip", "hybrid_step.hip", "seqops.hip"]
+           "attn_window.hip", "linear_attn.hip", "hybrid_step.hip", "seqops.hip",
+           "ssm.hip", "latent_attn.hip"]
 # -packed-fp32-ops off: hipcc must not form v_pk_*_f32 on this pool.
 FLAGS = ["-O3", "-std=c++17", "--offload-arch=gfx950", "-fPIC", "-fno-gpu-rdc",
          "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",

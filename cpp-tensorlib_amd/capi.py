@@ -25,7 +25,8 @@ OPS = dict(add=0, sub=1, mul=2, div=3, pow=4, exp=5, log=6, sqrt=7, sigmoid=8, r
 CENSUS = ["binary", "bcast", "unary", "row_op", "gemm", "gemv_f32", "gemv_bf16", "gemv_bf16_row",
           "gemv_q4", "attn_decode", "rope", "rmsnorm", "rmsnorm_res", "swiglu", "argmax",
           "kv_append", "kv_fill", "split_heads", "merge_heads", "gemm_bf16_nt", "attn_prefill",
-          "convert", "quantize_q4", "mix_step", "window_attn", "linear_attn", "polynorm", "embed", "residual"]
+          "convert", "quantize_q4", "mix_step", "window_attn", "linear_attn", "polynorm", "embed", "residual",
+          "ssm", "latent_attn", "act"]
 
 # name -> (restype, argtypes): exactly the declarations of include/tensorlib_hip.h
 SIGNATURES = {
@@ -135,6 +136,18 @@ SIGNATURES = {
     "tlhip_embed_sinusoid": (cint, [P, P, P, i64, i64, i64, i64, i64, P]),
     "tlhip_residual_sum": (cint, [P, P, i64, P, P, P, i64, i64]),
     "tlhip_gather_rows": (cint, [P, P, P, i64, i64, i64]),
+    "tlhip_gemv_bf16_row_postnorm": (cint, [P, P, P, P, i64, i64, P, P, P, i64, i64, f32]),
+    "tlhip_gemv_bf16_row_postnorm_geglu": (cint, [P, P, P, P, P, P, P, P, i64, i64, f32]),
+    "tlhip_postnorm_res_parts": (cint, [P, P, i64, P, P, P, i64, f32, i64, P]),
+    "tlhip_rms_rows": (cint, [P, i64, P, P, i64, i64, i64, i64, f32, i64]),
+    "tlhip_geglu_rows": (cint, [P, P, P, i64, i64]),
+    "tlhip_embed_scaled": (cint, [P, i64, P, P, i64, i64, i64, i64, f32]),
+    "tlhip_ssm_state_bytes": (i64, [i64, i64, i64]),
+    "tlhip_ssm_conv_bytes": (i64, [i64, i64, i64, i64, i64]),
+    "tlhip_ssm_step": (cint, [P, P, P, i64, P]),
+    "tlhip_ssm_chunk": (cint, [P, i64, P, i64, P, i64, i64]),
+    "tlhip_latent_cache_bytes": (i64, [i64, i64, i64, i64, cint]),
+    "tlhip_latent_attn_run": (cint, [P, i64, P, i64, P, i64, P, i64, i64, P]),
     "tlhip_tune_gemv_q4": (cint, [cint, cint, cint, cint, cint]),
     "tlhip_tune_gemv_cols": (cint, [cint]),
     "tlhip_tune_attn_prefill": (cint, [cint]),
@@ -165,6 +178,19 @@ class LinearAttn(C.Structure):
 class PolyNorm(C.Structure):
     """tlhip_polynorm"""
     _fields_ = [(n, i64) for n in ("ff", "z_off", "y_off")] + [(n, f32) for n in ("c1", "c2", "c3", "c0", "eps")]
+
+
+class Ssm(C.Structure):
+    """tlhip_ssm"""
+    _fields_ = [(n, i64) for n in ("heads", "state", "groups", "vdim", "taps", "z_off", "x_off", "dt_off", "y_off")] + \
+               [(n, P) for n in ("conv_w", "conv_b", "dt_bias", "decay", "skip", "conv_state", "ssm_state")]
+
+
+class LatentAttn(C.Structure):
+    """tlhip_latent_attn"""
+    _fields_ = [(n, i64) for n in ("heads", "dim", "rot_dim", "vdim", "kv_rank", "kv_off", "gate_off", "y_off")] + \
+               [(n, P) for n in ("uk", "uv", "kv_norm", "angles", "keys", "values")] + \
+               [(n, i64) for n in ("capacity", "planes")] + [("scale", f32), ("eps", f32)]
 
 
 class TlHipError(RuntimeError):
@@ -598,6 +624,38 @@ class TlHip:
     def embed_sinusoid(self, table, tokens, out, T, width, ld, vocab, pos0, d_pos=None):
         self._chk(self.c.tlhip_embed_sinusoid(table.ptr, tokens.ptr, out.ptr, T, width, ld, vocab, pos0,
                                               d_pos.ptr if d_pos else None))
+
+    def gemv_bf16_row_postnorm(self, x, delta, bias, norm_w, n, parts, xout, W, y, N, K, eps):
+        opt = lambda b: b.ptr if b is not None else None
+        self._chk(self.c.tlhip_gemv_bf16_row_postnorm(opt(x), delta.ptr, opt(bias), norm_w.ptr, n, parts, opt(xout), W.ptr, y.ptr, N, K, eps))
+
+    def gemv_bf16_row_postnorm_geglu(self, x, delta, bias, norm_w, xout, W, gu_bias, act, N2, K, eps):
+        opt = lambda b: b.ptr if b is not None else None
+        self._chk(self.c.tlhip_gemv_bf16_row_postnorm_geglu(x.ptr, delta.ptr, opt(bias), norm_w.ptr, opt(xout), W.ptr, gu_bias.ptr, act.ptr,
+                                                            N2, K, eps))
+
+    def postnorm_res_parts(self, x, parts, S, bias, norm_w, xout, n, eps, rows, aimage=None):
+        opt = lambda b: b.ptr if b is not None else None
+        self._chk(self.c.tlhip_postnorm_res_parts(x.ptr, parts.ptr, S, opt(bias), norm_w.ptr, xout.ptr, n, eps, rows, opt(aimage)))
+
+    def rms_rows(self, x, ldx, w, out, ldo, n, n_out, parts, eps, rows):
+        self._chk(self.c.tlhip_rms_rows(x.ptr, ldx, w.ptr, out.ptr, ldo, n, n_out, parts, eps, rows))
+
+    def geglu_rows(self, gu, bias, out, ff, rows):
+        self._chk(self.c.tlhip_geglu_rows(gu.ptr, bias.ptr, out.ptr, ff, rows))
+
+    def embed_scaled(self, table, ldt, tokens, out, T, width, ld, vocab, scale):
+        self._chk(self.c.tlhip_embed_scaled(table.ptr, ldt, tokens.ptr, out.ptr, T, width, ld, vocab, scale))
+
+    def ssm_step(self, u, y, a, pos, d_pos=None):
+        self._chk(self.c.tlhip_ssm_step(u.ptr, y.ptr, C.byref(a), pos, d_pos.ptr if d_pos is not None else None))
+
+    def ssm_chunk(self, u, ldu, y, ldy, a, T, pos0):
+        self._chk(self.c.tlhip_ssm_chunk(u.ptr, ldu, y.ptr, ldy, C.byref(a), T, pos0))
+
+    def latent_attn(self, u, ldu, q, ldq, y, ldy, a, T, pos0, d_pos=None):
+        self._chk(self.c.tlhip_latent_attn_run(u.ptr, ldu, q.ptr, ldq, y.ptr, ldy, C.byref(a), T, pos0,
+                                               d_pos.ptr if d_pos is not None else None))
 
     def residual_sum(self, x, parts, S, add, vec, out, n, rows):
         opt = lambda b: b.ptr if b is not None else None

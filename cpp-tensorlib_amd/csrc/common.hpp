@@ -51,6 +51,9 @@ Context& ctx();
 int fail(int code, const char* fmt, ...);   // records the message, returns code
 int hip_fail(hipError_t e, const char* what);
 void* scratch(size_t bytes);                // nullptr on allocation failure
+// gemm_f16t.hip: the rows of tlhip_postnorm_res_parts with their activation image
+int postnorm_aimage(const float* x, const float* parts, int S, const float* bias, const float* w, float* xout, int n, float eps, int rows,
+                    void* aimage);
 int attn_static_setup(int device);          // attn.hip: address of the allocation-free entry point's array
 
 inline const char* at(const void* base, int64_t byte_off) {

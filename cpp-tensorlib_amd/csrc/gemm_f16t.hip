@@ -199,12 +199,14 @@ __global__ __launch_bounds__(256) void a_image_kernel(const float* __restrict__ 
 // and small-element mark for the row of hout, which is still in registers - in one launch and
 // without reading hout back. One block of 1024 threads per image row (rows past M are zero rows).
 // x and xout may be the same buffer (a thread writes only what it has read).
-template <int RV>
+// POST: the norm is of what is added instead, xout = x + ((parts + bias) / rms) w (the arithmetic of
+// postnorm_rows_kernel, seqops.hip), and the image is that of xout; hout is not written.
+template <int RV, bool POST = false>
 __global__ __launch_bounds__(1024) void rmsnorm_aimage_kernel(const float* x, const float* __restrict__ delta,
                                                               const float* __restrict__ w, float* xout,
                                                               float* __restrict__ hout, int n, float eps, int S,
                                                               size_t part_stride, int* __restrict__ ea,
-                                                              char* __restrict__ img, int M) {
+                                                              char* __restrict__ img, int M, const float* __restrict__ bias = nullptr) {
   __shared__ float red[16];
   __shared__ uint32_t part[16], cnt[16];
   const int gm = blockIdx.x, t = threadIdx.x, n4 = n >> 2, nslab = n / kBK;
@@ -218,7 +220,7 @@ __global__ __launch_bounds__(1024) void rmsnorm_aimage_kernel(const float* x, co
     const float4* x4 = reinterpret_cast<const float4*>(x + base);
     const float4* d4 = reinterpret_cast<const float4*>(delta + base);
     const float4* w4 = reinterpret_cast<const float4*>(w);
-    float4 v[RV], wv[RV];
+    float4 v[RV], wv[RV], xv[RV];
     float acc = 0.f;
 #pragma unroll
     for (int k = 0; k < RV; k++) {
@@ -231,26 +233,40 @@ __global__ __launch_bounds__(1024) void rmsnorm_aimage_kernel(const float* x, co
           const float4 e = d4[sidx * (part_stride >> 2) + i];
           d.x += e.x; d.y += e.y; d.z += e.z; d.w += e.w;
         }
-        v[k].x += d.x; v[k].y += d.y; v[k].z += d.z; v[k].w += d.w;
+        if constexpr (POST) {
+          if (bias) {
+            const float4 e = reinterpret_cast<const float4*>(bias)[i];
+            d.x += e.x; d.y += e.y; d.z += e.z; d.w += e.w;
+          }
+          xv[k] = v[k];
+          v[k] = d;
+        } else {
+          v[k].x += d.x; v[k].y += d.y; v[k].z += d.z; v[k].w += d.w;
+        }
       }
     }
 #pragma unroll
     for (int k = 0; k < RV; k++) {
       const int i = t + k * 1024;
       if (i < n4) {
-        reinterpret_cast<float4*>(xout + base)[i] = v[k];
+        if (!POST) reinterpret_cast<float4*>(xout + base)[i] = v[k];
         acc += (v[k].x * v[k].x + v[k].y * v[k].y) + (v[k].z * v[k].z + v[k].w * v[k].w);
       }
     }
     const float sum = block_sum<16>(acc, red);
-    const float inv = 1.0f / sqrtf(sum * (1.0f / (float)n) + eps);
+    const float inv = 1.0f / sqrtf((POST ? sum / (float)n : sum * (1.0f / (float)n)) + eps);
 #pragma unroll
     for (int k = 0; k < RV; k++) {
       const int i = t + k * 1024;
       if (i < n4) {
-        o[k].x = (v[k].x * inv) * wv[k].x; o[k].y = (v[k].y * inv) * wv[k].y;
-        o[k].z = (v[k].z * inv) * wv[k].z; o[k].w = (v[k].w * inv) * wv[k].w;
-        reinterpret_cast<float4*>(hout + base)[i] = o[k];
+        if constexpr (POST) {
+          o[k] = make_float4(fmaf(v[k].x * inv, wv[k].x, xv[k].x), fmaf(v[k].y * inv, wv[k].y, xv[k].y),
+                             fmaf(v[k].z * inv, wv[k].z, xv[k].z), fmaf(v[k].w * inv, wv[k].w, xv[k].w));
+        } else {
+          o[k].x = (v[k].x * inv) * wv[k].x; o[k].y = (v[k].y * inv) * wv[k].y;
+          o[k].z = (v[k].z * inv) * wv[k].z; o[k].w = (v[k].w * inv) * wv[k].w;
+        }
+        reinterpret_cast<float4*>((POST ? xout : hout) + base)[i] = o[k];
         mx = max(mx, __float_as_uint(o[k].x) & 0x7fffffffu);
         mx = max(mx, __float_as_uint(o[k].y) & 0x7fffffffu);
         mx = max(mx, __float_as_uint(o[k].z) & 0x7fffffffu);
@@ -897,3 +913,21 @@ int tlhip_gemm_f16w_nt_parts(const void* A, const void* image, const void* exps,
 }
 
 }  // extern "C"
+
+namespace tlhip {
+
+int postnorm_aimage(const float* x, const float* parts, int S, const float* bias, const float* w, float* xout, int n, float eps, int rows,
+                    void* aimage) {
+  if (n % f16t::kBK != 0 || n > 8192 || !aligned16(aimage))
+    return fail(TLHIP_EUNSUPPORTED, "tlhip_postnorm_res_parts: an activation image needs n %% 32 == 0 and n <= 8192");
+  const int64_t timg = cdiv64(rows, f16t::kTile);
+  if (timg * f16t::kTile > 0x7fffffff) return fail(TLHIP_EUNSUPPORTED, "tlhip_postnorm_res_parts: too many rows");
+  int* ea = static_cast<int*>(aimage);
+  char* img = static_cast<char*>(aimage) + (((size_t)rows * sizeof(int) + 1023) & ~(size_t)1023);
+  auto fn = n <= 4096 ? f16t::rmsnorm_aimage_kernel<1, true> : f16t::rmsnorm_aimage_kernel<2, true>;
+  hipLaunchKernelGGL(fn, dim3((unsigned)(timg * f16t::kTile)), dim3(1024), 0, ctx().stream, x, parts, w, xout, (float*)nullptr, n, eps, S,
+                     (size_t)rows * n, ea, img, rows, bias);
+  TLHIP_CHECK_LAUNCH(TLHIP_C_RMSNORM_RES);
+}
+
+}  // namespace tlhip

@@ -20,6 +20,8 @@
 #include "common.hpp"
 #include "gemv_shared.hpp"
 
+#include <algorithm>
+
 namespace tlhip {
 
 // ---------------------------------------------------------------------------
@@ -100,7 +102,11 @@ __global__ __launch_bounds__(R >= 8 ? 512 : 1024) void gemv_rows_kernel(
   const int groups = nw / KW;        // wavefront row groups per block tile
   const int rows_per_tile = groups * QN * R;
   const int wrow = (wn * QN + q) * R;  // this lane's first row inside a tile
-  constexpr bool kPair = EPI == kGateUp;
+  float* psum = fw;                                         // sums of squares, then 1 / rms (post-norm producer)
+  constexpr bool kPair = EPI != kStore;
+  const auto act = [&](float g, float u, int i) {
+    return EPI == kGeglu ? gelu_tanh(g + pro.gu_bias[i]) * (u + pro.gu_bias[N / 2 + i]) : gated(g, u);
+  };
   static_assert(!kPair || R >= 2, "a gate/up pair needs two rows per lane group");
   // first row of work item (tile tt): a row of W, or with kPair a row of each half
   const auto item_row = [&](int tt) { return kPair ? (tt * rows_per_tile + wrow) >> 1 : tt * rows_per_tile + wrow; };
@@ -114,8 +120,8 @@ __global__ __launch_bounds__(R >= 8 ? 512 : 1024) void gemv_rows_kernel(
   const float4* d4 = reinterpret_cast<const float4*>(pro.delta);
   // float4s a thread requests up front: all of x up to 20 floats per thread (K = 18944 on 1024
   // threads), 8 per thread in the norm form, whose vector is the hidden size (registers)
-  constexpr int PL = PRO == kRmsnorm ? 2 : 5;
-  float4 px[PL], pa[PL], pn[PL];
+  constexpr int PL = PRO == kRmsnorm || PRO == kPostnorm ? 2 : 5;
+  float4 px[PL], pa[PL], pn[PL], pb[PL];
   // attention-merge producer: this thread's first float4 of the first kPre splits' accumulators, and
   // the (head, split) pair whose maximum and sum it weighs
   constexpr int kPre = 8;
@@ -138,7 +144,8 @@ __global__ __launch_bounds__(R >= 8 ? 512 : 1024) void gemv_rows_kernel(
       const int i = min(tid + k * (int)blockDim.x, n4 - 1);
       if (PRO != kAttnMerge) px[k] = x4[i];
       if (PRO != kPlain && PRO != kAttnMerge) pa[k] = aux4[i];
-      if (PRO == kRmsnorm) pn[k] = reinterpret_cast<const float4*>(pro.norm_w)[i];
+      if (PRO == kRmsnorm || PRO == kPostnorm) pn[k] = reinterpret_cast<const float4*>(pro.norm_w)[i];
+      if (PRO == kPostnorm && pro.bias) pb[k] = reinterpret_cast<const float4*>(pro.bias)[i];
     }
   }
   asm volatile("" ::: "memory");
@@ -189,6 +196,31 @@ __global__ __launch_bounds__(R >= 8 ? 512 : 1024) void gemv_rows_kernel(
     __syncthreads();
   }
 
+  // Post-norm producer: 1 / rms of every run. A run is summed by `seg` wavefronts where there are fewer runs
+  // than wavefronts, in a fixed order.
+  if constexpr (PRO == kPostnorm) {
+    const int seg = pro.parts < nw ? nw / pro.parts : 1, sums = pro.parts * seg, len = pro.part_len;
+    for (int s = wave; s < sums; s += nw) {
+      const int p = s / seg, b = p * len;
+      float ss = 0.f;
+      for (int i = (s - p * seg) * 64 + lane; i < len; i += 64 * seg) {
+        const float v = pro.delta[b + i] + (pro.bias ? pro.bias[b + i] : 0.f);
+        ss = fmaf(v, v, ss);
+      }
+      ss = wave_sum(ss);
+      if (lane == 0) psum[s] = ss;
+    }
+    __syncthreads();
+    float* pinv = psum + sums;
+    for (int p = tid; p < pro.parts; p += blockDim.x) {
+      float t = psum[p * seg];
+      for (int k = 1; k < seg; k++) t += psum[p * seg + k];
+      pinv[p] = 1.0f / sqrtf(t / (float)len + pro.eps);
+    }
+    __syncthreads();
+    psum = pinv;
+  }
+
   {  // stage x (K = upr*E floats) into the interleaved layout, one pass:
      // thread i owns float4 i; the J threads of a unit are adjacent lanes, so the
      // unit's sum(x) is a J-lane shuffle reduction (J is 8 or 2, both divide 64).
@@ -213,15 +245,26 @@ __global__ __launch_bounds__(R >= 8 ? 512 : 1024) void gemv_rows_kernel(
         const float L = fL[h];
         return make_float4(v.x / L, v.y / L, v.z / L, v.w / L);
       }
-      float4 v, aux;
+      float4 v, aux, ab;
       bool have = false;
 #pragma unroll
       for (int kk = 0; kk < PL; kk++)
-        if (k == kk) { v = px[kk]; aux = pa[kk]; nv = pn[kk]; have = true; }
+        if (k == kk) { v = px[kk]; aux = pa[kk]; nv = pn[kk]; ab = pb[kk]; have = true; }
       if (!have) {
         v = x4[i];
         if (PRO == kSwiglu) aux = x4[n4 + i];
-        if (PRO == kRmsnorm) { nv = reinterpret_cast<const float4*>(pro.norm_w)[i]; if (d4) aux = d4[i]; }
+        if (PRO == kRmsnorm || PRO == kPostnorm) { nv = reinterpret_cast<const float4*>(pro.norm_w)[i]; if (d4) aux = d4[i]; }
+        if (PRO == kPostnorm && pro.bias) ab = reinterpret_cast<const float4*>(pro.bias)[i];
+      }
+      if constexpr (PRO == kPostnorm) {
+        if (pro.bias) { aux.x += ab.x; aux.y += ab.y; aux.z += ab.z; aux.w += ab.w; }
+        const int last = pro.parts - 1;
+        const auto inv_of = [&](int e) { return psum[last == 0 ? 0 : min(e / pro.part_len, last)]; };
+        const float i0 = inv_of(4 * i), i1 = inv_of(4 * i + 1), i2 = inv_of(4 * i + 2), i3 = inv_of(4 * i + 3);
+        if (!pro.add_x) v = make_float4(0.f, 0.f, 0.f, 0.f);
+        v.x = fmaf(aux.x * i0, nv.x, v.x); v.y = fmaf(aux.y * i1, nv.y, v.y);
+        v.z = fmaf(aux.z * i2, nv.z, v.z); v.w = fmaf(aux.w * i3, nv.w, v.w);
+        return v;
       }
       if (PRO == kRmsnorm && d4) { v.x += aux.x; v.y += aux.y; v.z += aux.z; v.w += aux.w; }
       if (PRO == kSwiglu) { v.x = gated(v.x, aux.x); v.y = gated(v.y, aux.y); v.z = gated(v.z, aux.z); v.w = gated(v.w, aux.w); }
@@ -253,6 +296,7 @@ __global__ __launch_bounds__(R >= 8 ? 512 : 1024) void gemv_rows_kernel(
           if (pro.xout && blockIdx.x == 0) reinterpret_cast<float4*>(pro.xout)[i] = v;
           v.x *= nv.x; v.y *= nv.y; v.z *= nv.z; v.w *= nv.w;
         }
+        if (PRO == kPostnorm && pro.xout && blockIdx.x == 0) reinterpret_cast<float4*>(pro.xout)[i] = v;
       }
       const int u = i / J, j = i - u * J;
       if (live) xs[((u / LPR) * J + j) * XS + (u & (LPR - 1))] = Fmt::stage(v);
@@ -328,7 +372,7 @@ __global__ __launch_bounds__(R >= 8 ? 512 : 1024) void gemv_rows_kernel(
         if constexpr (kPair) {
           // the up row's total sits half a wavefront (64-lane form) or R/2 lanes (16-lane form) away
           const float up = LPR == 64 ? swap32(v, v).second : __shfl_down(v, R / 2, kWave);   // .second: the upper half's value in the lower lanes
-          if (writer && r < R / 2 && row0 + r < N / 2) y[row0 + r] = gated(v, up);
+          if (writer && r < R / 2 && row0 + r < N / 2) y[row0 + r] = act(v, up, row0 + r);
         } else {
           if (writer && row0 + r < N) y[row0 + r] = v;
         }
@@ -341,7 +385,7 @@ __global__ __launch_bounds__(R >= 8 ? 512 : 1024) void gemv_rows_kernel(
           if (kw == 0 && li < R)
             for (int sidx = 0; sidx < KW; sidx++) sum += red[(wrow / R * KW + sidx) * R + li];
           const float up = __shfl_down(sum, R / 2, kWave);
-          if (kw == 0 && li < R / 2 && row0 + li < N / 2) y[row0 + li] = gated(sum, up);
+          if (kw == 0 && li < R / 2 && row0 + li < N / 2) y[row0 + li] = act(sum, up, row0 + li);
         } else if (kw == 0 && li < R && row0 + li < N) {
           float sum = 0.f;
           for (int sidx = 0; sidx < KW; sidx++) sum += red[(wrow / R * KW + sidx) * R + li];
@@ -618,7 +662,7 @@ static auto pick_rows_fn(int R) -> void (*)(const float*, const uint4*, const fl
                                             int, int, const Producer) {
   switch (R) {
     case 1:
-      if constexpr (EPI == kStore) return gemv_rows_kernel<Fmt, 1, PRO, LPR, EPI>;
+      if constexpr (EPI == kStore) return gemv_rows_kernel<Fmt, 1, PRO, LPR, EPI>;   // (a pair needs two rows)
       else return nullptr;
     case 2: return gemv_rows_kernel<Fmt, 2, PRO, LPR, EPI>;
     case 4: return gemv_rows_kernel<Fmt, 4, PRO, LPR, EPI>;
@@ -641,17 +685,18 @@ static int launch_rows(const float* x, const void* W, const float* scales, float
   if (max_rows >= (1 << 24)) max_rows = (1 << 24) - 1;
   max_rows &= ~(int64_t)255;
   if (max_rows <= 0) return fail(TLHIP_EUNSUPPORTED, "gemv: K too large");
-  if (EPI == kGateUp && N > max_rows) return fail(TLHIP_EUNSUPPORTED, "gemv: gate|up matrix too large for one launch");
+  if (EPI != kStore && N > max_rows) return fail(TLHIP_EUNSUPPORTED, "gemv: gate|up matrix too large for one launch");
   for (int64_t n0 = 0; n0 < N; n0 += max_rows) {
     const int64_t n = N - n0 < max_rows ? N - n0 : max_rows;
     RowCfg cfg = pick_rows_cfg(n, upr, Fmt::E, c.cus, c.lds_per_cu, tn);
-    if (EPI == kGateUp && cfg.R == 1) {   // a lane group needs a gate row and its up row
+    if (EPI != kStore && cfg.R == 1) {   // a lane group needs a gate row and its up row
       RowTune two = tn;
       two.R = 2;
       if (cfg.nw / cfg.KW >= 2 && cfg.nw > 4) two.nw = cfg.nw / 2;   // keeps the rows of a block tile
       cfg = pick_rows_cfg(n, upr, Fmt::E, c.cus, c.lds_per_cu, two);
     }
     if (PRO == kAttnMerge) cfg.lds += (size_t)pro.heads * (kMergeMax + 1) * sizeof(float);
+    if (PRO == kPostnorm) cfg.lds += (size_t)(std::max(pro.parts, cfg.nw) + pro.parts) * sizeof(float);
     if (cfg.lds > (size_t)c.lds_per_cu) return fail(TLHIP_EUNSUPPORTED, "gemv: K too large for the LDS-staged kernel");
     const int rows_per_tile = (cfg.nw / cfg.KW) * (64 / cfg.lpr) * cfg.R;
     const int ntiles = (int)((n + rows_per_tile - 1) / rows_per_tile);
@@ -914,6 +959,49 @@ int tlhip_gemv_bf16_row_rmsnorm(const void* x, const void* delta, const void* no
                      static_cast<float*>(xout), eps};
   return launch_rows<FmtBf16, kRmsnorm>(static_cast<const float*>(x), W, nullptr, static_cast<float*>(y),
                                         n, k, TLHIP_C_GEMV_BF16_ROW, RowTune{0, 0, 0, 0, 0}, pro);
+}
+
+static int check_postnorm(const void* x, const void* delta, const void* bias, const void* norm_w, const void* xout, int64_t n,
+                          int64_t parts, int64_t K, const char* who) {
+  if (!delta) return fail(TLHIP_EINVAL, "%s: null delta", who);
+  if (int rc = check_norm_args(x, delta, norm_w, xout, who)) return rc;
+  if (bias && !aligned16(bias)) return fail(TLHIP_EINVAL, "%s: vectors must be 16-byte aligned", who);
+  if (parts <= 0 || n <= 0 || n > K || n % parts || parts > 4096) return fail(TLHIP_EINVAL, "%s: bad norm size", who);
+  return 0;
+}
+
+int tlhip_gemv_bf16_row_postnorm(const void* x, const void* delta, const void* bias, const void* norm_w, int64_t n,
+                                 int64_t parts, void* xout, const void* W, void* y, int64_t N, int64_t K, float eps) {
+  TLHIP_REQUIRE_READY();
+  const char* who = "tlhip_gemv_bf16_row_postnorm";
+  if (int rc = check_gemv_args(x ? x : delta, W, y, N, K, who)) return rc;
+  if (int rc = check_fused_bf16(W, K, who)) return rc;
+  if (int rc = check_postnorm(x, delta, bias, norm_w, xout, n, parts, K, who)) return rc;
+  Producer pro{static_cast<const float*>(delta), static_cast<const float*>(norm_w), static_cast<float*>(xout), eps};
+  pro.bias = static_cast<const float*>(bias);
+  pro.parts = (int)parts;
+  pro.part_len = (int)(n / parts);
+  pro.add_x = x != nullptr;
+  return launch_rows<FmtBf16, kPostnorm>(static_cast<const float*>(x ? x : delta), W, nullptr, static_cast<float*>(y), N, K,
+                                         TLHIP_C_GEMV_BF16_ROW, RowTune{0, 0, 0, 0, 0}, pro);
+}
+
+int tlhip_gemv_bf16_row_postnorm_geglu(const void* x, const void* delta, const void* bias, const void* norm_w, void* xout,
+                                       const void* W, const void* gu_bias, void* act, int64_t N2, int64_t K, float eps) {
+  TLHIP_REQUIRE_READY();
+  const char* who = "tlhip_gemv_bf16_row_postnorm_geglu";
+  if (int rc = check_gemv_args(x, W, act, N2, K, who)) return rc;
+  if (N2 % 2 || !gu_bias) return fail(TLHIP_EINVAL, "%s: odd row count, or no bias", who);
+  if (int rc = check_fused_bf16(W, K, who)) return rc;
+  if (int rc = check_postnorm(x, delta, bias, norm_w, xout, K, 1, K, who)) return rc;
+  Producer pro{static_cast<const float*>(delta), static_cast<const float*>(norm_w), static_cast<float*>(xout), eps};
+  pro.bias = static_cast<const float*>(bias);
+  pro.parts = 1;
+  pro.part_len = (int)K;
+  pro.add_x = 1;
+  pro.gu_bias = static_cast<const float*>(gu_bias);
+  return launch_rows<FmtBf16, kPostnorm, kGeglu>(static_cast<const float*>(x), W, nullptr, static_cast<float*>(act), N2, K,
+                                                 TLHIP_C_GEMV_BF16_ROW, RowTune{0, 0, 0, 0, 0}, pro);
 }
 
 }  // extern "C"

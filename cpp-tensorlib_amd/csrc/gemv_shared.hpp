@@ -163,16 +163,24 @@ __device__ __forceinline__ float wave_sum_rows(float (&a)[R], int lane) {
 //             x[h*D + d] = sum_s e^(m_s - M) acc_s[d] / sum_s e^(m_s - M) l_s, at most 16 splits,
 //             in the summation order of the stand-alone merge kernel (same bits). The merge's
 //             launch goes; what it read (a few KB per head) every block now reads from L2.
+//   kPostnorm: x = in (when there is one) + (delta + bias) / rms * norm_w, the norm over `parts` runs of part_len
+//             entries, each by its own root mean square; block 0 writes x to xout. The factor is needed before
+//             anything can be staged, so the block meets a barrier for it; the weights are on their way meanwhile.
 // How a block leaves its results (EPI):
 //   kStore:  y[row] = dot.
 //   kGateUp: W is [gate rows | up rows] (N/2 each); a lane group owns R/2 gate rows and the
 //            matching up rows, and writes y[i] = (g*sigmoid(g))*u for i < N/2 - the gated
 //            activation in the GEMV that produces it, once per element, instead of in every
 //            block of the GEMV that consumes it.
-enum { kPlain = 0, kSwiglu = 1, kRmsnorm = 2, kAttnMerge = 3 };
+//   kGeglu:  as kGateUp with y[i] = gelu_tanh(g + gu_bias[i]) * (u + gu_bias[N/2 + i]).
+enum { kPlain = 0, kSwiglu = 1, kRmsnorm = 2, kAttnMerge = 3, kPostnorm = 4 };
 constexpr int kMergeMax = 16;  // splits the kAttnMerge producer takes (its lanes per head)
-enum { kStore = 0, kGateUp = 1 };
+enum { kStore = 0, kGateUp = 1, kGeglu = 2 };
 __device__ __forceinline__ float gated(float g, float u) { return (g * (1.0f / (1.0f + expf(-g)))) * u; }
+// z * Phi(z) in its tanh form: (1 + tanh(w)) / 2 = 1 / (1 + e^-2w)
+__device__ __forceinline__ float gelu_tanh(float z) {
+  return z / (1.0f + expf(-1.5957691216057308f * (z + 0.044715f * z * z * z)));
+}
 struct Producer {
   const float* delta;
   const float* norm_w;
@@ -180,6 +188,11 @@ struct Producer {
   float eps;
   // kAttnMerge: x points at the partials [heads*S] m | [heads*S] l | [heads*S][D] acc
   int S = 0, heads = 0, D = 0;
+  // kPostnorm
+  const float* bias = nullptr;
+  int parts = 0, part_len = 0, add_x = 0;
+  // kGeglu
+  const float* gu_bias = nullptr;
 };
 
 }  // namespace tlhip

@@ -199,6 +199,22 @@ struct api {
   int (*residual_sum)(const void*, const void*, int64_t, const void*, const void*, void*, int64_t,
                       int64_t) = nullptr;
   int (*gather_rows)(const void*, const void*, void*, int64_t, int64_t, int64_t) = nullptr;
+  int (*gemv_bf16_row_postnorm)(const void*, const void*, const void*, const void*, int64_t, int64_t, void*, const void*,
+                                void*, int64_t, int64_t, float) = nullptr;
+  int (*gemv_bf16_row_postnorm_geglu)(const void*, const void*, const void*, const void*, void*, const void*, const void*,
+                                      void*, int64_t, int64_t, float) = nullptr;
+  int (*postnorm_res_parts)(const void*, const void*, int64_t, const void*, const void*, void*, int64_t, float, int64_t,
+                            void*) = nullptr;
+  int (*rms_rows)(const void*, int64_t, const void*, void*, int64_t, int64_t, int64_t, int64_t, float, int64_t) = nullptr;
+  int (*geglu_rows)(const void*, const void*, void*, int64_t, int64_t) = nullptr;
+  int (*embed_scaled)(const void*, int64_t, const void*, void*, int64_t, int64_t, int64_t, int64_t, float) = nullptr;
+  int64_t (*ssm_state_bytes)(int64_t, int64_t, int64_t) = nullptr;
+  int64_t (*ssm_conv_bytes)(int64_t, int64_t, int64_t, int64_t, int64_t) = nullptr;
+  int (*ssm_step)(const void*, void*, const void*, int64_t, const void*) = nullptr;
+  int (*ssm_chunk)(const void*, int64_t, void*, int64_t, const void*, int64_t, int64_t) = nullptr;
+  int64_t (*latent_cache_bytes)(int64_t, int64_t, int64_t, int64_t, int) = nullptr;
+  int (*latent_attn_run)(const void*, int64_t, const void*, int64_t, void*, int64_t, const void*, int64_t, int64_t,
+                         const void*) = nullptr;
   int (*event_create)(void**) = nullptr;
   int (*event_record)(void*) = nullptr;
   int (*event_elapsed_ms)(void*, void*, float*) = nullptr;
@@ -400,7 +416,14 @@ struct context {
               bind(f.window_fill, "tlhip_window_fill") && bind(f.window_attn_chunk, "tlhip_window_attn_chunk") &&
               bind(f.linear_attn_chunk, "tlhip_linear_attn_chunk") && bind(f.polynorm_rows, "tlhip_polynorm_rows") &&
               bind(f.embed_sinusoid, "tlhip_embed_sinusoid") && bind(f.residual_sum, "tlhip_residual_sum") &&
-              bind(f.gather_rows, "tlhip_gather_rows");
+              bind(f.gather_rows, "tlhip_gather_rows") &&
+              bind(f.gemv_bf16_row_postnorm, "tlhip_gemv_bf16_row_postnorm") &&
+              bind(f.gemv_bf16_row_postnorm_geglu, "tlhip_gemv_bf16_row_postnorm_geglu") &&
+              bind(f.postnorm_res_parts, "tlhip_postnorm_res_parts") && bind(f.rms_rows, "tlhip_rms_rows") &&
+              bind(f.geglu_rows, "tlhip_geglu_rows") && bind(f.embed_scaled, "tlhip_embed_scaled") &&
+              bind(f.ssm_state_bytes, "tlhip_ssm_state_bytes") && bind(f.ssm_conv_bytes, "tlhip_ssm_conv_bytes") &&
+              bind(f.ssm_step, "tlhip_ssm_step") && bind(f.ssm_chunk, "tlhip_ssm_chunk") &&
+              bind(f.latent_cache_bytes, "tlhip_latent_cache_bytes") && bind(f.latent_attn_run, "tlhip_latent_attn_run");
     if (!ok) return;
     bind(f.warm_fork, "tlhip_warm_fork") && bind(f.warm_join, "tlhip_warm_join");   // optional
     why.clear();
@@ -1687,6 +1710,123 @@ inline bool gather_rows(void* src, void* idx, void* out, int64_t n, int64_t rows
   L.writes(out);
   return L.sent(L.lib.gather_rows(src, idx, out, n, rows, src_rows));
 }
+
+// ---- layers that norm what a sublayer writes (tensorlib_hip.h says what each field means) ---------
+struct ssm {
+  int64_t heads = 0, state = 0, groups = 0, vdim = 0, taps = 0;
+  int64_t z_off = 0, x_off = 0, dt_off = 0, y_off = 0;
+  void *conv_w = nullptr, *conv_b = nullptr, *dt_bias = nullptr, *decay = nullptr, *skip = nullptr;
+  void *conv_state = nullptr, *ssm_state = nullptr;
+};
+struct latent_attn {
+  int64_t heads = 0, dim = 0, rot_dim = 0, vdim = 0, kv_rank = 0;
+  int64_t kv_off = 0, gate_off = -1, y_off = 0;
+  void *uk = nullptr, *uv = nullptr, *kv_norm = nullptr, *angles = nullptr;
+  void *keys = nullptr, *values = nullptr;
+  int64_t capacity = 0, planes = 1;
+  float scale = 1, eps = 0;
+};
+// s = x (may be nullptr: 0) + rms(delta + bias) w over `parts` runs of the first n entries -> xout; y = W . s
+inline bool gemv_bf16_row_postnorm(void* x, void* delta, void* bias, void* norm_w, int64_t n, int64_t parts, void* xout,
+                                   void* W, void* y, int64_t N, int64_t K, float eps) {
+  launch L;
+  if (!L.ok || (K % 8) != 0) return false;
+  L.reads(delta, norm_w, W);
+  if (x) L.reads(x);
+  if (bias) L.reads(bias);
+  if (xout) L.writes(xout);
+  L.writes(y);
+  return L.sent(L.lib.gemv_bf16_row_postnorm(x, delta, bias, norm_w, n, parts, xout, W, y, N, K, eps));
+}
+// The same, W = [gate | up]: act = gelu_tanh(gate . s + b) (up . s + b)
+inline bool gemv_bf16_row_postnorm_geglu(void* x, void* delta, void* bias, void* norm_w, void* xout, void* W, void* gu_bias,
+                                         void* act, int64_t N2, int64_t K, float eps) {
+  launch L;
+  if (!L.ok || (K % 8) != 0) return false;
+  L.reads(x, delta, norm_w, W, gu_bias);
+  if (bias) L.reads(bias);
+  if (xout) L.writes(xout);
+  L.writes(act);
+  return L.sent(L.lib.gemv_bf16_row_postnorm_geglu(x, delta, bias, norm_w, xout, W, gu_bias, act, N2, K, eps));
+}
+// xout = x + rms(parts + bias) w; next_n as for rmsnorm_res_parts (the image is xout's)
+inline bool postnorm_res_parts(void* x, void* parts, int64_t n_parts, void* bias, void* w, void* xout, int64_t n, float eps,
+                               int64_t rows = 1, int64_t next_n = 0) {
+  launch L;
+  if (!L.ok || n <= 0 || rows <= 0 || n_parts <= 0) return false;
+  L.reads(x, parts, w);
+  if (bias) L.reads(bias);
+  L.writes(xout);
+  if (next_n > 0 && prompt_product_is_large(rows, next_n, n) && (n % 32) == 0 && n <= 8192)
+    if (void* room = L.act_room(xout, rows, n)) {
+      if (L.sent(L.lib.postnorm_res_parts(x, parts, n_parts, bias, w, xout, n, eps, rows, room))) {
+        L.act_made(xout);
+        return true;
+      }
+    }
+  return L.sent(L.lib.postnorm_res_parts(x, parts, n_parts, bias, w, xout, n, eps, rows, nullptr));
+}
+inline bool rms_rows(void* x, int64_t ldx, void* w, void* out, int64_t ldo, int64_t n, int64_t n_out, int64_t parts, float eps,
+                     int64_t rows) {
+  launch L;
+  if (!L.ok) return false;
+  L.reads(x, w);
+  L.writes(out);
+  return L.sent(L.lib.rms_rows(x, ldx, w, out, ldo, n, n_out, parts, eps, rows));
+}
+inline bool geglu_rows(void* gu, void* bias, void* out, int64_t ff, int64_t rows) {
+  launch L;
+  if (!L.ok) return false;
+  L.reads(gu, bias);
+  L.writes(out);
+  return L.sent(L.lib.geglu_rows(gu, bias, out, ff, rows));
+}
+inline bool embed_scaled(void* table, int64_t ldt, void* tokens, void* out, int64_t T, int64_t width, int64_t ld, int64_t vocab,
+                         float scale) {
+  launch L;
+  if (!L.ok) return false;
+  L.reads(table, tokens);
+  L.writes(out);
+  return L.sent(L.lib.embed_scaled(table, ldt, tokens, out, T, width, ld, vocab, scale));
+}
+inline int64_t ssm_state_bytes(const ssm& a) {
+  auto& c = context::get();
+  return c.ready ? c.f.ssm_state_bytes(a.heads, a.state, a.vdim) : 0;
+}
+inline int64_t ssm_conv_bytes(const ssm& a) {
+  auto& c = context::get();
+  return c.ready ? c.f.ssm_conv_bytes(a.heads, a.state, a.groups, a.vdim, a.taps) : 0;
+}
+inline bool ssm_step(void* u, void* y, const ssm& a, int64_t pos, void* d_pos) {
+  launch L;
+  if (!L.ok || !u || !y) return false;
+  L.reads(u, a.conv_w, a.conv_b, a.dt_bias, a.decay, a.skip);
+  if (d_pos) L.reads(d_pos);
+  L.writes(y, a.conv_state, a.ssm_state);
+  return L.sent(L.lib.ssm_step(u, y, &a, pos, d_pos));
+}
+inline bool ssm_chunk(void* u, int64_t ldu, void* y, int64_t ldy, const ssm& a, int64_t T, int64_t pos0) {
+  launch L;
+  if (!L.ok || !u || !y) return false;
+  L.reads(u, a.conv_w, a.conv_b, a.dt_bias, a.decay, a.skip);
+  L.writes(y, a.conv_state, a.ssm_state);
+  return L.sent(L.lib.ssm_chunk(u, ldu, y, ldy, &a, T, pos0));
+}
+inline int64_t latent_cache_bytes(const latent_attn& a, bool values) {
+  auto& c = context::get();
+  return c.ready ? c.f.latent_cache_bytes(a.capacity, a.kv_rank, a.rot_dim, a.planes, values ? 1 : 0) : 0;
+}
+// T tokens at pos0 (d_pos: one, position on the device): new rows cached, u and q -> y
+inline bool latent_attn_run(void* u, int64_t ldu, void* q, int64_t ldq, void* y, int64_t ldy, const latent_attn& a, int64_t T,
+                            int64_t pos0, void* d_pos = nullptr) {
+  launch L;
+  if (!L.ok || !u || !q || !y) return false;
+  L.reads(u, q, a.uk, a.uv, a.kv_norm, a.angles);
+  if (d_pos) L.reads(d_pos);
+  L.writes(y, a.keys, a.values);
+  return L.sent(L.lib.latent_attn_run(u, ldu, q, ldq, y, ldy, &a, T, pos0, d_pos));
+}
+
 // A device-only buffer of zeros (bytes a multiple of 4).
 inline void* alloc_zeros(int64_t bytes) {
   void* p = alloc_device(bytes);

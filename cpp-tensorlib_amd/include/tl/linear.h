@@ -89,6 +89,18 @@ inline bool gemv_rmsnorm_gateup(const linear& L, void* x, void* delta, void* nor
   return hip::gemv_bf16_row_rmsnorm_gateup(x, delta, norm_w, xout, L.w, act, L.N, L.K, eps);
 }
 
+// s = x (nullptr: 0) + rms(delta + bias) norm_w over `parts` runs of n -> xout ; y = W . s (bf16 rows)
+inline bool gemv_postnorm(const linear& L, void* x, void* delta, void* bias, void* norm_w, int64_t n, int64_t parts, void* xout,
+                          void* y, float eps) {
+  return L.fmt == wfmt::bf16_row && hip::gemv_bf16_row_postnorm(x, delta, bias, norm_w, n, parts, xout, L.w, y, L.N, L.K, eps);
+}
+// L = [gate rows | up rows] with biases: act = gelu_tanh(gate . s + b) (up . s + b)
+inline bool gemv_postnorm_geglu(const linear& L, void* x, void* delta, void* bias, void* norm_w, void* xout, void* gu_bias,
+                                void* act, float eps) {
+  return L.fmt == wfmt::bf16_row &&
+         hip::gemv_bf16_row_postnorm_geglu(x, delta, bias, norm_w, xout, L.w, gu_bias, act, L.N, L.K, eps);
+}
+
 namespace detail {
 
 inline void* dev_from_host(const void* src, int64_t bytes) {

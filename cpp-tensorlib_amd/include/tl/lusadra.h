@@ -32,7 +32,7 @@
 #include "hip.h"
 #include "json.h"
 #include "linear.h"
-#include "safetensors.h"
+#include "model_source.h"
 
 namespace tl {
 namespace lusadra {
@@ -181,82 +181,10 @@ struct model {
   }
 };
 
-namespace detail {
-
-inline int64_t up(int64_t n, int64_t to) { return (n + to - 1) / to * to; }
-
-// Where tensors come from: a file, or a generator for throughput runs. Values are bf16 bits.
-struct source {
-  virtual ~source() = default;
-  // rows x cols of `name` (checked against the shape; cols 0: a vector, rows 0: one number)
-  virtual void read(const std::string& name, int64_t rows, int64_t cols, uint16_t* dst, int64_t ld) = 0;
-  virtual int64_t rows_of(const std::string& name) = 0;
-};
-
-struct file_source : source {
-  const safetensors::file& f;
-  explicit file_source(const safetensors::file& file) : f(file) {}
-  const safetensors::tensor& get(const std::string& name) const {
-    const safetensors::tensor* t = f.find(name);
-    if (!t) throw std::runtime_error("missing tensor " + name);
-    if (t->dtype != "BF16") throw std::runtime_error(name + ": bf16 expected");
-    return *t;
-  }
-  void read(const std::string& name, int64_t rows, int64_t cols, uint16_t* dst, int64_t ld) override {
-    const safetensors::tensor& t = get(name);
-    std::vector<int64_t> want;
-    if (rows) want.push_back(rows);
-    if (cols) want.push_back(cols);
-    // a single number may be stored with or without a dimension of 1
-    const bool one = !rows && !cols && t.elements() == 1;
-    if (!one && t.shape != want) throw std::runtime_error(name + ": shape does not match the configuration");
-    const int64_t r = rows ? rows : 1, n = cols ? cols : 1;
-    const char* p = static_cast<const char*>(t.data);
-    if (!cols) {                       // a vector: contiguous
-      std::memcpy(dst, p, (size_t)r * 2);
-      return;
-    }
-    for (int64_t i = 0; i < r; i++) std::memcpy(dst + i * ld, p + i * n * 2, (size_t)n * 2);
-  }
-  int64_t rows_of(const std::string& name) override {
-    const safetensors::tensor& t = get(name);
-    if (t.shape.empty()) throw std::runtime_error(name + ": a matrix expected");
-    return t.shape[0];
-  }
-};
-
-// Seeded values of a size that keeps activations finite; for throughput runs.
-struct random_source : source {
-  int64_t rank;
-  std::vector<float> block;            // uniform in [-1, 1), drawn once and walked through again and again
-  size_t at = 0;
-  random_source(uint32_t seed, int64_t low_rank) : rank(low_rank), block((size_t)(1 << 20) + 7) {
-    uint32_t s = seed * 2654435761u + 1u;
-    for (auto& v : block) {
-      s ^= s << 13; s ^= s >> 17; s ^= s << 5;
-      v = (float)(int32_t)s * (1.0f / 2147483648.0f);
-    }
-  }
-  void read(const std::string&, int64_t rows, int64_t cols, uint16_t* dst, int64_t ld) override {
-    const int64_t r = rows ? rows : 1, n = cols ? cols : 1;
-    const float amp = cols ? std::sqrt(3.0f / (float)n) : 1.0f;
-    for (int64_t i = 0; i < r; i++)
-      for (int64_t k = 0; k < n; k++) {
-        dst[i * (cols ? ld : 1) + k] = f32_to_bf16(amp * block[at]);
-        if (++at == block.size()) at = 0;
-      }
-  }
-  int64_t rows_of(const std::string&) override { return rank; }
-};
-
-struct part { std::string name; int64_t rows, at; };   // rows of a stacked matrix
-
-}  // namespace detail
-
 // Allocates everything and fills the weights from `src`. max_ctx: the longest sequence; chunk: the
 // longest prompt chunk (the key rings hold a window and a chunk).
-inline void build(model& M, const config& cfg, detail::source& src, int64_t max_ctx, int64_t chunk = 512) {
-  using detail::up;
+inline void build(model& M, const config& cfg, source::reader& src, int64_t max_ctx, int64_t chunk = 512) {
+  using source::up;
   if (!hip::available()) throw std::runtime_error(std::string("GPU backend unavailable: ") + hip::unavailable_reason());
   if (max_ctx <= 0 || chunk <= 0 || chunk > 65535) throw std::runtime_error("bad context or chunk length");
   M.c = cfg;
@@ -286,13 +214,13 @@ inline void build(model& M, const config& cfg, detail::source& src, int64_t max_
     return upload(v.data(), WP * 4);
   };
   // projections stacked by rows
-  const auto stack = [&](const std::vector<detail::part>& parts, int64_t N) {
+  const auto stack = [&](const std::vector<source::part>& parts, int64_t N) {
     host.assign((size_t)(N * WP), 0);
     for (const auto& p : parts) src.read(p.name, p.rows, E, host.data() + p.at * WP, WP);
     return linear{upload(host.data(), N * WP * 2), N, WP, wfmt::bf16_row};
   };
   // output projections side by side: part.rows = its columns, part.at = its first column
-  const auto beside = [&](const std::vector<detail::part>& parts, int64_t K) {
+  const auto beside = [&](const std::vector<source::part>& parts, int64_t K) {
     host.assign((size_t)(WP * K), 0);
     for (const auto& p : parts) src.read(p.name, E, p.rows, host.data() + p.at, K);
     return linear{upload(host.data(), WP * K * 2), WP, K, wfmt::bf16_row};
@@ -305,9 +233,9 @@ inline void build(model& M, const config& cfg, detail::source& src, int64_t max_
     const layer_config& lc = cfg.layers[i];
     layer& L = M.layers[i];
     const std::string p = "l" + std::to_string(i) + ".", pl = p + "mix.left.", pr = p + "mix.right.";
-    std::vector<detail::part> in, out;
+    std::vector<source::part> in, out;
     int64_t nu = 0, ny = 0;
-    const auto seg = [&](std::vector<detail::part>& list, int64_t& end, const std::string& name, int64_t n) {
+    const auto seg = [&](std::vector<source::part>& list, int64_t& end, const std::string& name, int64_t n) {
       const int64_t at = end;
       list.push_back({name, n, at});
       end = up(at + n, 8);
@@ -416,11 +344,11 @@ inline void build(model& M, const config& cfg, detail::source& src, int64_t max_
 // A folder with config.json and model.safetensors.
 inline void load(model& M, const json::value& cfg, const std::string& dir, int64_t max_ctx, int64_t chunk = 512) {
   const safetensors::file f(dir + "/model.safetensors");
-  detail::file_source src(f);
+  source::file src(f);
   build(M, parse_config(cfg), src, max_ctx, chunk);
 }
 inline void load_random(model& M, const json::value& cfg, uint32_t seed, int64_t rank, int64_t max_ctx, int64_t chunk = 512) {
-  detail::random_source src(seed, rank);
+  source::random src(seed, rank);
   build(M, parse_config(cfg), src, max_ctx, chunk);
 }
 
@@ -551,6 +479,7 @@ inline const float* logits_host(const model& M) { return M.s.logits_host; }
 inline const linear& head(const model& M) { return M.lm_head; }
 inline void* chunk_rows(model& M) { return M.ps.h; }
 inline int64_t chunk_row_width(const model& M) { return M.wp; }
+inline int64_t layer_runs(const model& M) { return (int64_t)M.runs.size(); }
 inline bool stage_embed(model& M, int64_t token) {
   if (token < 0 || token >= M.c.vocab) return false;
   hip::upload_u32(M.s.tok, (unsigned)token);

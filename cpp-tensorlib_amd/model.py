@@ -20,7 +20,7 @@ def _load():
         sig = {
             "tlm_error": (C.c_char_p, []),
             "tlm_open": (P, [C.c_char_p, i64, i64, cint, cint]),
-            "tlm_random_lusadra": (P, [C.c_char_p, u32, i64, i64, i64, cint]),
+            "tlm_random": (P, [C.c_char_p, u32, i64, i64, i64, cint]),
             "tlm_close": (None, [P]),
             "tlm_architecture": (C.c_char_p, [P]),
             "tlm_vocab": (i64, [P]),
@@ -66,10 +66,11 @@ class Model:
         return cls(L, L.tlm_open(os.fsencode(path), max_ctx, chunk, int(exact), int(q4)))
 
     @classmethod
-    def random_lusadra(cls, config, seed=1, rank=16, max_ctx=4096, chunk=512, exact=False):
-        """A Lusadra of the given configuration (a dict) with seeded weights; rank: of its decay inputs."""
+    def random(cls, config, seed=1, rank=16, max_ctx=4096, chunk=512, exact=False):
+        """A model of the given configuration (a dict with its "architecture") with seeded weights; rank: of
+        Lusadra's decay inputs."""
         L = _load()
-        return cls(L, L.tlm_random_lusadra(json.dumps(config).encode(), seed, rank, max_ctx, chunk, int(exact)))
+        return cls(L, L.tlm_random(json.dumps(config).encode(), seed, rank, max_ctx, chunk, int(exact)))
 
     @property
     def architecture(self):
@@ -100,7 +101,7 @@ class Model:
             raise RuntimeError("generate: %d of %d tokens (context full, or the loop could not be recorded)" % (done + 1, n))
         return ([first] + [int(v) for v in out[:done]])[:n]
 
-    # ---- Lusadra: launch forms, diagnostics, throughput ------------------------------------------
+    # ---- launch forms, diagnostics, throughput (designs read from folders) -----------------------
     def set_fused(self, on):
         if self.L.tlm_set_fused(self.h, int(on)) != 0:
             raise RuntimeError("set_fused: not offered by this model")

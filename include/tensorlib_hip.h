@@ -99,7 +99,7 @@ typedef enum {
   TLHIP_C_ARGMAX, TLHIP_C_KV_APPEND, TLHIP_C_KV_FILL, TLHIP_C_SPLIT_HEADS,
   TLHIP_C_MERGE_HEADS, TLHIP_C_GEMM_BF16_NT, TLHIP_C_ATTN_PREFILL, TLHIP_C_CONVERT,
   TLHIP_C_QUANTIZE_Q4, TLHIP_C_MIX_STEP, TLHIP_C_WINDOW_ATTN, TLHIP_C_LINEAR_ATTN, TLHIP_C_POLYNORM,
-  TLHIP_C_EMBED, TLHIP_C_RESIDUAL, TLHIP_C_COUNT
+  TLHIP_C_EMBED, TLHIP_C_RESIDUAL, TLHIP_C_SSM, TLHIP_C_LATENT_ATTN, TLHIP_C_ACT, TLHIP_C_COUNT
 } tlhip_census_id;
 int tlhip_census(uint64_t* counts, int n);  /* copies min(n, TLHIP_C_COUNT) counters */
 int tlhip_census_reset(void);
@@ -538,6 +538,72 @@ int tlhip_residual_sum(const void* x, const void* parts, int64_t S, const void* 
                        void* out, int64_t n, int64_t rows);
 /* out[i] = src[idx[i]], rows of n f32; idx: device int32, clamped to [0, src_rows). */
 int tlhip_gather_rows(const void* src, const void* idx, void* out, int64_t n, int64_t rows, int64_t src_rows);
+
+/* ---- layers that norm what a sublayer writes (no reference counterpart) ----------------------------
+ * A sublayer reads the residual itself; its output, plus a bias, is RMS-normed and then added:
+ *   xout = x + rms(delta + bias) * norm_w.
+ * norm_w is applied as given, so a residual factor is folded into it. */
+
+/* s = x (NULL: 0) + delta', delta' = (delta + bias) / its root mean square * norm_w, over `parts` equal runs of the
+ * first n entries, each by its own root mean square (norm_w and the weight's columns past n: zero);
+ * xout (when non-NULL) receives s; y = W . s. bias may be NULL; xout must not alias x or delta. */
+int tlhip_gemv_bf16_row_postnorm(const void* x, const void* delta, const void* bias, const void* norm_w, int64_t n,
+                                 int64_t parts, void* xout, const void* W, void* y, int64_t N, int64_t K, float eps);
+/* The same with parts = 1, n = K and the gated activation as the GEMV's epilogue: W = [gate rows | up rows], N2 / 2
+ * each, gu_bias f32 [N2]: act[i] = gelu_tanh(gate_i + bias) (up_i + bias). */
+int tlhip_gemv_bf16_row_postnorm_geglu(const void* x, const void* delta, const void* bias, const void* norm_w, void* xout,
+                                       const void* W, const void* gu_bias, void* act, int64_t N2, int64_t K, float eps);
+/* Rows of a chunk: xout = x + rms(parts[0] + ... + parts[S-1] + bias) * norm_w, rows of n (n % 4 == 0). xout may
+ * alias x. aimage (may be NULL): also xout's activation image (gemm_f16w_aimage_bytes(rows, n) bytes). */
+int tlhip_postnorm_res_parts(const void* x, const void* parts, int64_t S, const void* bias, const void* norm_w, void* xout,
+                             int64_t n, float eps, int64_t rows, void* aimage);
+/* out[t][i] = rms over `parts` equal runs of the n columns of x[t] times w[i]; out's columns n .. n_out - 1 are zeroed. Rows ldx and
+ * ldo apart; out may be x. */
+int tlhip_rms_rows(const void* x, int64_t ldx, const void* w, void* out, int64_t ldo, int64_t n, int64_t n_out, int64_t parts,
+                   float eps, int64_t rows);
+/* out[t][i] = gelu_tanh(gu[t][i] + bias[i]) (gu[t][ff + i] + bias[ff + i]), i < ff; rows of 2 ff and ff. */
+int tlhip_geglu_rows(const void* gu, const void* bias, void* out, int64_t ff, int64_t rows);
+/* out[t][ld] f32 = scale x the widened bf16 row tokens[t] of a [vocab, width] table with rows ldt apart; zeros from
+ * width on. tokens: device int32, clamped to the table. */
+int tlhip_embed_scaled(const void* table, int64_t ldt, const void* tokens, void* out, int64_t T, int64_t width, int64_t ld,
+                       int64_t vocab, float scale);
+
+/* State-space layer with one decay per head and step (Mamba-2). u holds z [heads x vdim] at z_off, the convolution's
+ * channels x [heads x vdim] | B [groups x state] | C [groups x state] at x_off, dt [heads] at dt_off; y gets
+ * heads x vdim at y_off, gated by silu(z), not normed. conv_w f32 [taps][channels] (the last row meets the current
+ * token), conv_b [channels]; dt_bias, decay (base-2 log of the decay per unit of dt), skip: f32 [heads].
+ * conv_state: taps rows of the channels; ssm_state: two slots of heads x state rows of vdim (tlhip_ssm_*_bytes).
+ * Position 0 starts from zeros whatever they hold; a step can be repeated at its position. */
+typedef struct {
+  int64_t heads, state, groups, vdim, taps;
+  int64_t z_off, x_off, dt_off, y_off;
+  const void *conv_w, *conv_b, *dt_bias, *decay, *skip;
+  void *conv_state, *ssm_state;
+} tlhip_ssm;
+int64_t tlhip_ssm_state_bytes(int64_t heads, int64_t state, int64_t vdim);
+int64_t tlhip_ssm_conv_bytes(int64_t heads, int64_t state, int64_t groups, int64_t vdim, int64_t taps);
+int tlhip_ssm_step(const void* u, void* y, const tlhip_ssm* a, int64_t pos, const void* d_pos);
+int tlhip_ssm_chunk(const void* u, int64_t ldu, void* y, int64_t ldy, const tlhip_ssm* a, int64_t T, int64_t pos0);
+
+/* Latent attention: per position one latent of kv_rank numbers (RMS-normed with kv_norm) and rot_dim rotated key
+ * dims that all heads share are cached; per head the key is [uk c | rotated], the value uv c. u holds the raw
+ * latent and the raw key part behind it at kv_off, and (gate_off >= 0) the output gate [heads x vdim] whose
+ * sigmoid multiplies the result; q rows are head by head [dim | rot_dim], not rotated. y gets heads x vdim at y_off.
+ * uk bf16 [heads x dim] rows of kv_rank rounded up to 8 (zeros), uv bf16 [heads x vdim] likewise; angles: (cos, sin)
+ * f32 pairs [capacity][rot_dim / 2], pair i turning dims i and i + rot_dim / 2. keys, values: the cache in matrix
+ * operand form (tlhip_latent_cache_bytes), as one bf16 (planes 1) or as three that add up to the f32 (planes 3).
+ * T tokens at pos0 (d_pos: one token, position on the device), the new rows cached on the way. */
+typedef struct {
+  int64_t heads, dim, rot_dim, vdim, kv_rank;
+  int64_t kv_off, gate_off, y_off;
+  const void *uk, *uv, *kv_norm, *angles;
+  void *keys, *values;
+  int64_t capacity, planes;
+  float scale, eps;
+} tlhip_latent_attn;
+int64_t tlhip_latent_cache_bytes(int64_t capacity, int64_t kv_rank, int64_t rot_dim, int64_t planes, int values);
+int tlhip_latent_attn_run(const void* u, int64_t ldu, const void* q, int64_t ldq, void* y, int64_t ldy,
+                          const tlhip_latent_attn* a, int64_t T, int64_t pos0, const void* d_pos);
 
 /* Upper bound on the K splits of the [K,N] GEMVs (tlhip_gemv_f32 / tlhip_gemv_bf16); 1 = no
  * split, 0 = the built-in choice. The reference's diagnostic knob set_no_splitk (cuda.h:193-197,

@@ -72,7 +72,7 @@ def test_large_products_in_both_forms(Model):
     want = [0, 1, 100, 159, 160, 161, 511, 512, 513, 699]
     lg = {}
     for exact in (True, False):
-        m = Model.random_lusadra(cfg, seed=3, rank=10, max_ctx=800, exact=exact)
+        m = Model.random(cfg, seed=3, rank=10, max_ctx=800, exact=exact)
         lg[exact] = m.feed(t, want)
         if exact:
             m.reset()

@@ -61,19 +61,23 @@ def state_space(x, B, C, dt, A_log, D, heads, groups, N, vdim, S=None):
     return y, S
 
 
-def mamba2(h, W, p, c, eps, st):
-    """st: {"tail": inputs of the convolution, "S": state} of one sequence, updated."""
+def mamba2_core(u, w, b, dt_bias, A_log, D, c, st):
+    """Rows u = [z | x | B | C | dt] to the gated output ahead of its norm. st: {"tail": inputs of the
+    convolution, "S": state} of one sequence, updated."""
     H, N, G, V = c["heads"], c["state"], c["groups"], c["vdim"]
     inner, ch = H * V, H * V + 2 * G * N
-    u = h @ W[p + "in"].T
-    z, xbc, dt = u[:, :inner], u[:, inner:inner + ch], u[:, inner + ch:]
+    z, xbc, dt = u[:, :inner], u[:, inner:inner + ch], u[:, inner + ch:inner + ch + H]
     tail = st.get("tail", np.zeros((c["conv"] - 1, ch), F))
-    xbc, st["tail"] = causal_conv(xbc, W[p + "conv"], W[p + "conv.b"], tail)
+    xbc, st["tail"] = causal_conv(xbc, w, b, tail)
     xbc = silu(xbc)
     x, B, C = xbc[:, :inner], xbc[:, inner:inner + G * N], xbc[:, inner + G * N:]
-    y, st["S"] = state_space(x, B, C, softplus(dt + W[p + "dt_bias"]), W[p + "A_log"], W[p + "D"], H, G, N, V, st.get("S"))
-    y = grouped_rms_norm(y * silu(z), W[p + "norm"], c["norm_groups"], eps)
-    return y @ W[p + "o"].T
+    y, st["S"] = state_space(x, B, C, softplus(dt + dt_bias), A_log, D, H, G, N, V, st.get("S"))
+    return y * silu(z)
+
+
+def mamba2(h, W, p, c, eps, st):
+    y = mamba2_core(h @ W[p + "in"].T, W[p + "conv"], W[p + "conv.b"], W[p + "dt_bias"], W[p + "A_log"], W[p + "D"], c, st)
+    return grouped_rms_norm(y, W[p + "norm"], c["norm_groups"], eps) @ W[p + "o"].T
 
 
 def rotate_half(x, p, base):
@@ -90,28 +94,33 @@ def attend(q, keys, values, scale):
     return (w / w.sum()) @ values
 
 
-def latent_attention(h, W, p, c, eps, pos0, st):
-    """Keys and values are formed from the latents head by head. st: {"c": latents, "r": rotated key
-    parts} of the positions so far, updated."""
-    H, D, R, V = c["heads"], c["dim"], c["rot_dim"], c["vdim"]
-    T, base = len(h), c["rot"]["base"]
-    cq = rms_norm(h @ W[p + "dq"].T, W[p + "dq.norm"], eps)
-    q = (cq @ W[p + "uq"].T).reshape(T, H, D + R)
-    kv = h @ W[p + "dkv"].T
-    L = c["kv_rank"]
-    lat = rms_norm(kv[:, :L], W[p + "dkv.norm"], eps)
-    rot = np.stack([rotate_half(kv[t, L:], pos0 + t, base) for t in range(T)])
+def latent_core(q, kv, kv_norm, uk, uv, c, base, eps, pos0, st):
+    """Rows q (heads side by side, [dim | rot_dim], not rotated) and kv = [latent | key part], both raw, to
+    the heads' outputs. Keys and values are formed from the latents head by head. st: {"c": latents, "r":
+    rotated key parts} of the positions so far, updated."""
+    H, D, R, V, L = c["heads"], c["dim"], c["rot_dim"], c["vdim"], c["kv_rank"]
+    T = len(q)
+    q = q.reshape(T, H, D + R)
+    lat = rms_norm(kv[:, :L], kv_norm, eps)
+    rot = np.stack([rotate_half(kv[t, L:L + R], pos0 + t, base) for t in range(T)])
     st["c"] = np.concatenate([st["c"], lat]) if "c" in st else lat
     st["r"] = np.concatenate([st["r"], rot]) if "r" in st else rot
     n = len(st["c"])
-    k = (st["c"] @ W[p + "uk"].T).reshape(n, H, D)
-    v = (st["c"] @ W[p + "uv"].T).reshape(n, H, V)
+    k = (st["c"] @ uk.T).reshape(n, H, D)
+    v = (st["c"] @ uv.T).reshape(n, H, V)
     out = np.zeros((T, H * V), F)
     for t in range(T):
         m = pos0 + t + 1
         for e in range(H):
             qe = np.concatenate([q[t, e, :D], rotate_half(q[t, e, D:], pos0 + t, base)])
             out[t, e * V:(e + 1) * V] = attend(qe, np.concatenate([k[:m, e], st["r"][:m]], axis=1), v[:m, e], c["scale"])
+    return out
+
+
+def latent_attention(h, W, p, c, eps, pos0, st):
+    cq = rms_norm(h @ W[p + "dq"].T, W[p + "dq.norm"], eps)
+    out = latent_core(cq @ W[p + "uq"].T, h @ W[p + "dkv"].T, W[p + "dkv.norm"], W[p + "uk"], W[p + "uv"], c,
+                      c["rot"]["base"], eps, pos0, st)
     return (out * sigmoid(h @ W[p + "g"].T)) @ W[p + "o"].T
 
 

@@ -1,6 +1,6 @@
 """CPU: model folders (config.json + model.safetensors) are read strictly - what is missing, misshapen
-or unknown is named before anything touches the GPU -, and the plain Lusadra implementation the GPU tests
-compare with agrees with itself however its input is cut."""
+or unknown is named before anything touches the GPU -, and the plain implementations the GPU tests
+compare with agree with themselves however their input is cut."""
 import copy
 import importlib
 import json
@@ -10,6 +10,8 @@ import struct
 import numpy as np
 import pytest
 
+import girirax_models as GM
+import girirax_oracle as GO
 import lusadra_models as LM
 import lusadra_oracle as O
 
@@ -25,11 +27,12 @@ def refused(Model, folder):
     return str(e.value)
 
 
-def test_good_folder_reaches_the_backend(tmp_path, Model):
+@pytest.mark.parametrize("models,name", [(LM, "loop_of_unlike_layers"), (GM, "state_first")])
+def test_good_folder_reaches_the_backend(tmp_path, Model, models, name):
     if os.path.exists("/dev/kfd"):
         pytest.skip("a GPU is present")
-    cfg = LM.SMALL["loop_of_unlike_layers"]
-    assert "backend unavailable" in refused(Model, LM.write(tmp_path / "m", cfg, LM.weights(cfg)))
+    cfg = models.SMALL[name]
+    assert "backend unavailable" in refused(Model, LM.write(tmp_path / "m", cfg, models.weights(cfg)))
 
 
 @pytest.mark.parametrize("edit,words", [
@@ -49,6 +52,26 @@ def test_good_folder_reaches_the_backend(tmp_path, Model):
 def test_configurations_that_are_refused(tmp_path, Model, edit, words):
     cfg = copy.deepcopy(LM.SMALL["loop_of_unlike_layers"])
     W = LM.weights(cfg)
+    edit(cfg)
+    assert words in refused(Model, LM.write(tmp_path / "m", cfg, W))
+
+
+@pytest.mark.parametrize("edit,words", [
+    (lambda c: c.pop("residual_mult"), "residual_mult"),
+    (lambda c: c.pop("embedding"), "embedding"),
+    (lambda c: c["layers"][0].update(type="mamba"), "unknown mixer"),
+    (lambda c: c["layers"][0]["mixer"].update(groups=4), "layer 0"),
+    (lambda c: c["layers"][0]["mixer"].update(norm_groups=5), "layer 0"),
+    (lambda c: c["layers"][2]["mixer"].update(conv=0), "layer 2"),
+    (lambda c: c["layers"][1]["mixer"].update(rot_dim=7), "layer 1"),
+    (lambda c: c["layers"][1]["mixer"]["rot"].update(dims=4), "rot.dims"),
+    (lambda c: c["layers"][3]["mixer"].pop("q_rank"), "q_rank"),
+    (lambda c: c["layers"][3]["mlp"].update(kind="experts"), "unknown feed-forward"),
+    (lambda c: c.update(layers=[]), "no layers"),
+])
+def test_girirax_configurations_that_are_refused(tmp_path, Model, edit, words):
+    cfg = copy.deepcopy(GM.SMALL["state_first"])
+    W = GM.weights(cfg)
     edit(cfg)
     assert words in refused(Model, LM.write(tmp_path / "m", cfg, W))
 
@@ -97,10 +120,10 @@ def test_malformed_safetensors(tmp_path, Model):
     assert "not found" in refused(Model, tmp_path / "nowhere")
 
 
-@pytest.mark.parametrize("name", list(LM.SMALL))
-def test_oracle_does_not_depend_on_the_cut(name):
-    cfg = LM.SMALL[name]
-    o = O.Oracle(cfg, LM.weights(cfg, 3))
+@pytest.mark.parametrize("oracle,models,name", [(O, LM, n) for n in LM.SMALL] + [(GO, GM, n) for n in GM.SMALL])
+def test_oracle_does_not_depend_on_the_cut(oracle, models, name):
+    cfg = models.SMALL[name]
+    o = oracle.Oracle(cfg, models.weights(cfg, 3))
     t = [int(x) for x in np.random.default_rng(4).integers(0, cfg["vocab"], 60)]
     whole = o.feed(t)
     o.reset()
@@ -128,3 +151,34 @@ def test_oracle_mechanisms_against_closed_forms():
     assert np.allclose(O.position_vector(0, 6), [0, 1, 0, 1, 0, 1])
     assert O.layer_runs({"layers": [{}] * 4, "loop": {"start": 1, "stop": 3, "times": 2}}) == \
         [(0, None), (1, 0), (2, None), (1, 1), (2, None), (3, None)]
+
+
+def test_girirax_mechanisms_against_closed_forms():
+    """Cases whose answers can be written down."""
+    g = np.random.default_rng(0)
+    # constant inputs: the state is a geometric sum, read by C, with the skip beside it
+    one = np.ones((6, 1))
+    x = np.arange(1.0, 7.0)[:, None]
+    a = np.exp(-2.0 * 0.3)
+    y, S = GO.state_space(x, one, 3 * one, 0.3 * one, np.log([2.0]), [0.5], 1, 1, 1, 1)
+    want = [3 * sum(0.3 * x[s, 0] * a ** (t - s) for s in range(t + 1)) + 0.5 * x[t, 0] for t in range(6)]
+    assert np.allclose(y[:, 0], want)
+    # heads of a group read its B and C: with B = 0 in group 1 only heads 0 and 1 write
+    B = np.concatenate([np.ones((4, 2)), np.zeros((4, 2))], axis=1)
+    y, S = GO.state_space(np.ones((4, 4)), B, B, np.ones((4, 4)), np.zeros(4), np.zeros(4), 4, 2, 2, 1)
+    assert (y[:, :2] > 0).all() and not y[:, 2:].any() and S[1].any() and not S[2].any()
+    y, tail = GO.causal_conv(x, np.array([[100.0, 10.0, 1.0]]), np.array([0.5]), np.zeros((2, 1)))
+    assert np.allclose(y[:, 0], [1.5, 12.5, 123.5, 234.5, 345.5, 456.5]) and np.allclose(tail[:, 0], [5, 6])
+    # a rotation keeps lengths, and products depend on the distance
+    u, v = g.standard_normal(8), g.standard_normal(8)
+    turned = [GO.rotate_half(u, p + 5, 50.0) @ GO.rotate_half(v, p, 50.0) for p in (0, 3, 1000)]
+    assert np.allclose(turned, turned[0]) and np.isclose(np.linalg.norm(GO.rotate_half(u, 77, 9.0)), np.linalg.norm(u))
+    assert np.allclose(GO.rotate_half(np.array([1.0, 0, 0, 0]), 1, 100.0), [np.cos(1), 0, np.sin(1), 0])
+    assert np.allclose(GO.rotate_half(np.array([0, 1.0, 0, 0]), 2, 100.0), [0, np.cos(0.2), 0, np.sin(0.2)])
+    # equal scores: the mean of the values
+    k = g.standard_normal((5, 3))
+    assert np.allclose(GO.attend(np.zeros(3), k, k, 1.0), k.mean(axis=0))
+    n = GO.grouped_rms_norm(np.array([[3.0, 4.0, 0.0, 2.0]]), np.array([1.0, 1.0, 1.0, 10.0]), 2, 0.0)
+    assert np.allclose(n, [[3 / np.sqrt(12.5), 4 / np.sqrt(12.5), 0, 10 * np.sqrt(2)]])
+    assert np.allclose(GO.gelu_tanh(np.array([0.0, 40.0, -40.0])), [0, 40, 0]) and np.isclose(GO.gelu_tanh(1.0), 0.841192, atol=1e-6)
+    assert np.allclose(GO.softplus(np.array([-800.0, 0.0, 800.0])), [0, np.log(2), 800])

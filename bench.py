@@ -565,74 +565,153 @@ def lusadra_config(z):
             "layers": [layer] * z["layers"], "loop": None}
 
 
+# Girirax: state-space and latent-attention layers in turn, state-space heads for twice the width.
+GIRIRAX_SIZES = {
+    "small": dict(layers=12, vocab=32000, width=896, ssm=(28, 64, 128, 1), latent=(14, 64, 32, 64, 256, 384), ff=4864),
+    "medium": dict(layers=8, vocab=32000, width=2048, ssm=(64, 64, 128, 8), latent=(16, 128, 64, 128, 512, 768), ff=8192),
+    "large": dict(layers=4, vocab=32000, width=3584, ssm=(112, 64, 128, 8), latent=(28, 128, 64, 128, 512, 1536), ff=18944),
+}
+
+
+def girirax_config(z):
+    h, p, n, g = z["ssm"]
+    H, D, R, V, L, Q = z["latent"]
+    mlp = {"kind": "dense", "ff": z["ff"]}
+    ssm = {"type": "mamba2", "mlp": mlp,
+           "mixer": {"heads": h, "vdim": p, "state": n, "groups": g, "conv": 4, "norm_groups": g}}
+    att = {"type": "latent_attention", "mlp": mlp,
+           "mixer": {"heads": H, "dim": D, "rot_dim": R, "vdim": V, "kv_rank": L, "q_rank": Q, "scale": (D + R) ** -0.5,
+                     "rot": {"base": 1e6, "dims": R}}}
+    return {"architecture": "Girirax", "vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-6},
+            "embedding": {"scale": 4.0}, "residual_mult": 0.5, "layers": [ssm, att] * (z["layers"] // 2)}
+
+
+def girirax_weights(z):
+    """Weights of a state-space layer, of an attention layer, with their feed-forward."""
+    h, p, n, g = z["ssm"]
+    H, D, R, V, L, Q = z["latent"]
+    E = z["width"]
+    return (E * (3 * h * p + 2 * g * n + h + 3 * z["ff"]),
+            E * (Q + L + R + 2 * H * V + 3 * z["ff"]) + Q * H * (D + R) + L * H * (D + V))
+
+
+def lusadra_weights(z):
+    H, G, D, _ = z["left"]
+    h, d, v = z["right"]
+    return z["width"] * (3 * H * D + G * D + 2 * h * d + 3 * h * v + 16 + 2 * z["ff"])
+
+
+BENCH_T, BENCH_POS = 512, 4095       # tokens of a prompt chunk (at 3584), position of a decode step
+
+
+def best_ms(lib, call, n, rounds=4):
+    e0, e1 = lib.event(), lib.event()
+    call()
+    ms = []
+    for _ in range(rounds):
+        lib.record(e0)
+        for _ in range(n):
+            call()
+        lib.record(e1)
+        ms.append(lib.elapsed_ms(e0, e1) / n)
+    return min(ms)
+
+
+def folder_design_ms(lib, cfg, steps):
+    """(decode step, prompt chunk) of a design that is read from a folder, random weights: the recorded step at
+    position 4095, the 512-token chunk at position 3584."""
+    Model = importlib.import_module("cpp-tensorlib_amd.model").Model
+    T = BENCH_T
+    ids = np.random.default_rng(5).integers(0, 32000, T)
+    m = Model.random(cfg, seed=1, rank=16, max_ctx=8192)
+    m.stage_chunk(ids)
+    for p0 in range(0, 3584, T):
+        m.chunk_layers(T, p0)
+    chunk = best_ms(lib, lambda: m.chunk_layers(T, 3584), 2)
+    m.chunk_layers(T - 1, 3584)
+    m.capture_step(11, BENCH_POS)
+    step = best_ms(lib, m.replay_step, steps)
+    m.close()
+    return step, chunk
+
+
+def qwen_ms(lib, z, contexts, chunk_at, steps):
+    """The Qwen2.5-architecture model of size z["qwen"], bf16 weights: (weights per layer, times)."""
+    qwen = importlib.import_module("cpp-tensorlib_amd.qwen")
+    E, n, q = z["width"], z["layers"], z["qwen"]
+    g = qwen.QwenGPU(dict(n_layers=n, hidden=E, vocab=z["vocab"], max_ctx=8192, eps=1e-6, rope_base=1e6, **q))
+    g.set_random(1, fmt="bf16")
+    g.fill_cache_random(4096, 2)
+    out = {}
+    for ctx in contexts:
+        g.step(11, ctx - 1)
+        g.capture(11, ctx - 1)
+        out["decode_ms_ctx_%d" % ctx] = round(best_ms(lib, g.replay, steps), 4)
+    g.stage_chunk(np.random.default_rng(5).integers(0, 32000, BENCH_T))
+    for p0 in chunk_at:
+        out["chunk_ms_pos0_%d" % p0] = round(best_ms(lib, lambda: g.prefill_layers(BENCH_T, p0), 2), 3)
+    g.close()
+    return E * ((2 * q["n_q_heads"] + 2 * q["n_kv_heads"]) * q["head_dim"] + 3 * q["ff"]), out
+
+
+def rates(weights, head, step, chunk):
+    """weights: of all layers; head: of the output product."""
+    return {"decode_ms": round(step, 4), "decode_tok_s": round(1e3 / step, 1),
+            "decode_weight_GB/s": round(2 * (weights + head) / step / 1e6, 1), "chunk_ms": round(chunk, 3),
+            "prefill_tok_s": round(BENCH_T / chunk * 1e3, 1), "chunk_TFLOP/s": round(2.0 * BENCH_T * weights / chunk / 1e9, 1)}
+
+
 def bench_lusadra(lib, steps, only=None):
     """Decode step (hipGraph replay at position 4095) and 512-token prompt chunk (at position 3584) of the
     Lusadra sizes above beside the Qwen2.5-architecture model of the same width, bf16 weights both."""
-    qwen = importlib.import_module("cpp-tensorlib_amd.qwen")
-    Model = importlib.import_module("cpp-tensorlib_amd.model").Model
-    T, pos = 512, 4095
-    ids = np.random.default_rng(5).integers(0, 32000, T)
-    e0, e1 = lib.event(), lib.event()
-
-    def best_ms(call, n, rounds=4):
-        call()
-        ms = []
-        for _ in range(rounds):
-            lib.record(e0)
-            for _ in range(n):
-                call()
-            lib.record(e1)
-            ms.append(lib.elapsed_ms(e0, e1) / n)
-        return min(ms)
-
     out = {}
     for name, z in LUSADRA_SIZES.items():
         if only and name != only:
             continue
         H, G, D, window = z["left"]
         h, d, v = z["right"]
-        E, n = z["width"], z["layers"]
-        per_layer = E * (3 * H * D + G * D + 2 * h * d + 3 * h * v + 16 + 2 * z["ff"])
-        m = Model.random(lusadra_config(z), seed=1, rank=16, max_ctx=8192)
-        m.stage_chunk(ids)
-        for p0 in range(0, 3584, T):
-            m.chunk_layers(T, p0)
-        chunk = best_ms(lambda: m.chunk_layers(T, 3584), 2)
-        m.chunk_layers(T - 1, 3584)
-        m.capture_step(11, pos)
-        step = best_ms(m.replay_step, steps)
-        m.close()
-        state = n * (2 * h * d * v * 4 + G * min(window, pos + 1) * D * 4)
-        q = z["qwen"]
-        g = qwen.QwenGPU(dict(n_layers=n, hidden=E, vocab=z["vocab"], max_ctx=8192, eps=1e-6, rope_base=1e6, **q))
-        g.set_random(1, fmt="bf16")
-        g.fill_cache_random(4096, 2)
-        q_layer = E * ((2 * q["n_q_heads"] + 2 * q["n_kv_heads"]) * q["head_dim"] + 3 * q["ff"])
-        beside = {}
-        for ctx in sorted({window, 4096}):
-            g.step(11, ctx - 1)
-            g.capture(11, ctx - 1)
-            beside["decode_ms_ctx_%d" % ctx] = round(best_ms(g.replay, steps), 4)
-        g.stage_chunk(ids)
-        for p0 in (window - T if window >= T else 0, 3584):
-            beside["chunk_ms_pos0_%d" % p0] = round(best_ms(lambda: g.prefill_layers(T, p0), 2), 3)
-        g.close()
-        head = E * z["vocab"]
-        rate = lambda params, ms: round((2 * (n * params + head)) / ms / 1e6, 1)
-        flops = lambda params, ms: round(2.0 * T * n * params / ms / 1e9, 1)
-        out[name] = {
-            "layers": n, "width": E, "window": window, "weights_per_layer": per_layer, "qwen_weights_per_layer": q_layer,
-            "decode_ms": round(step, 4), "decode_tok_s": round(1e3 / step, 1), "decode_weight_GB/s": rate(per_layer, step),
-            "decode_state_bytes": state, "chunk_ms": round(chunk, 3), "prefill_tok_s": round(T / chunk * 1e3, 1),
-            "chunk_TFLOP/s": flops(per_layer, chunk),
-            "qwen": dict(beside, **{"decode_weight_GB/s_ctx_window": rate(q_layer, beside["decode_ms_ctx_%d" % window]),
-                                    "chunk_TFLOP/s_pos0_3584": flops(q_layer, beside["chunk_ms_pos0_3584"])})}
+        E, n, T = z["width"], z["layers"], BENCH_T
+        per_layer, head = lusadra_weights(z), E * z["vocab"]
+        step, chunk = folder_design_ms(lib, lusadra_config(z), steps)
+        state = n * (2 * h * d * v * 4 + G * min(window, BENCH_POS + 1) * D * 4)
+        q_layer, beside = qwen_ms(lib, z, sorted({window, 4096}), (window - T if window >= T else 0, 3584), steps)
+        out[name] = dict(
+            {"layers": n, "width": E, "window": window, "weights_per_layer": per_layer, "qwen_weights_per_layer": q_layer,
+             "decode_state_bytes": state}, **rates(n * per_layer, head, step, chunk),
+            qwen=dict(beside, **{
+                "decode_weight_GB/s_ctx_window": round(2 * (n * q_layer + head) / beside["decode_ms_ctx_%d" % window] / 1e6, 1),
+                "chunk_TFLOP/s_pos0_3584": round(2.0 * T * n * q_layer / beside["chunk_ms_pos0_3584"] / 1e9, 1)}))
     return out
+
+
+def bench_girirax(lib, steps, only=None):
+    """The same of the Girirax sizes above, beside Lusadra (its recurrence is the like of the state-space layers')
+    and the Qwen2.5-architecture model (full attention) of the same width and feed-forward."""
+    out = {}
+    for name, z in GIRIRAX_SIZES.items():
+        if only and name != only:
+            continue
+        H, D, R, V, L, Q = z["latent"]
+        h, p, s, g = z["ssm"]
+        n, head, l = z["layers"], z["width"] * z["vocab"], LUSADRA_SIZES[name]
+        w = sum(girirax_weights(z)) * n // 2
+        step, chunk = folder_design_ms(lib, girirax_config(z), steps)
+        state = n // 2 * (2 * h * s * p * 4 + (BENCH_POS + 1) * (2 * L + R) * 2)
+        l_step, l_chunk = folder_design_ms(lib, lusadra_config(l), steps)
+        q_layer, beside = qwen_ms(lib, l, (4096,), (3584,), steps)
+        out[name] = dict({"layers": n, "width": z["width"], "weights": w, "decode_state_bytes": state}, **rates(w, head, step, chunk),
+                         lusadra=dict({"weights": n * lusadra_weights(l)}, **rates(n * lusadra_weights(l), head, l_step, l_chunk)),
+                         qwen=dict({"weights": n * q_layer}, **rates(n * q_layer, head, beside["decode_ms_ctx_4096"],
+                                                                     beside["chunk_ms_pos0_3584"])))
+    return out
+
+
+DESIGNS = {"lusadra": bench_lusadra, "girirax": bench_girirax}
 
 
 def main():
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", default="", choices=["", "lusadra"],
+    ap.add_argument("--design", default="", choices=[""] + list(DESIGNS),
                     help="instead of the headline workload: decode and prefill of this model design at several sizes")
     ap.add_argument("--size", default="", choices=[""] + list(LUSADRA_SIZES), help="with --design: one size only")
     ap.add_argument("--gpus", type=int, default=1)
@@ -661,12 +740,12 @@ def main():
     pkg = importlib.import_module("cpp-tensorlib_amd")
     lib = pkg.load()                      # raises when the HIP library or the GPU is missing
     if a.design:
-        res = bench_lusadra(lib, a.steps, a.size or None)
+        res = DESIGNS[a.design](lib, a.steps, a.size or None)
         last = res[list(res)[-1]]
-        print(json.dumps({"metric": "lusadra_decode_tok_s", "value": last["decode_tok_s"], "unit": "tokens/s", "n_gpus": 1,
+        print(json.dumps({"metric": a.design + "_decode_tok_s", "value": last["decode_tok_s"], "unit": "tokens/s", "n_gpus": 1,
                           "steps": a.steps, "warmup": a.warmup, "ms_per_step": last["decode_ms"], "higher_is_better": True,
-                          "scaling": "weak", "vs_baseline": None, "dtype": "bf16 weights, f32 activations",
-                          "data": "synthetic, random weights", "config": {"model": "Lusadra, " + list(res)[-1], "sizes": res}}))
+                          "scaling": "weak", "vs_baseline": None, "dtype": "bf16 weights, f32 activations", "data": "synthetic, random weights",
+                          "config": {"model": a.design.capitalize() + ", " + list(res)[-1], "sizes": res}}))
         return
 
     # ---- device-resident inputs: a ring of weight copies per shape -----------------

@@ -16,9 +16,9 @@
 // (S^T = K Q^T, O^T = V^T P^T): a lane owns one query row, and the scores' registers are the second
 // product's operand as they are.
 //
-// Launches: latent_query_kernel (queries into operand images, new cache rows), latent_attend_kernel
-// (blocks: query tile x key split, four wavefronts that share a tile's dims), latent_out_kernel (splits
-// joined, uv, gate).
+// Launches: queries into operand images and new cache rows (latent_query_kernel; in prompt chunks of the one-plane
+// form latent_query_mfma_kernel), attention (latent_attend_kernel, three planes: latent_attend_exact_kernel; blocks:
+// query tile x key split), splits joined, uv, gate (latent_out_kernel; latent_out_mfma_kernel).
 #include "common.hpp"
 
 #include <algorithm>
@@ -30,6 +30,7 @@ typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef float f32x16 __attribute__((ext_vector_type(16)));
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
+typedef uint32_t u32x2 __attribute__((ext_vector_type(2)));
 
 struct Dims {
   int H, D, R, V, L, DS, LT, NC;
@@ -192,13 +193,282 @@ __global__ __launch_bounds__(256) void latent_query_kernel(const float* __restri
   }
 }
 
+// The same for chunks on the matrix cores: C^T = uk_h^T qn^T, queries in two bf16 terms. Blocks: (slice of 128 latent dims,
+// head, 128 tokens), a wavefront per 32 tokens; then rotated parts and padding (256 numbers a block); then cache rows.
+// LDS: the slice of uk_h as operand fragments [4 tiles of 32 dims][KST steps of 16][lane][8].
+constexpr int kQTok = 128;
+template <bool VEC>
+__device__ __forceinline__ void query_frag(const float* __restrict__ x, int k, int D, u32x4 (&f)[2]) {
+  float v[8];
+  if (VEC && k + 8 <= D) {
+    const f32x4 lo = *reinterpret_cast<const f32x4*>(x + k), hi = *reinterpret_cast<const f32x4*>(x + k + 4);
+#pragma unroll
+    for (int j = 0; j < 4; j++) { v[j] = lo[j]; v[4 + j] = hi[j]; }
+  } else {
+#pragma unroll
+    for (int j = 0; j < 8; j++) {
+      const float t = x[min(k + j, D - 1)];
+      v[j] = k + j < D ? t : 0.f;
+    }
+  }
+#pragma unroll
+  for (int j = 0; j < 4; j++) {
+    uint16_t a[2], b[2];
+    cut<2>(v[2 * j], a);
+    cut<2>(v[2 * j + 1], b);
+#pragma unroll
+    for (int n = 0; n < 2; n++) f[n][j] = (uint32_t)a[n] | ((uint32_t)b[n] << 16);
+  }
+}
+template <bool VEC>
+__global__ __launch_bounds__(256) void latent_query_mfma_kernel(const float* __restrict__ u, int64_t ldu, const float* __restrict__ q,
+                                                                int64_t ldq, const tlhip_latent_attn a, uint16_t* __restrict__ qimg,
+                                                                int T, int pos0, int slices, int tail_blocks) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const Dims d = dims_of(a);
+  const int tid = threadIdx.x, groups = (T + kQTok - 1) / kQTok, work = slices * d.H * groups;
+  const float sc = a.scale * 1.4426950408889634f;
+  const auto image_at = [&](int row, int e) {
+    return ((size_t)(row >> 5) * 2 * d.DS + (e >> 4)) * 512 + (((e >> 3) & 1) * 32 + (row & 31)) * 8 + (e & 7);
+  };
+  if ((int)blockIdx.x >= work + tail_blocks) {
+    const int t = (int)blockIdx.x - work - tail_blocks;
+    fill_row<1>(u + (size_t)t * ldu, a, pos0 + t, lds);
+    return;
+  }
+  if ((int)blockIdx.x >= work) {       // a pair of rotated dims, or a number of the padding
+    const int half = d.R / 2, pad = d.DS * 16 - d.L - d.R, items = half + pad;
+    const int64_t i = (int64_t)((int)blockIdx.x - work) * 256 + tid;
+    if (i >= (int64_t)T * d.H * items) return;
+    const int j = (int)(i % items), row = (int)(i / items), t = row / d.H, h = row - t * d.H;
+    const auto put = [&](int e, float v) {
+      uint16_t o[2];
+      cut<2>(v, o);
+      const size_t at = image_at(row, e);
+      qimg[at] = o[0];
+      qimg[at + (size_t)d.DS * 512] = o[1];
+    };
+    if (j >= half) {
+      put(d.L + d.R + j - half, 0.f);
+      return;
+    }
+    const float2 cs = static_cast<const float2*>(a.angles)[(size_t)(pos0 + t) * half + j];
+    const float* x = q + (size_t)t * ldq + h * (d.D + d.R) + d.D;
+    const float lo = x[j], hi = x[half + j];
+    put(d.L + j, (lo * cs.x - hi * cs.y) * sc);
+    put(d.L + half + j, (hi * cs.x + lo * cs.y) * sc);
+    return;
+  }
+  const int slice = blockIdx.x % slices, h = blockIdx.x / slices % d.H, t0 = blockIdx.x / slices / d.H * kQTok;
+  const int KST = (d.D + 15) / 16, ldk = up8(d.L);
+  u32x4* frag = reinterpret_cast<u32x4*>(lds);
+  for (int i = tid; i < 16 * 2 * KST; i += 256) {        // 8 latent dims x 8 query dims, transposed
+    const int e8 = i & 15, k8 = i >> 4, e = slice * kSliceDims + 8 * e8;
+    u32x4 x[8];
+#pragma unroll
+    for (int k = 0; k < 8; k++) {
+      x[k] = u32x4{0, 0, 0, 0};
+      if (8 * k8 + k < d.D && e < ldk)
+        x[k] = *reinterpret_cast<const u32x4*>(static_cast<const uint16_t*>(a.uk) + ((size_t)h * d.D + 8 * k8 + k) * ldk + e);
+    }
+#pragma unroll
+    for (int n = 0; n < 8; n++) {
+      u32x4 o;
+#pragma unroll
+      for (int j = 0; j < 4; j++) {
+        const uint32_t lo = x[2 * j][n >> 1], hi = x[2 * j + 1][n >> 1];
+        o[j] = n & 1 ? (lo >> 16) | (hi & 0xffff0000u) : (lo & 0xffffu) | (hi << 16);
+      }
+      const int c = 8 * e8 + n;
+      frag[((c >> 5) * KST + (k8 >> 1)) * 64 + (k8 & 1) * 32 + (c & 31)] = o;
+    }
+  }
+  __syncthreads();
+  const int lane = tid & 63, g = lane >> 5, c = lane & 31, t = t0 + (tid >> 6) * 32 + c;
+  const float* x = q + (size_t)min(t, T - 1) * ldq + h * (d.D + d.R);
+  f32x16 acc[4];
+#pragma unroll
+  for (int m = 0; m < 4; m++)
+#pragma unroll
+    for (int v = 0; v < 16; v++) acc[m][v] = 0.f;
+  u32x4 nf[2];
+  query_frag<VEC>(x, 8 * g, d.D, nf);
+  for (int st = 0; st < KST; st++) {
+    const u32x4 qf[2] = {nf[0], nf[1]};
+    query_frag<VEC>(x, min(16 * st + 16, 16 * KST - 16) + 8 * g, d.D, nf);
+#pragma unroll
+    for (int m = 0; m < 4; m++) {
+      const bf16x8 k = __builtin_bit_cast(bf16x8, frag[(m * KST + st) * 64 + lane]);
+      acc[m] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(k, __builtin_bit_cast(bf16x8, qf[1]), acc[m], 0, 0, 0);
+      acc[m] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(k, __builtin_bit_cast(bf16x8, qf[0]), acc[m], 0, 0, 0);
+    }
+  }
+  if (t >= T) return;
+  const int row = t * d.H + h;
+#pragma unroll
+  for (int m = 0; m < 4; m++)
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+      const int e = slice * kSliceDims + 32 * m + 8 * i + 4 * g;
+      uint16_t o[4][2];
+#pragma unroll
+      for (int b = 0; b < 4; b++) cut<2>(acc[m][4 * i + b] * sc, o[b]);
+#pragma unroll
+      for (int n = 0; n < 2; n++) {
+        uint16_t* at = qimg + image_at(row, e) + (size_t)n * d.DS * 512;
+        if (e + 4 <= d.L)
+          *reinterpret_cast<u32x2*>(at) = u32x2{(uint32_t)o[0][n] | ((uint32_t)o[1][n] << 16), (uint32_t)o[2][n] | ((uint32_t)o[3][n] << 16)};
+        else
+#pragma unroll
+          for (int b = 0; b < 4; b++)
+            if (e + b < d.L) at[b] = o[b][n];
+      }
+    }
+}
+
 // ---- attention -----------------------------------------------------------------------------------
 // Partials per (split, row): m [S][rows], l [S][rows], acc [S][rows][32 LT].
-// Block (query tile, split) of four wavefronts; key tiles split, split + S, ... Scores: every wavefront takes
-// each fourth dim step, the four partial sums meet in LDS and every wavefront adds them in the same order.
-// Values: wavefront w takes value tiles w, w + 4, ... (NL of them).
+// Block (query tile, split) of eight wavefronts, 64 keys at a time: pairs of key tiles split, split + S, ...
+// Scores: wavefront (k, d) takes key tile k and every fourth dim step from d, its queries in registers; the four
+// partial tiles meet in LDS and d's owner keeps eight keys of a lane pair: maximum, weights (two bf16 terms, half an
+// operand fragment) and sum are formed once. Values: wavefront w takes value tiles w, w + 8, ... (NL of them).
+template <int KS, int NL>
+__global__ __launch_bounds__(512) void latent_attend_kernel(const tlhip_latent_attn a, const uint16_t* __restrict__ qimg,
+                                                            float* __restrict__ part, int T, int pos0,
+                                                            const uint32_t* __restrict__ d_pos, int S, int rows) {
+  __shared__ f32x4 ex[8][4][64];       // partial scores of (wavefront, eight keys)
+  __shared__ u32x4 pb[4][2][64];       // weights of (16 keys, term)
+  __shared__ float mx[8][32];
+  const Dims d = dims_of(a);
+  const int tid = threadIdx.x, lane = tid & 63, g = lane >> 5, c = lane & 31;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6), kt = wave & 1, dq = wave >> 1;
+  const int rt = blockIdx.x / S, split = blockIdx.x % S;
+  const int p0 = d_pos ? (int)*d_pos : pos0;
+  const int row = rt * 32 + c;                       // this lane's query row
+  const int limit = row < T * d.H ? p0 + row / d.H : -1;
+  const int last = p0 + min(rt * 32 + 31, T * d.H - 1) / d.H, ntiles = last / 32 + 1, npairs = (ntiles + 1) / 2;
+  const u32x4* kc = reinterpret_cast<const u32x4*>(a.keys) + lane;
+  const u32x4* vc = reinterpret_cast<const u32x4*>(a.values) + lane;
+  const u32x4* qg = reinterpret_cast<const u32x4*>(qimg) + (size_t)rt * 2 * d.DS * 64 + lane;
+
+  u32x4 kr[KS], qr[KS][2];
+  const auto load_keys = [&](int pair) {             // (steps past the last: any key meets a zero query)
+    const u32x4* k = kc + (size_t)min(2 * pair + kt, ntiles - 1) * d.DS * 64;
+#pragma unroll
+    for (int i = 0; i < KS; i++) kr[i] = k[min(dq + 4 * i, d.DS - 1) * 64];
+  };
+  load_keys(split);
+#pragma unroll
+  for (int i = 0; i < KS; i++)
+#pragma unroll
+    for (int n = 0; n < 2; n++) {
+      const u32x4 x = qg[(n * d.DS + min(dq + 4 * i, d.DS - 1)) * 64];
+      qr[i][n] = dq + 4 * i < d.DS ? x : u32x4{0, 0, 0, 0};
+    }
+  f32x16 o[NL];
+#pragma unroll
+  for (int i = 0; i < NL; i++)
+#pragma unroll
+    for (int v = 0; v < 16; v++) o[i][v] = 0.f;
+  float m = -INFINITY, l = 0.f;
+  for (int pair = split; pair < npairs; pair += S) {
+    u32x4 vr[NL][4];                   // values of these keys, requested before the scores are formed
+#pragma unroll
+    for (int i = 0; i < NL; i++)
+#pragma unroll
+      for (int k = 0; k < 4; k++)
+        vr[i][k] = vc[(((size_t)min(2 * pair + (k >> 1), ntiles - 1) * d.LT + min(wave + 8 * i, d.LT - 1)) * 2 + (k & 1)) * 64];
+    f32x16 s[2];
+#pragma unroll
+    for (int n = 0; n < 2; n++)
+#pragma unroll
+      for (int v = 0; v < 16; v++) s[n][v] = 0.f;
+#pragma unroll
+    for (int i = 0; i < KS; i++)
+#pragma unroll
+      for (int n = 1; n >= 0; n--)
+        s[n] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, kr[i]), __builtin_bit_cast(bf16x8, qr[i][n]), s[n], 0, 0, 0);
+    load_keys(min(pair + S, npairs - 1));
+#pragma unroll
+    for (int i = 0; i < 4; i++)
+      ex[wave][i][lane] = f32x4{s[0][4 * i] + s[1][4 * i], s[0][4 * i + 1] + s[1][4 * i + 1], s[0][4 * i + 2] + s[1][4 * i + 2],
+                                s[0][4 * i + 3] + s[1][4 * i + 3]};
+    __syncthreads();
+    f32x4 e = ex[kt][dq][lane];
+#pragma unroll
+    for (int w = 1; w < 4; w++) e += ex[2 * w + kt][dq][lane];
+#pragma unroll
+    for (int b = 0; b < 4; b++)
+      if (64 * pair + 32 * kt + 8 * dq + 4 * g + b > limit) e[b] = -INFINITY;
+    const float mt = fmaxf(fmaxf(e[0], e[1]), fmaxf(e[2], e[3]));
+    const LanePair pr = swap32(mt, mt);
+    if (g == 0) mx[wave][c] = fmaxf(pr.first, pr.second);
+    __syncthreads();
+    float mn = m;
+#pragma unroll
+    for (int w = 0; w < 8; w++) mn = fmaxf(mn, mx[w][c]);
+    const float mz = mn == -INFINITY ? 0.f : mn;
+    const float f = exp2f(m - mz);                   // (m = -inf: 0)
+    m = mn;
+    uint16_t p[4][2];
+    float sum = 0.f;
+#pragma unroll
+    for (int b = 0; b < 4; b++) {
+      const float w = exp2f(e[b] - mz);
+      sum += w;
+      cut<2>(w, p[b]);
+    }
+    l = fmaf(l, f, sum);                             // this lane's keys
+#pragma unroll
+    for (int n = 0; n < 2; n++)
+      reinterpret_cast<u32x2*>(&pb[2 * kt + (dq >> 1)][n][lane])[dq & 1] =
+          u32x2{(uint32_t)p[0][n] | ((uint32_t)p[1][n] << 16), (uint32_t)p[2][n] | ((uint32_t)p[3][n] << 16)};
+    if (__any(f != 1.f))
+#pragma unroll
+      for (int i = 0; i < NL; i++)
+#pragma unroll
+        for (int v = 0; v < 16; v++) o[i][v] *= f;
+    __syncthreads();
+#pragma unroll
+    for (int k = 0; k < 4; k++)
+#pragma unroll
+      for (int n = 1; n >= 0; n--) {
+        const bf16x8 pf = __builtin_bit_cast(bf16x8, pb[k][n][lane]);
+#pragma unroll
+        for (int i = 0; i < NL; i++)
+          o[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, vr[i][k]), pf, o[i], 0, 0, 0);
+      }
+  }
+  const LanePair lp = swap32(l, l);
+  __syncthreads();                     // mx has been read
+  if (g == 0) mx[wave][c] = lp.first + lp.second;
+  __syncthreads();
+  const size_t R = (size_t)rows, at = (size_t)split * R + row;
+  float* pm = part;
+  float* pl = part + (size_t)S * R;
+  float* pa = pl + (size_t)S * R;
+  if (wave == 0 && g == 0) {
+    float t = mx[0][c];
+#pragma unroll
+    for (int w = 1; w < 8; w++) t += mx[w][c];
+    pm[at] = m;
+    pl[at] = t;
+  }
+#pragma unroll
+  for (int i = 0; i < NL; i++) {
+    const int lt = wave + 8 * i;
+    if (lt < d.LT)
+#pragma unroll
+      for (int k = 0; k < 4; k++)
+        *reinterpret_cast<f32x4*>(pa + at * (32 * d.LT) + 32 * lt + 8 * k + 4 * g) = f32x4{o[i][4 * k], o[i][4 * k + 1], o[i][4 * k + 2], o[i][4 * k + 3]};
+  }
+}
+
+// Every term against every term. Four wavefronts; key tiles split, split + S, ... Scores: every wavefront takes each
+// fourth dim step, the four partial sums meet in LDS and every wavefront adds them in the same order. Values:
+// wavefront w takes value tiles w, w + 4, ... (NL of them).
 template <int NL, int NC, int NQ>
-__global__ __launch_bounds__(256) void latent_attend_kernel(const tlhip_latent_attn a, const uint16_t* __restrict__ qimg,
+__global__ __launch_bounds__(256) void latent_attend_exact_kernel(const tlhip_latent_attn a, const uint16_t* __restrict__ qimg,
                                                             float* __restrict__ part, int T, int pos0,
                                                             const uint32_t* __restrict__ d_pos, int S, int rows) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
@@ -240,7 +510,6 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(const tlhip_latent_a
     f32x16 s;
 #pragma unroll
     for (int v = 0; v < 16; v++) s[v] = 0.f;
-#pragma unroll 3
     for (int st = wave; st < d.DS; st += 4) {
       u32x4 kr[NC], qr[NQ];
 #pragma unroll
@@ -322,22 +591,30 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(const tlhip_latent_a
 }
 
 // ---- splits joined, values' up-projection, gate ---------------------------------------------------
-// Block (slice of kOutRows value rows, head, TQ <= 4 tokens) of 256 threads.
+// Block (slice of kOutRows value rows, head, TQ <= 4 tokens) of NT threads; G groups of threads share the splits.
 constexpr int kMaxSplits = 64;
 constexpr int kOutRows = 32;
-template <int TQ>
-__global__ __launch_bounds__(256) void latent_out_kernel(const float* __restrict__ u, int64_t ldu, float* __restrict__ y, int64_t ldy,
-                                                         const tlhip_latent_attn a, const float* __restrict__ part, int T, int S,
-                                                         int rows, int slices) {
+__host__ __device__ inline int out_groups(int NT, int TQ, int LV) { const int n = TQ * (LV / 4); return n >= NT ? 1 : NT / n; }
+template <int TQ, int NT>
+__global__ __launch_bounds__(NT) void latent_out_kernel(const float* __restrict__ u, int64_t ldu, float* __restrict__ y, int64_t ldy,
+                                                        const tlhip_latent_attn a, const float* __restrict__ part, int T, int S,
+                                                        int rows, int slices) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
+  constexpr int NW = NT / 64;
   const Dims d = dims_of(a);
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int slice = blockIdx.x % slices, h = blockIdx.x / slices % d.H, t0 = blockIdx.x / slices / d.H * TQ;
-  const int nt = min(TQ, T - t0), LV = 32 * d.LT, ldv = up8(d.L);
-  float* oc = lds;                     // [TQ][LV] normalised sums of latents
-  float* w = oc + TQ * LV;             // [TQ][S] the splits' weights
+  const int nt = min(TQ, T - t0), LV = 32 * d.LT, ldv = up8(d.L), n8 = ldv / 8, G = out_groups(NT, TQ, LV), items = TQ * (LV / 4);
+  float* oc = lds;                     // [G][TQ][LV] sums of latents, normalised
+  float* w = oc + G * TQ * LV;         // [TQ][S] the splits' weights
   const size_t R = (size_t)rows;
   const float *pm = part, *pl = part + (size_t)S * R, *pa = pl + (size_t)S * R;
+  const int v1 = min(d.V, (slice + 1) * kOutRows), vw = slice * kOutRows + wave;
+  const u32x4* uv = reinterpret_cast<const u32x4*>(static_cast<const uint16_t*>(a.uv)) + (size_t)h * d.V * n8;
+  constexpr int PRE = kOutRows / NW < 2 ? 1 : 2;     // rows whose weights are requested up front
+  u32x4 pre[PRE];
+#pragma unroll
+  for (int i = 0; i < PRE; i++) pre[i] = uv[(size_t)min(vw + i * NW, d.V - 1) * n8 + min(lane, n8 - 1)];
   if (wave < TQ) {                     // a wavefront weighs the (up to 64) splits of one token
     const int row = (t0 + min(wave, nt - 1)) * d.H + h;
     const float m = lane < S ? pm[lane * R + row] : -INFINITY, l = lane < S ? pl[lane * R + row] : 0.f;
@@ -345,32 +622,44 @@ __global__ __launch_bounds__(256) void latent_out_kernel(const float* __restrict
     if (lane < S) w[wave * S + lane] = f / tot;
   }
   __syncthreads();
-  for (int i = tid; i < TQ * (LV / 4); i += 256) {
-    const int t = i / (LV / 4), e = 4 * (i - t * (LV / 4));
+  for (int i = tid; i < items * G; i += NT) {
+    const int grp = i / items, j = i - grp * items, t = j / (LV / 4), e = 4 * (j - t * (LV / 4));
     const float* src = pa + ((size_t)(t0 + min(t, nt - 1)) * d.H + h) * LV + e;
     f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-    for (int s0 = 0; s0 < S; s0 += 8) {
+    for (int s0 = grp; s0 < S; s0 += 8 * G) {
       f32x4 v[8];
 #pragma unroll
-      for (int k = 0; k < 8; k++) v[k] = *reinterpret_cast<const f32x4*>(src + (size_t)min(s0 + k, S - 1) * R * LV);
+      for (int k = 0; k < 8; k++) v[k] = *reinterpret_cast<const f32x4*>(src + (size_t)min(s0 + k * G, S - 1) * R * LV);
 #pragma unroll
       for (int k = 0; k < 8; k++)
-        if (s0 + k < S) {
-          const float f = w[t * S + s0 + k];
+        if (s0 + k * G < S) {
+          const float f = w[t * S + s0 + k * G];
           acc += v[k] * f;
         }
     }
-    *reinterpret_cast<f32x4*>(oc + t * LV + e) = acc;
+    *reinterpret_cast<f32x4*>(oc + grp * TQ * LV + t * LV + e) = acc;
   }
   __syncthreads();
-  const int v1 = min(d.V, (slice + 1) * kOutRows), n8 = ldv / 8;
-  const u32x4* uv = reinterpret_cast<const u32x4*>(static_cast<const uint16_t*>(a.uv)) + (size_t)h * d.V * n8;
-  for (int v = slice * kOutRows + wave; v < v1; v += 4) {
+  if (G > 1) {
+    for (int i = tid; i < TQ * LV; i += NT) {
+      float t = oc[i];
+      for (int k = 1; k < G; k++) t += oc[k * TQ * LV + i];
+      oc[i] = t;
+    }
+    __syncthreads();
+  }
+  for (int v = vw, i = 0; v < v1; v += NW, i++) {
     float acc[TQ];
 #pragma unroll
     for (int t = 0; t < TQ; t++) acc[t] = 0.f;
     for (int k = lane; k < n8; k += 64) {
-      const u32x4 x = uv[(size_t)v * n8 + k];
+      u32x4 x;
+      if (k == lane && i < PRE) {
+        x = pre[0];
+        if (PRE > 1 && i == 1) x = pre[PRE - 1];
+      } else {
+        x = uv[(size_t)v * n8 + k];
+      }
 #pragma unroll
       for (int t = 0; t < TQ; t++) {
         const f32x4 c0 = *reinterpret_cast<const f32x4*>(oc + t * LV + 8 * k), c1 = *reinterpret_cast<const f32x4*>(oc + t * LV + 8 * k + 4);
@@ -396,6 +685,102 @@ __global__ __launch_bounds__(256) void latent_out_kernel(const float* __restrict
   }
 }
 
+// The same for chunks on the matrix cores: block (head, 32 tokens) of 256 threads, y^T = uv_h oc^T with the joined
+// latents in two bf16 terms as operand fragments in LDS [KST steps of 16][term][lane][8]; a wavefront per 32 values.
+// VEC: rows of u and y take 16-byte accesses.
+template <bool VEC>
+__global__ __launch_bounds__(256) void latent_out_mfma_kernel(const float* __restrict__ u, int64_t ldu, float* __restrict__ y, int64_t ldy,
+                                                              const tlhip_latent_attn a, const float* __restrict__ part, int T, int S,
+                                                              int rows) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const Dims d = dims_of(a);
+  const int tid = threadIdx.x, lane = tid & 63, g = lane >> 5, c = lane & 31;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int h = blockIdx.x % d.H, t0 = blockIdx.x / d.H * 32, nt = min(32, T - t0);
+  const int LV = 32 * d.LT, KST = 2 * d.LT, ldv = up8(d.L);
+  u32x4* frag = reinterpret_cast<u32x4*>(lds);
+  float* w = lds + (size_t)KST * 512;  // [32][S] the splits' weights
+  const size_t R = (size_t)rows;
+  const float *pm = part, *pl = part + (size_t)S * R, *pa = pl + (size_t)S * R;
+  if (S == 1) {
+    if (tid < 32) w[tid] = 1.f / pl[(t0 + min(tid, nt - 1)) * d.H + h];
+  } else {
+    for (int t = wave; t < 32; t += 4) {
+      const int row = (t0 + min(t, nt - 1)) * d.H + h;
+      const float m = lane < S ? pm[lane * R + row] : -INFINITY, l = lane < S ? pl[lane * R + row] : 0.f;
+      const float f = exp2f(m - wave_max(m)), tot = wave_sum(f * l);
+      if (lane < S) w[t * S + lane] = f / tot;
+    }
+  }
+  __syncthreads();
+  for (int i = tid; i < 32 * 2 * KST; i += 256) {        // 8 latent dims of a token; 16 tokens x 4 runs to a wavefront
+    const int t = ((i >> 2) & 15) + 16 * ((i >> 6) & 1), r = (i & 3) + 4 * (i >> 7);
+    const float* src = pa + ((size_t)(t0 + min(t, nt - 1)) * d.H + h) * LV + 8 * r;
+    f32x4 lo = {0.f, 0.f, 0.f, 0.f}, hi = lo;
+    for (int s = 0; s < S; s++) {
+      const float f = w[t * S + s];
+      lo += *reinterpret_cast<const f32x4*>(src + (size_t)s * R * LV) * f;
+      hi += *reinterpret_cast<const f32x4*>(src + (size_t)s * R * LV + 4) * f;
+    }
+    u32x4 o[2];
+#pragma unroll
+    for (int j = 0; j < 4; j++) {
+      uint16_t x[2], z[2];
+      cut<2>(j < 2 ? lo[2 * j] : hi[2 * j - 4], x);
+      cut<2>(j < 2 ? lo[2 * j + 1] : hi[2 * j - 3], z);
+#pragma unroll
+      for (int n = 0; n < 2; n++) o[n][j] = (uint32_t)x[n] | ((uint32_t)z[n] << 16);
+    }
+#pragma unroll
+    for (int n = 0; n < 2; n++) frag[((r >> 1) * 2 + n) * 64 + (r & 1) * 32 + t] = o[n];
+  }
+  __syncthreads();
+  const uint16_t* uv = static_cast<const uint16_t*>(a.uv) + (size_t)h * d.V * ldv;
+  for (int vt = wave; 32 * vt < d.V; vt += 4) {
+    const uint16_t* wr = uv + (size_t)min(32 * vt + c, d.V - 1) * ldv;
+    f32x16 acc;
+#pragma unroll
+    for (int v = 0; v < 16; v++) acc[v] = 0.f;
+    const auto weights = [&](int st) -> u32x4 {
+      const int k = 16 * st + 8 * g;
+      const u32x4 x = *reinterpret_cast<const u32x4*>(wr + min(k, ldv - 8));
+      return k < ldv ? x : u32x4{0, 0, 0, 0};
+    };
+    u32x4 x[2] = {weights(0), weights(1)};
+    for (int s0 = 0; s0 < KST; s0 += 2) {
+      u32x4 nx[2] = {weights(min(s0 + 2, KST - 2)), weights(min(s0 + 3, KST - 1))};
+#pragma unroll
+      for (int k = 0; k < 2; k++) {
+#pragma unroll
+        for (int n = 1; n >= 0; n--)
+          acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, x[k]),
+                                                        __builtin_bit_cast(bf16x8, frag[((s0 + k) * 2 + n) * 64 + lane]), acc, 0, 0, 0);
+        x[k] = nx[k];
+      }
+    }
+    if (c >= nt) continue;
+    const float* gate = u + (size_t)(t0 + c) * ldu + a.gate_off + h * d.V;
+    float* out = y + (size_t)(t0 + c) * ldy + a.y_off + h * d.V;
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+      const int v = 32 * vt + 8 * i + 4 * g;
+      f32x4 o = {acc[4 * i], acc[4 * i + 1], acc[4 * i + 2], acc[4 * i + 3]};
+      if (VEC && v + 4 <= d.V) {
+        if (a.gate_off >= 0) {
+          const f32x4 z = *reinterpret_cast<const f32x4*>(gate + v);
+#pragma unroll
+          for (int b = 0; b < 4; b++) o[b] = o[b] / (1.f + expf(-z[b]));
+        }
+        *reinterpret_cast<f32x4*>(out + v) = o;
+      } else {
+#pragma unroll
+        for (int b = 0; b < 4; b++)
+          if (v + b < d.V) out[v + b] = a.gate_off >= 0 ? o[b] / (1.f + expf(-gate[v + b])) : o[b];
+      }
+    }
+  }
+}
+
 static int check(const tlhip_latent_attn* a, const char* who) {
   if (!a || a->heads <= 0 || a->dim <= 0 || a->rot_dim < 0 || a->rot_dim % 2 || a->vdim <= 0 || a->kv_rank <= 0)
     return fail(TLHIP_EINVAL, "%s: bad sizes", who);
@@ -412,15 +797,32 @@ static int check(const tlhip_latent_attn* a, const char* who) {
 // Splits of the keys. A decode step's plan does not depend on the position (it may be on the device).
 static int splits(const tlhip_latent_attn* a, int64_t T, int64_t pos0) {
   const int cus = ctx().cus > 0 ? ctx().cus : 256;
-  const int64_t rts = (T * a->heads + 31) / 32, tiles = T == 1 ? a->capacity / 32 : (pos0 + T + 31) / 32;
+  const int64_t keys = a->planes == 1 ? 64 : 32;     // of a block at a time
+  const int64_t rts = (T * a->heads + 31) / 32, runs = ((T == 1 ? a->capacity : pos0 + T) + keys - 1) / keys;
   int64_t S = T == 1 ? kMaxSplits : (cus + rts - 1) / rts;
   if (T == 1) S = std::max<int64_t>(1, std::min<int64_t>(S, 2 * cus / rts));
-  return (int)std::max<int64_t>(1, std::min<int64_t>({S, tiles, kMaxSplits}));
+  return (int)std::max<int64_t>(1, std::min<int64_t>({S, runs, kMaxSplits}));
+}
+
+typedef void (*attend_fn)(const tlhip_latent_attn, const uint16_t*, float*, int, int, const uint32_t*, int, int);
+template <int KS>
+static attend_fn pick_values(int nl) {
+  return nl <= 1 ? latent_attend_kernel<KS, 1> : nl <= 2 ? latent_attend_kernel<KS, 2> : latent_attend_kernel<KS, 4>;
+}
+static attend_fn pick_attend(const Dims& d) {
+  const int ks = (d.DS + 3) / 4, nl = (d.LT + 7) / 8;
+  return ks <= 3 ? pick_values<3>(nl) : ks <= 5 ? pick_values<5>(nl) : ks <= 9 ? pick_values<9>(nl) : ks <= 17 ? pick_values<17>(nl) : nullptr;
+}
+static attend_fn pick_attend_exact(const Dims& d) {
+  const int nl = (d.LT + 3) / 4;
+  return nl <= 1 ? latent_attend_exact_kernel<1, 3, 3> : nl <= 2 ? latent_attend_exact_kernel<2, 3, 3>
+                       : nl <= 4 ? latent_attend_exact_kernel<4, 3, 3> : latent_attend_exact_kernel<8, 3, 3>;
 }
 
 template <int NC, int NQ>
 static int launch(const float* u, int64_t ldu, const float* q, int64_t ldq, float* y, int64_t ldy, const tlhip_latent_attn& a, int T,
                   int pos0, const uint32_t* d_pos) {
+  constexpr bool kExact = NC == 3;
   Context& c = ctx();
   const Dims d = dims_of(a);
   const int rts = (T * d.H + 31) / 32, rows = rts * 32, S = splits(&a, T, pos0), LV = 32 * d.LT;
@@ -435,22 +837,40 @@ static int launch(const float* u, int64_t ldu, const float* q, int64_t ldq, floa
     const hipError_t e = hipFuncSetAttribute(fn, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     return e == hipSuccess ? (int)TLHIP_OK : hip_fail(e, "hipFuncSetAttribute(LDS)");
   };
-  const int TQ = T == 1 ? 1 : 4, tiles = (T + TQ - 1) / TQ, slices = (d.DS * 16 + kSliceDims - 1) / kSliceDims;
-  const size_t lq = (size_t)(TQ * d.D + 16 * 16 * 8) * sizeof(float);
+  // plan everything, then launch
+  const int TQ = T == 1 ? 1 : 4, tiles = (T + TQ - 1) / TQ;
+  const size_t lqm = (size_t)((d.D + 15) / 16) * 4096, lom = (size_t)d.LT * 4096 + (size_t)32 * S * sizeof(float);
+  const bool q_mfma = !kExact && T > 1 && lqm <= 128 * 1024, o_mfma = !kExact && T > 1 && lom <= (size_t)c.lds_per_cu;
+  const int slices = q_mfma ? (d.L + kSliceDims - 1) / kSliceDims : (d.DS * 16 + kSliceDims - 1) / kSliceDims;
+  const bool q_vec = ldq % 4 == 0 && (d.D + d.R) % 4 == 0 && aligned16(q);
+  const bool o_vec = ldy % 4 == 0 && a.y_off % 4 == 0 && d.V % 4 == 0 && aligned16(y) &&
+                     (a.gate_off < 0 || (ldu % 4 == 0 && a.gate_off % 4 == 0 && aligned16(u)));
+  const size_t lq = q_mfma ? lqm : (size_t)(TQ * d.D + 16 * 16 * 8) * sizeof(float);
   auto fq = TQ == 1 ? latent_query_kernel<1, NC, NQ> : latent_query_kernel<4, NC, NQ>;
-  if (int rc = allow(reinterpret_cast<const void*>(fq), lq)) return rc;
-  const size_t la = (size_t)NQ * d.DS * 1024 + 2 * 16 * 1024;
-  const int nl = (d.LT + 3) / 4;
-  auto fa = nl <= 1 ? latent_attend_kernel<1, NC, NQ> : nl <= 2 ? latent_attend_kernel<2, NC, NQ> : nl <= 4 ? latent_attend_kernel<4, NC, NQ>
-                                                                                                    : latent_attend_kernel<8, NC, NQ>;
+  auto fqm = q_vec ? latent_query_mfma_kernel<true> : latent_query_mfma_kernel<false>;
+  if (int rc = allow(q_mfma ? reinterpret_cast<const void*>(fqm) : reinterpret_cast<const void*>(fq), lq)) return rc;
+  const attend_fn fa = kExact ? pick_attend_exact(d) : pick_attend(d);
+  if (!fa) return fail(TLHIP_EUNSUPPORTED, "tlhip_latent_attn: latent and rotated dims beyond what the kernel holds");
+  const size_t la = kExact ? (size_t)NQ * d.DS * 1024 + 2 * 16 * 1024 : 0;
   if (int rc = allow(reinterpret_cast<const void*>(fa), la)) return rc;
-  const int oslices = (d.V + kOutRows - 1) / kOutRows;
-  const size_t lo = (size_t)TQ * (LV + S) * sizeof(float);
-  auto fo = TQ == 1 ? latent_out_kernel<1> : latent_out_kernel<4>;
-  if (int rc = allow(reinterpret_cast<const void*>(fo), lo)) return rc;
-  hipLaunchKernelGGL(fq, dim3((unsigned)(slices * d.H * tiles + T)), dim3(256), lq, c.stream, u, ldu, q, ldq, a, qimg, T, pos0, d_pos, slices);
-  hipLaunchKernelGGL(fa, dim3((unsigned)(rts * S)), dim3(256), la, c.stream, a, qimg, part, T, pos0, d_pos, S, rows);
-  hipLaunchKernelGGL(fo, dim3((unsigned)(oslices * d.H * tiles)), dim3(256), lo, c.stream, u, ldu, y, ldy, a, part, T, S, rows, oslices);
+  const int oslices = (d.V + kOutRows - 1) / kOutRows, ont = TQ == 1 ? 1024 : 256;
+  const size_t lo = o_mfma ? lom : (size_t)TQ * (out_groups(ont, TQ, LV) * LV + S) * sizeof(float);
+  auto fo = TQ == 1 ? latent_out_kernel<1, 1024> : latent_out_kernel<4, 256>;
+  auto fom = o_vec ? latent_out_mfma_kernel<true> : latent_out_mfma_kernel<false>;
+  if (int rc = allow(o_mfma ? reinterpret_cast<const void*>(fom) : reinterpret_cast<const void*>(fo), lo)) return rc;
+
+  if (q_mfma) {
+    const int64_t items = (int64_t)T * d.H * (d.R / 2 + d.DS * 16 - d.L - d.R), work = (int64_t)slices * d.H * ((T + kQTok - 1) / kQTok);
+    const int tail = (int)((items + 255) / 256);
+    hipLaunchKernelGGL(fqm, dim3((unsigned)(work + tail + T)), dim3(256), lq, c.stream, u, ldu, q, ldq, a, qimg, T, pos0, slices, tail);
+  } else {
+    hipLaunchKernelGGL(fq, dim3((unsigned)(slices * d.H * tiles + T)), dim3(256), lq, c.stream, u, ldu, q, ldq, a, qimg, T, pos0, d_pos, slices);
+  }
+  hipLaunchKernelGGL(fa, dim3((unsigned)(rts * S)), dim3(kExact ? 256 : 512), la, c.stream, a, qimg, part, T, pos0, d_pos, S, rows);
+  if (o_mfma)
+    hipLaunchKernelGGL(fom, dim3((unsigned)(d.H * ((T + 31) / 32))), dim3(256), lo, c.stream, u, ldu, y, ldy, a, part, T, S, rows);
+  else
+    hipLaunchKernelGGL(fo, dim3((unsigned)(oslices * d.H * tiles)), dim3((unsigned)ont), lo, c.stream, u, ldu, y, ldy, a, part, T, S, rows, oslices);
   TLHIP_CHECK_LAUNCH(TLHIP_C_LATENT_ATTN);
 }
 

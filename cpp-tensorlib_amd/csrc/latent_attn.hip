@@ -615,6 +615,14 @@ __global__ __launch_bounds__(NT) void latent_out_kernel(const float* __restrict_
   u32x4 pre[PRE];
 #pragma unroll
   for (int i = 0; i < PRE; i++) pre[i] = uv[(size_t)min(vw + i * NW, d.V - 1) * n8 + min(lane, n8 - 1)];
+  f32x4 v[8];                          // eight splits' latents of this thread's item, the first ones before the weights are known
+  const auto load_splits = [&](int i, int s0) {
+    const int j = i % items, t = j / (LV / 4), e = 4 * (j - t * (LV / 4));
+    const float* src = pa + ((size_t)(t0 + min(t, nt - 1)) * d.H + h) * LV + e;
+#pragma unroll
+    for (int k = 0; k < 8; k++) v[k] = *reinterpret_cast<const f32x4*>(src + (size_t)min(s0 + k * G, S - 1) * R * LV);
+  };
+  load_splits(tid, tid / items);
   if (wave < TQ) {                     // a wavefront weighs the (up to 64) splits of one token
     const int row = (t0 + min(wave, nt - 1)) * d.H + h;
     const float m = lane < S ? pm[lane * R + row] : -INFINITY, l = lane < S ? pl[lane * R + row] : 0.f;
@@ -624,12 +632,9 @@ __global__ __launch_bounds__(NT) void latent_out_kernel(const float* __restrict_
   __syncthreads();
   for (int i = tid; i < items * G; i += NT) {
     const int grp = i / items, j = i - grp * items, t = j / (LV / 4), e = 4 * (j - t * (LV / 4));
-    const float* src = pa + ((size_t)(t0 + min(t, nt - 1)) * d.H + h) * LV + e;
     f32x4 acc = {0.f, 0.f, 0.f, 0.f};
     for (int s0 = grp; s0 < S; s0 += 8 * G) {
-      f32x4 v[8];
-#pragma unroll
-      for (int k = 0; k < 8; k++) v[k] = *reinterpret_cast<const f32x4*>(src + (size_t)min(s0 + k * G, S - 1) * R * LV);
+      if (i != tid || s0 != grp) load_splits(i, s0);
 #pragma unroll
       for (int k = 0; k < 8; k++)
         if (s0 + k * G < S) {

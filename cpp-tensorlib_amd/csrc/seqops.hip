@@ -102,26 +102,40 @@ __global__ __launch_bounds__(1024) void postnorm_rows_kernel(const float* x, con
 }
 
 // Block (row) of 256 threads; a wavefront norms whole runs, or the four share one where there are fewer than four.
+// VEC: runs and rows of whole float4s. A thread keeps up to kKeep of its entries.
+template <bool VEC>
 __global__ __launch_bounds__(256) void rms_rows_kernel(const float* x, int64_t ldx, const float* __restrict__ w, float* out,
                                                        int64_t ldo, int n, int n_out, int parts, float eps) {
+  typedef float vec __attribute__((ext_vector_type(VEC ? 4 : 1)));
+  constexpr int E = VEC ? 4 : 1, kKeep = 4;
   __shared__ float red[4];
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, len = n / parts;
-  const float* r = x + (size_t)blockIdx.x * ldx;
+  const int tid = threadIdx.x, len = n / parts / E;
+  const bool whole = parts < 4;        // the block shares a run
+  const int at = whole ? tid : tid & 63, step = whole ? 256 : 64;
   float* o = out + (size_t)blockIdx.x * ldo;
-  if (parts >= 4) {
-    for (int p = wave; p < parts; p += 4) {
-      float ss = 0.f;
-      for (int i = lane; i < len; i += 64) ss = fmaf(r[p * len + i], r[p * len + i], ss);
-      const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)len + eps);
-      for (int i = lane; i < len; i += 64) o[p * len + i] = r[p * len + i] * inv * w[p * len + i];
-    }
-  } else {
-    for (int p = 0; p < parts; p++) {
-      float ss = 0.f;
-      for (int i = tid; i < len; i += 256) ss = fmaf(r[p * len + i], r[p * len + i], ss);
-      const float inv = 1.0f / sqrtf(block_sum<4>(ss, red) / (float)len + eps);
-      for (int i = tid; i < len; i += 256) o[p * len + i] = r[p * len + i] * inv * w[p * len + i];
-    }
+  for (int p = whole ? 0 : tid >> 6; p < parts; p += whole ? 1 : 4) {
+    const vec* r = reinterpret_cast<const vec*>(x + (size_t)blockIdx.x * ldx) + p * len;
+    const vec* wr = reinterpret_cast<const vec*>(w) + p * len;
+    vec* q = reinterpret_cast<vec*>(o) + p * len;
+    const auto square = [](vec v) {
+      float s = 0.f;
+#pragma unroll
+      for (int e = 0; e < E; e++) s = fmaf(v[e], v[e], s);
+      return s;
+    };
+    vec v[kKeep];
+    float ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < kKeep; k++) v[k] = r[min(at + k * step, len - 1)];
+#pragma unroll
+    for (int k = 0; k < kKeep; k++)
+      if (at + k * step < len) ss += square(v[k]);
+    for (int i = at + kKeep * step; i < len; i += step) ss += square(r[i]);
+    const float inv = 1.0f / sqrtf((whole ? block_sum<4>(ss, red) : wave_sum(ss)) / (float)(len * E) + eps);
+#pragma unroll
+    for (int k = 0; k < kKeep; k++)
+      if (at + k * step < len) q[at + k * step] = v[k] * inv * wr[at + k * step];
+    for (int i = at + kKeep * step; i < len; i += step) q[i] = r[i] * inv * wr[i];
   }
   for (int i = n + tid; i < n_out; i += 256) o[i] = 0.f;
 }
@@ -224,8 +238,10 @@ int tlhip_rms_rows(const void* x, int64_t ldx, const void* w, void* out, int64_t
   if (!x || !w || !out) return fail(TLHIP_EINVAL, "tlhip_rms_rows: null pointer");
   if (n <= 0 || n_out < n || n_out > (1 << 30) || ldx < n || ldo < n_out || parts <= 0 || n % parts || rows <= 0 || rows > (1 << 30))
     return fail(TLHIP_EINVAL, "tlhip_rms_rows: bad sizes");
-  rms_rows_kernel<<<dim3((unsigned)rows), dim3(256), 0, ctx().stream>>>(static_cast<const float*>(x), ldx, static_cast<const float*>(w),
-                                                                        static_cast<float*>(out), ldo, (int)n, (int)n_out, (int)parts, eps);
+  const bool vec = n / parts % 4 == 0 && ldx % 4 == 0 && ldo % 4 == 0 && aligned16(x) && aligned16(w) && aligned16(out);
+  hipLaunchKernelGGL(vec ? rms_rows_kernel<true> : rms_rows_kernel<false>, dim3((unsigned)rows), dim3(256), 0, ctx().stream,
+                     static_cast<const float*>(x), ldx, static_cast<const float*>(w), static_cast<float*>(out), ldo, (int)n, (int)n_out,
+                     (int)parts, eps);
   TLHIP_CHECK_LAUNCH(TLHIP_C_RMSNORM);
 }
 

@@ -8,7 +8,7 @@
 // the log decays since the piece began:
 //   y_t = 2^l_t C_t^T S_0 + sum_(s <= t) (C_t . B_s) 2^(l_t - l_s) dt_s x_s
 //   S_C = 2^l_C S_0 + sum_s 2^(l_C - l_s) dt_s B_s x_s^T
-// every exponent <= 0. Four launches: ssm_conv_kernel (convolution, activation, dt), ssm_piece_kernel
+// every exponent <= 0. Four launches: ssm_conv_kernel (convolution, activation; steps and log decays), ssm_piece_kernel
 // (each piece's own part of S_C), ssm_scan_kernel (the state through the pieces, the convolution's new
 // tail), ssm_out_kernel (y). Products on the fp32 matrix pipe.
 //
@@ -134,10 +134,33 @@ struct SsmBuf {
 
 constexpr int kConvTok = 16;         // tokens of one block of ssm_conv_kernel
 
-// Grid (columns of xbc / 256 + one for dt, token tiles). TAPS 0: any number of taps.
+// dt and the log decays summed along each piece: a wavefront owns a head and a piece, a lane a token.
+__device__ __forceinline__ void ssm_steps(const float* __restrict__ u, int64_t ldu, const tlhip_ssm& a, int T, const SsmBuf& b, int i) {
+  const int H = (int)a.heads;
+  if (i >= H * b.np) return;
+  const int lane = threadIdx.x & 63, h = i % H, t = i / H * b.C + lane;
+  const bool live = lane < b.C && t < T;
+  const float dt = softplus_f(u[(size_t)min(t, T - 1) * ldu + a.dt_off + h] + static_cast<const float*>(a.dt_bias)[h]);
+  float l = live ? static_cast<const float*>(a.decay)[h] * dt : 0.f;
+#pragma unroll
+  for (int k = 1; k < 64; k *= 2) {
+    const float o = __shfl_up(l, k, kWave);
+    if (lane >= k) l += o;
+  }
+  if (live) {
+    b.dt[(size_t)t * H + h] = dt;
+    b.lsum[(size_t)t * H + h] = l;
+  }
+}
+
+// Grid (columns of xbc / 256, then steps; token tiles). TAPS 0: any number of taps.
 template <int TAPS>
 __global__ __launch_bounds__(256) void ssm_conv_kernel(const float* __restrict__ u, int64_t ldu, const tlhip_ssm a, int T, int pos0,
-                                                       const SsmBuf b) {
+                                                       const SsmBuf b, int cols) {
+  if ((int)blockIdx.x >= cols) {
+    ssm_steps(u, ldu, a, T, b, (((int)blockIdx.x - cols) * (int)gridDim.y + (int)blockIdx.y) * 4 + ((int)threadIdx.x >> 6));
+    return;
+  }
   const SsmDims d = ssm_dims(a);
   const int j = blockIdx.x * 256 + threadIdx.x, t0 = blockIdx.y * kConvTok, t1 = min(T, t0 + kConvTok);
   if (j >= b.xw) return;
@@ -185,28 +208,6 @@ __global__ __launch_bounds__(256) void ssm_conv_kernel(const float* __restrict__
       for (int i = 0; i < d.taps; i++) s = fmaf(w[(size_t)i * d.ch], input(t - (d.taps - 1) + i), s);
       o[(size_t)t * b.xw] = silu_f(s + bias);
     }
-  }
-}
-
-// dt and the log decays summed along each piece: a thread owns a head and a piece.
-__global__ __launch_bounds__(256) void ssm_dt_kernel(const float* __restrict__ u, int64_t ldu, const tlhip_ssm a, int T, const SsmBuf b) {
-  const int H = (int)a.heads, i = blockIdx.x * 256 + threadIdx.x;
-  if (i >= H * b.np) return;
-  const int h = i % H, t0 = i / H * b.C, t1 = min(T, t0 + b.C);
-  const float bias = static_cast<const float*>(a.dt_bias)[h], dec = static_cast<const float*>(a.decay)[h];
-  float l = 0.f;
-  for (int t = t0; t < t1; t += 8) {
-    float z[8];
-#pragma unroll
-    for (int k = 0; k < 8; k++) z[k] = u[(size_t)min(t + k, t1 - 1) * ldu + a.dt_off + h];
-#pragma unroll
-    for (int k = 0; k < 8; k++)
-      if (t + k < t1) {
-        const float dt = softplus_f(z[k] + bias);
-        l = fmaf(dec, dt, l);
-        b.dt[(size_t)(t + k) * H + h] = dt;
-        b.lsum[(size_t)(t + k) * H + h] = l;
-      }
   }
 }
 
@@ -307,92 +308,139 @@ __global__ __launch_bounds__(256) void ssm_scan_kernel(const float* __restrict__
   if (kept) *reinterpret_cast<float4*>(state + (size_t)((pos0 + T) & 1) * slot + at) = s;
 }
 
-// Block (piece, run of HB heads of a group) of 256 threads: C_t . B_s once for the run, then per head both
-// terms of y, skip and gate.
+// Block (piece, head) of 512 threads: C_t . B_s with the head's decays and steps, then both terms of y, skip and gate.
+// What is needed last - x and the state ahead of the piece - is requested first.
 template <int C>
-__global__ __launch_bounds__(256) void ssm_out_kernel(const float* __restrict__ u, int64_t ldu, float* __restrict__ y, int64_t ldy,
-                                                      const tlhip_ssm a, int T, const SsmBuf b, int HB) {
+__global__ __launch_bounds__(512) __attribute__((amdgpu_waves_per_eu(4))) void ssm_out_kernel(const float* __restrict__ u, int64_t ldu, float* __restrict__ y, int64_t ldy,
+                                                      const tlhip_ssm a, int T, const SsmBuf b) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
-  constexpr int NB = C / 16, AS = C + 4;
+  constexpr int NB = C / 16, AS = C + 4, NW = 8, HALF = NB > 1 ? NB / 2 : 1;
+  constexpr int TILES = NB * (NB + 1) / 2, TW = (TILES + NW - 1) / NW;   // tiles of C . B, of a wavefront
   const SsmDims d = ssm_dims(a);
   const int tid = threadIdx.x, lane = tid & 63, l15 = lane & 15, lg = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int per = d.H / d.G, runs = (per + HB - 1) / HB;
-  const int piece = blockIdx.x, g = blockIdx.y / runs, h0 = g * per + blockIdx.y % runs * HB, h1 = min(h0 + HB, (g + 1) * per);
+  const int piece = blockIdx.x, h = blockIdx.y, g = h / (d.H / d.G);
   const int t0 = piece * C, nt = min(C, T - t0), BS = b.Np + 4, XS = b.Vp + 4;
   float* Cm = lds;                     // [C][BS]
-  float* CB = Cm + C * BS;             // [C][AS] C_t . B_s, s <= t
-  float* M = CB + C * AS;              // [C][AS] with the head's decays and steps
-  float* BX = M + C * AS;              // B [C][BS], then x of the head [C][XS]
-  float* L = BX + C * (BS > XS ? BS : XS);   // [C] log decay sums, [C] steps
+  float* B = Cm + C * BS;              // [C][BS], then
+  float* M = B;                        // [C][AS] C_t . B_s 2^(l_t - l_s) dt_s, s <= t, and
+  float* X = M + C * AS;               // [C][XS] x of the head
+  float* L = B + max(C * BS, C * (AS + XS));   // [C] log decay sums, [C] steps
   float* D = L + C;
   const float* row = b.xbc + (size_t)t0 * b.xw;
-  ssm_tile(Cm, BS, row + d.H * b.Vp + (d.G + g) * b.Np, b.xw, C, b.Np, nt, tid, 256);
-  ssm_tile(BX, BS, row + d.H * b.Vp + g * b.Np, b.xw, C, b.Np, nt, tid, 256);
+  const float* st = b.st + ((size_t)h * b.np + piece) * b.Np * b.Vp;
+  const int nvt = b.Vp / 16, v4 = b.Vp >> 2, items = nvt * (NB > 1 ? 2 : 1);
+  constexpr int XR = 2;
+  f32x4 xr[XR];
+#pragma unroll
+  for (int k = 0; k < XR; k++) {
+    const int i = min(tid + 512 * k, C * v4 - 1), t = i / v4;
+    xr[k] = *reinterpret_cast<const f32x4*>(row + (size_t)min(t, nt - 1) * b.xw + h * b.Vp + 4 * (i - t * v4));
+  }
+  float sv[2][4][4];                   // state rows n0 .. n0 + 127 of an item's columns
+  const auto load_state = [&](int item, int n0) {
+    const int v = 16 * (item % nvt) + l15;
+#pragma unroll
+    for (int q = 0; q < 2; q++)
+#pragma unroll
+      for (int k = 0; k < 4; k++)
+#pragma unroll
+        for (int e = 0; e < 4; e++) sv[q][k][e] = st[(size_t)(min(n0 + 64 * q + 16 * k, b.Np - 16) + 4 * lg + e) * b.Vp + v];
+  };
+  load_state(min(wave, items - 1), 0);
+  ssm_tile(Cm, BS, row + d.H * b.Vp + (d.G + g) * b.Np, b.xw, C, b.Np, nt, tid, 512);
+  ssm_tile(B, BS, row + d.H * b.Vp + g * b.Np, b.xw, C, b.Np, nt, tid, 512);
+  if (tid < C) {
+    const int t = t0 + min(tid, nt - 1);
+    L[tid] = b.lsum[(size_t)t * d.H + h];
+    D[tid] = tid < nt ? b.dt[(size_t)t * d.H + h] : 0.f;
+  }
   __syncthreads();
-  for (int tile = wave; tile < NB * (NB + 1) / 2; tile += 4) {
-    int i = 0, j = tile;
+  f32x4 cb[TW];
+#pragma unroll
+  for (int w = 0; w < TW; w++) {
+    cb[w] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (wave + NW * w >= TILES) continue;
+    int i = 0, j = wave + NW * w;
     while (j > i) { i++; j -= i; }
-    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
     for (int n0 = 0; n0 < b.Np; n0 += 16) {
       const f32x4 cf = *reinterpret_cast<const f32x4*>(Cm + (16 * i + l15) * BS + n0 + 4 * lg);
-      const f32x4 bf = *reinterpret_cast<const f32x4*>(BX + (16 * j + l15) * BS + n0 + 4 * lg);
+      const f32x4 bf = *reinterpret_cast<const f32x4*>(B + (16 * j + l15) * BS + n0 + 4 * lg);
 #pragma unroll
-      for (int k = 0; k < 4; k++) acc = ssm_mfma(cf[k], bf[k], acc);
+      for (int k = 0; k < 4; k++) cb[w] = ssm_mfma(cf[k], bf[k], cb[w]);
     }
-#pragma unroll
-    for (int k = 0; k < 4; k++) CB[(16 * i + 4 * lg + k) * AS + 16 * j + l15] = acc[k];
   }
-  for (int h = h0; h < h1; h++) {
-    __syncthreads();                   // B, or the head before, has been read
-    ssm_tile(BX, XS, row + h * b.Vp, b.xw, C, b.Vp, nt, tid, 256);
-    if (tid < C) {
-      const int t = t0 + min(tid, nt - 1);
-      L[tid] = b.lsum[(size_t)t * d.H + h];
-      D[tid] = tid < nt ? b.dt[(size_t)t * d.H + h] : 0.f;
-    }
-    __syncthreads();
-    for (int i = tid; i < C * C; i += 256) {
-      const int t = i / C, s = i % C;
-      if ((s >> 4) <= (t >> 4)) M[t * AS + s] = s <= t ? CB[t * AS + s] * exp2f(L[t] - L[s]) * D[s] : 0.f;
-    }
-    __syncthreads();
-    const float* st = b.st + ((size_t)h * b.np + piece) * b.Np * b.Vp;
-    const int nvt = b.Vp / 16;
-    const float skip = static_cast<const float*>(a.skip)[h];
-    // a wavefront's value tiles: two rows of blocks, i and NB - 1 - i, balance the triangle
-    for (int tile = wave; tile < NB * nvt; tile += 4) {
-      const int f = tile % NB, i = (tile / NB) & 1 ? NB - 1 - f : f, v0 = 16 * (tile / NB);
-      f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-      for (int n0 = 0; n0 < b.Np; n0 += 64) {          // the state's part, four steps requested at once
-        float sv[4][4];
+  __syncthreads();                     // B has been read
 #pragma unroll
-        for (int k = 0; k < 4; k++)
+  for (int w = 0; w < TW; w++) {
+    if (wave + NW * w >= TILES) continue;
+    int i = 0, j = wave + NW * w;
+    while (j > i) { i++; j -= i; }
+    const int s = 16 * j + l15;
 #pragma unroll
-          for (int e = 0; e < 4; e++) sv[k][e] = st[(size_t)(min(n0 + 16 * k, b.Np - 16) + 4 * lg + e) * b.Vp + v0 + l15];
+    for (int k = 0; k < 4; k++) {
+      const int t = 16 * i + 4 * lg + k;
+      M[t * AS + s] = s <= t ? cb[w][k] * exp2f(L[t] - L[s]) * D[s] : 0.f;
+    }
+  }
+  for (int i = tid, k = 0; i < C * v4; i += 512, k++) {
+    const int t = i / v4, c = 4 * (i - t * v4);
+    f32x4 v;
+    if (k == 0) v = xr[0];
+    else if (k == 1) v = xr[1];
+    else v = *reinterpret_cast<const f32x4*>(row + (size_t)min(t, nt - 1) * b.xw + h * b.Vp + c);
+    if (t >= nt) v = f32x4{0.f, 0.f, 0.f, 0.f};
+    *reinterpret_cast<f32x4*>(X + t * XS + c) = v;
+  }
+  __syncthreads();
+  const float skip = static_cast<const float*>(a.skip)[h];
+  // an item: 16 value columns and half of the row blocks, k and NB - 1 - k, which balances the triangle
+  for (int item = wave; item < items; item += NW) {
+    const int v0 = 16 * (item % nvt), half = item / nvt;
+    f32x4 acc[2];
+    float z[2][4];
+    int blk[2];
+#pragma unroll
+    for (int r = 0; r < 2; r++) {
+      blk[r] = NB == 1 ? 0 : NB == 2 ? half : r ? NB - 1 - half : half;
+      acc[r] = f32x4{0.f, 0.f, 0.f, 0.f};
+      if (r >= HALF) continue;
+#pragma unroll
+      for (int k = 0; k < 4; k++)
+        z[r][k] = u[(size_t)(t0 + min(16 * blk[r] + 4 * lg + k, nt - 1)) * ldu + a.z_off + h * d.V + min(v0 + l15, d.V - 1)];
+    }
+    if (item != wave) load_state(item, 0);
+    for (int n0 = 0; n0 < b.Np; n0 += 128) {
+      if (n0 > 0) load_state(item, n0);
+#pragma unroll
+      for (int q = 0; q < 2; q++)
 #pragma unroll
         for (int k = 0; k < 4; k++) {
-          if (n0 + 16 * k >= b.Np) break;
-          const f32x4 cf = *reinterpret_cast<const f32x4*>(Cm + (16 * i + l15) * BS + n0 + 16 * k + 4 * lg);
+          const int n = n0 + 64 * q + 16 * k;
+          if (n >= b.Np) continue;
 #pragma unroll
-          for (int e = 0; e < 4; e++) acc = ssm_mfma(cf[e], sv[k][e], acc);
+          for (int r = 0; r < HALF; r++) {
+            const f32x4 cf = *reinterpret_cast<const f32x4*>(Cm + (16 * blk[r] + l15) * BS + n + 4 * lg);
+#pragma unroll
+            for (int e = 0; e < 4; e++) acc[r] = ssm_mfma(cf[e], sv[q][k][e], acc[r]);
+          }
         }
-      }
+    }
 #pragma unroll
-      for (int k = 0; k < 4; k++) acc[k] *= exp2f(L[16 * i + 4 * lg + k]);
+    for (int r = 0; r < HALF; r++) {
+      const int i = blk[r];
+#pragma unroll
+      for (int k = 0; k < 4; k++) acc[r][k] *= exp2f(L[16 * i + 4 * lg + k]);
       for (int j = 0; j <= i; j++) {
         const f32x4 m = *reinterpret_cast<const f32x4*>(M + (16 * i + l15) * AS + 16 * j + 4 * lg);
 #pragma unroll
-        for (int e = 0; e < 4; e++) acc = ssm_mfma(m[e], BX[(16 * j + 4 * lg + e) * XS + v0 + l15], acc);
+        for (int e = 0; e < 4; e++) acc[r] = ssm_mfma(m[e], X[(16 * j + 4 * lg + e) * XS + v0 + l15], acc[r]);
       }
       const int v = v0 + l15;
 #pragma unroll
       for (int k = 0; k < 4; k++) {
         const int t = 16 * i + 4 * lg + k;
-        if (t < nt && v < d.V) {
-          const float z = u[(size_t)(t0 + t) * ldu + a.z_off + h * d.V + v];
-          y[(size_t)(t0 + t) * ldy + a.y_off + h * d.V + v] = fmaf(skip, BX[t * XS + v], acc[k]) * silu_f(z);
-        }
+        if (t < nt && v < d.V) y[(size_t)(t0 + t) * ldy + a.y_off + h * d.V + v] = fmaf(skip, X[t * XS + v], acc[r][k]) * silu_f(z[r][k]);
       }
     }
   }
@@ -400,7 +448,7 @@ __global__ __launch_bounds__(256) void ssm_out_kernel(const float* __restrict__ 
 
 static size_t ssm_piece_lds(int C, int Np, int Vp) { return (size_t)(C * (Np + 4) + C * (Vp + 4) + C) * sizeof(float); }
 static size_t ssm_out_lds(int C, int Np, int Vp) {
-  return (size_t)(C * (Np + 4) + 2 * C * (C + 4) + C * (std::max(Np, Vp) + 4) + 2 * C) * sizeof(float);
+  return (size_t)(C * (Np + 4) + std::max(C * (Np + 4), C * (C + 4 + Vp + 4)) + 2 * C) * sizeof(float);
 }
 
 static int check_ssm(const tlhip_ssm* a, const char* who) {
@@ -465,8 +513,8 @@ int tlhip_ssm_chunk(const void* u, int64_t ldu, void* y, int64_t ldy, const tlhi
   const unsigned tt = (unsigned)((T + kConvTok - 1) / kConvTok);
   if (tt > 65535) return fail(TLHIP_EUNSUPPORTED, "tlhip_ssm_chunk: chunk too long");
   auto conv = a->taps == 4 ? ssm_conv_kernel<4> : a->taps == 3 ? ssm_conv_kernel<3> : a->taps == 2 ? ssm_conv_kernel<2> : ssm_conv_kernel<0>;
-  hipLaunchKernelGGL(conv, dim3((unsigned)((b.xw + 255) / 256), tt), dim3(256), 0, c.stream, pu, ldu, *a, (int)T, (int)pos0, b);
-  hipLaunchKernelGGL(ssm_dt_kernel, dim3((unsigned)((a->heads * b.np + 255) / 256)), dim3(256), 0, c.stream, pu, ldu, *a, (int)T, b);
+  const int cols = (b.xw + 255) / 256, steps = (int)(((a->heads * b.np + 3) / 4 + tt - 1) / tt);
+  hipLaunchKernelGGL(conv, dim3((unsigned)(cols + steps), tt), dim3(256), 0, c.stream, pu, ldu, *a, (int)T, (int)pos0, b, cols);
   auto piece = b.C == 64 ? ssm_piece_kernel<64> : b.C == 32 ? ssm_piece_kernel<32> : ssm_piece_kernel<16>;
   hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(piece), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds1);
   if (e != hipSuccess) return hip_fail(e, "hipFuncSetAttribute(LDS)");
@@ -474,15 +522,11 @@ int tlhip_ssm_chunk(const void* u, int64_t ldu, void* y, int64_t ldy, const tlhi
   const size_t ns = (size_t)a->heads * b.Np * (b.Vp / 4);
   const int sb = (int)((ns + 255) / 256), ch = ssm_dims(*a).ch;
   hipLaunchKernelGGL(ssm_scan_kernel, dim3((unsigned)(sb + (ch + 255) / 256)), dim3(256), 0, c.stream, pu, ldu, *a, (int)T, (int)pos0, b, sb);
-  // heads that share a block's C . B: as many as leave two blocks per CU
-  const int per = (int)(a->heads / a->groups), cus = c.cus > 0 ? c.cus : 256;
-  int HB = 1;
-  while (HB < 8 && HB < per && (int64_t)b.np * a->groups * ((per + 2 * HB - 1) / (2 * HB)) >= 2 * cus) HB *= 2;
   auto out = b.C == 64 ? ssm_out_kernel<64> : b.C == 32 ? ssm_out_kernel<32> : ssm_out_kernel<16>;
   e = hipFuncSetAttribute(reinterpret_cast<const void*>(out), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds2);
   if (e != hipSuccess) return hip_fail(e, "hipFuncSetAttribute(LDS)");
-  hipLaunchKernelGGL(out, dim3((unsigned)b.np, (unsigned)(a->groups * ((per + HB - 1) / HB))), dim3(256), lds2, c.stream, pu, ldu,
-                     static_cast<float*>(y), ldy, *a, (int)T, b, HB);
+  hipLaunchKernelGGL(out, dim3((unsigned)b.np, (unsigned)a->heads), dim3(512), lds2, c.stream, pu, ldu, static_cast<float*>(y), ldy,
+                     *a, (int)T, b);
   TLHIP_CHECK_LAUNCH(TLHIP_C_SSM);
 }
 

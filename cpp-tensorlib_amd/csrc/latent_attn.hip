@@ -259,7 +259,9 @@ __global__ __launch_bounds__(256) void latent_query_mfma_kernel(const float* __r
     put(d.L + half + j, (hi * cs.x + lo * cs.y) * sc);
     return;
   }
-  const int slice = blockIdx.x % slices, h = blockIdx.x / slices % d.H, t0 = blockIdx.x / slices / d.H * kQTok;
+  // a line of the image holds rows of adjacent heads: their blocks on one die, where its L2 joins the stores
+  const int id = work % 8 == 0 ? (int)(blockIdx.x % 8) * (work / 8) + (int)blockIdx.x / 8 : (int)blockIdx.x;
+  const int h = id % d.H, slice = id / d.H % slices, t0 = id / d.H / slices * kQTok;
   const int KST = (d.D + 15) / 16, ldk = up8(d.L);
   u32x4* frag = reinterpret_cast<u32x4*>(lds);
   for (int i = tid; i < 16 * 2 * KST; i += 256) {        // 8 latent dims x 8 query dims, transposed
@@ -613,8 +615,13 @@ __global__ __launch_bounds__(NT) void latent_out_kernel(const float* __restrict_
   const u32x4* uv = reinterpret_cast<const u32x4*>(static_cast<const uint16_t*>(a.uv)) + (size_t)h * d.V * n8;
   constexpr int PRE = kOutRows / NW < 2 ? 1 : 2;     // rows whose weights are requested up front
   u32x4 pre[PRE];
+  float gate[PRE];                     // (of a single token)
 #pragma unroll
-  for (int i = 0; i < PRE; i++) pre[i] = uv[(size_t)min(vw + i * NW, d.V - 1) * n8 + min(lane, n8 - 1)];
+  for (int i = 0; i < PRE; i++) {
+    const int v = min(vw + i * NW, d.V - 1);
+    pre[i] = uv[(size_t)v * n8 + min(lane, n8 - 1)];
+    gate[i] = TQ == 1 && a.gate_off >= 0 ? u[(size_t)t0 * ldu + a.gate_off + h * d.V + v] : 0.f;
+  }
   f32x4 v[8];                          // eight splits' latents of this thread's item, the first ones before the weights are known
   const auto load_splits = [&](int i, int s0) {
     const int j = i % items, t = j / (LV / 4), e = 4 * (j - t * (LV / 4));
@@ -683,7 +690,12 @@ __global__ __launch_bounds__(NT) void latent_out_kernel(const float* __restrict_
       const float s = wave_sum(acc[t]);
       if (lane == 0 && t < nt) {
         float o = s;
-        if (a.gate_off >= 0) o = s / (1.f + expf(-u[(size_t)(t0 + t) * ldu + a.gate_off + h * d.V + v]));
+        if (a.gate_off >= 0) {
+          float z;
+          if (TQ == 1 && i < PRE) z = i == 0 ? gate[0] : gate[PRE - 1];
+          else z = u[(size_t)(t0 + t) * ldu + a.gate_off + h * d.V + v];
+          o = s / (1.f + expf(-z));
+        }
         y[(size_t)(t0 + t) * ldy + a.y_off + h * d.V + v] = o;
       }
     }

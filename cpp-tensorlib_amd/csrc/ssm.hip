@@ -337,15 +337,13 @@ __global__ __launch_bounds__(512) __attribute__((amdgpu_waves_per_eu(4))) void s
     const int i = min(tid + 512 * k, C * v4 - 1), t = i / v4;
     xr[k] = *reinterpret_cast<const f32x4*>(row + (size_t)min(t, nt - 1) * b.xw + h * b.Vp + 4 * (i - t * v4));
   }
-  float sv[2][4][4];                   // state rows n0 .. n0 + 127 of an item's columns
+  float sv[4][4];                      // state rows n0 .. n0 + 63 of an item's columns
   const auto load_state = [&](int item, int n0) {
     const int v = 16 * (item % nvt) + l15;
 #pragma unroll
-    for (int q = 0; q < 2; q++)
+    for (int k = 0; k < 4; k++)
 #pragma unroll
-      for (int k = 0; k < 4; k++)
-#pragma unroll
-        for (int e = 0; e < 4; e++) sv[q][k][e] = st[(size_t)(min(n0 + 64 * q + 16 * k, b.Np - 16) + 4 * lg + e) * b.Vp + v];
+      for (int e = 0; e < 4; e++) sv[k][e] = st[(size_t)(min(n0 + 16 * k, b.Np - 16) + 4 * lg + e) * b.Vp + v];
   };
   load_state(min(wave, items - 1), 0);
   ssm_tile(Cm, BS, row + d.H * b.Vp + (d.G + g) * b.Np, b.xw, C, b.Np, nt, tid, 512);
@@ -410,21 +408,19 @@ __global__ __launch_bounds__(512) __attribute__((amdgpu_waves_per_eu(4))) void s
         z[r][k] = u[(size_t)(t0 + min(16 * blk[r] + 4 * lg + k, nt - 1)) * ldu + a.z_off + h * d.V + min(v0 + l15, d.V - 1)];
     }
     if (item != wave) load_state(item, 0);
-    for (int n0 = 0; n0 < b.Np; n0 += 128) {
+    for (int n0 = 0; n0 < b.Np; n0 += 64) {
       if (n0 > 0) load_state(item, n0);
 #pragma unroll
-      for (int q = 0; q < 2; q++)
+      for (int k = 0; k < 4; k++) {
+        const int n = n0 + 16 * k;
+        if (n >= b.Np) continue;
 #pragma unroll
-        for (int k = 0; k < 4; k++) {
-          const int n = n0 + 64 * q + 16 * k;
-          if (n >= b.Np) continue;
+        for (int r = 0; r < HALF; r++) {
+          const f32x4 cf = *reinterpret_cast<const f32x4*>(Cm + (16 * blk[r] + l15) * BS + n + 4 * lg);
 #pragma unroll
-          for (int r = 0; r < HALF; r++) {
-            const f32x4 cf = *reinterpret_cast<const f32x4*>(Cm + (16 * blk[r] + l15) * BS + n + 4 * lg);
-#pragma unroll
-            for (int e = 0; e < 4; e++) acc[r] = ssm_mfma(cf[e], sv[q][k][e], acc[r]);
-          }
+          for (int e = 0; e < 4; e++) acc[r] = ssm_mfma(cf[e], sv[k][e], acc[r]);
         }
+      }
     }
 #pragma unroll
     for (int r = 0; r < HALF; r++) {
